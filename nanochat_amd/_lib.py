@@ -1,4 +1,5 @@
-"""ctypes binding of libnanochat_amd.so (the C ABI of include/nanochat_amd.h).
+"""ctypes binding of libnanochat_amd.so (the C ABI of include/nanochat_amd.h) and of libnanochat_amd_stack.so
+(include/nanochat_amd_stack.h).
 
 There is no fallback: if the library is missing or a call fails, an exception is raised.
 """
@@ -20,6 +21,10 @@ EXPORTS = [
     "nc_fp8_quantize_state_bytes", "nc_fp8_quantize_tensorwise_fused", "nc_fp8_quantize_tensorwise_fused_bounded", "nc_probe_fp8_mfma_ceiling", "nc_probe_hbm_read", "nc_fp8_quantize_tensorwise_transposed",
     "nc_decode_attention_shared", "nc_decode_attention_shared_workspace_bytes",
 ]
+
+
+STACK_EXPORTS = ["nc_stack_abi_version", "nc_last_error", "nc_stack_workspace_bytes", "nc_stack_forward", "nc_stack_linear", "nc_stack_cache_copy",
+                 "nc_profile_enable", "nc_profile_read", "nc_profile_read_gemm"]
 
 
 class LayerDesc(C.Structure):
@@ -44,7 +49,52 @@ class CacheDesc(C.Structure):
                 ("shared_prefix", C.c_int), ("uniform_pos", C.c_int), ("advance", C.c_int)]
 
 
+class StackLayer(C.Structure):
+    _fields_ = ([(n, C.c_int) for n in ("mixer", "ff", "heads", "dim", "dim_p", "vdim", "vdim_p", "rot_dim", "rot_p", "rank", "rank_p", "rot_dims")]
+                + [("score_scale", C.c_float)]
+                + [(n, C.c_int) for n in ("mix_cols", "router_cols", "ff_cols", "n_in", "mix_out", "ff_p", "k_out")]
+                + [("ff_limit", C.c_float), ("experts", C.c_int), ("top", C.c_int), ("expert_ff_p", C.c_int), ("expert_limit", C.c_float)]
+                + [(n, C.c_void_p) for n in ("norm_w", "w_in", "w_out", "kv_norm_w", "w_uk_t", "w_ukv", "decay", "rope", "w_e1", "w_e2")])
+
+
+class StackRun(C.Structure):
+    _fields_ = [("layer", C.c_int), ("slot", C.c_int), ("add_embedding", C.c_int), ("step", C.c_int)]
+
+
+class StackModel(C.Structure):
+    _fields_ = ([(n, C.c_int) for n in ("dtype", "width", "width_p", "vocab", "rope_len", "n_layers", "n_runs", "max_k_out")]
+                + [(n, C.c_float) for n in ("eps", "embed_scale", "logit_scale", "logit_softcap")]
+                + [(n, C.c_void_p) for n in ("embed", "head", "final_norm_w", "steps")]
+                + [("layers", C.POINTER(StackLayer)), ("runs", C.POINTER(StackRun))])
+
+
+class StackCacheDesc(C.Structure):
+    _fields_ = [("latents", C.POINTER(C.c_void_p)), ("state_in", C.POINTER(C.c_void_p)), ("state_out", C.POINTER(C.c_void_p)),
+                ("cache_seqlens", C.c_void_p), ("batch", C.c_int), ("max_seq_len", C.c_int), ("pos_max", C.c_int), ("advance", C.c_int)]
+
+
 _lib = None
+_stack_lib = None
+
+
+def _bind_stack(lib):
+    p, i, i64, f, sz = C.c_void_p, C.c_int, C.c_int64, C.c_float, C.c_size_t
+    sig = {
+        "nc_stack_abi_version": (i, []),
+        "nc_last_error": (C.c_char_p, []),
+        "nc_stack_workspace_bytes": (sz, [C.POINTER(StackModel), i, i, i, i]),
+        "nc_stack_forward": (i, [C.POINTER(StackModel), C.POINTER(StackCacheDesc), p, i, i, p, i, p, p, sz, p, p]),
+        "nc_stack_linear": (i, [i, p, i64, p, p, i, i, i, i, i, f, i, p]),
+        "nc_stack_cache_copy": (i, [p, p, i, i, i64, i64, i64, p]),
+        "nc_profile_enable": (i, [i]),
+        "nc_profile_read": (i, [i, C.POINTER(C.c_double), C.POINTER(C.c_double), C.POINTER(i64)]),
+        "nc_profile_read_gemm": (i, [i, i, C.POINTER(C.c_double), C.POINTER(C.c_double), C.POINTER(i64)]),
+    }
+    for name, (res, args) in sig.items():
+        fn = getattr(lib, name)
+        fn.restype = res
+        fn.argtypes = args
+    return lib
 
 
 def _bind(lib):
@@ -99,31 +149,45 @@ def _bind(lib):
     return lib
 
 
+def _load(target):
+    from . import build as _build
+    path = _build.lib_path(target)
+    if not os.path.exists(path):
+        raise RuntimeError(f"{path} is missing: build it with `python -m nanochat_amd.build {target}` "
+                           "(there is no non-HIP fallback)")
+    # a rebuild that failed leaves the previous library in place: refuse one whose build stamp names other sources
+    stamp = _build.stamp_path(target)
+    if os.path.exists(stamp) and open(stamp).read().strip() != _build.sources_digest(target):
+        raise RuntimeError(f"{path} was built from other sources than this tree holds: rebuild it with "
+                           f"`python -m nanochat_amd.build {target}`")
+    return C.CDLL(path)
+
+
 def lib():
     """The loaded library.  Raises RuntimeError when it has not been built."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
-            raise RuntimeError(f"{LIB_PATH} is missing: build it with `python -m nanochat_amd.build` "
-                               "(there is no non-HIP fallback)")
-        # a rebuild that failed leaves the previous library in place: refuse one whose build stamp names other sources
-        from . import build as _build
-        if os.path.exists(_build.STAMP_PATH) and open(_build.STAMP_PATH).read().strip() != _build.sources_digest():
-            raise RuntimeError(f"{LIB_PATH} was built from other sources than this tree holds: rebuild it with "
-                               "`python -m nanochat_amd.build`")
-        _lib = _bind(C.CDLL(LIB_PATH))
+        _lib = _bind(_load("gpt"))
     return _lib
+
+
+def stack_lib():
+    """The loaded layer-stack library.  Raises RuntimeError when it has not been built."""
+    global _stack_lib
+    if _stack_lib is None:
+        _stack_lib = _bind_stack(_load("stack"))
+    return _stack_lib
 
 
 class NcError(RuntimeError):
     pass
 
 
-def check(rc):
+def check(rc, library=None):
     """Turn a negative return code into an exception: -1 (bad argument) -> ValueError, else NcError."""
     if rc == 0:
         return
-    msg = lib().nc_last_error().decode("utf-8", "replace")
+    msg = (library or lib()).nc_last_error().decode("utf-8", "replace")
     if rc == -1:
         raise ValueError(msg)
     raise NcError(f"[{rc}] {msg}")

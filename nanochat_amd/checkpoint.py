@@ -5,6 +5,8 @@ Layout written by the reference's save_checkpoint: `model_%06d.pt` (the state di
 `backout_lambda`, `value_embeds.{i}.weight`, `lm_head.weight`) and `meta_%06d.json` with a `model_config` dict.
 Only tensors are read from the .pt file (`weights_only=True`: nothing in it is executed).  The tokenizer and
 the optimizer shards are not part of this path.
+
+Also the readers of folders with a config.json and a model.safetensors (registry.py chooses the model class).
 """
 import glob
 import json
@@ -13,8 +15,37 @@ import re
 
 import torch
 
-from .fp8 import convert_to_float8_training, fp8_module_filter
-from .gpt import GPT, GPTConfig
+
+def read_config(model_dir):
+    with open(os.path.join(model_dir, "config.json"), "r", encoding="utf-8") as f:
+        return json.load(f)
+
+
+_SAFETENSORS_DTYPES = {"BF16": torch.bfloat16, "F16": torch.float16, "F32": torch.float32, "F64": torch.float64, "I64": torch.int64, "I32": torch.int32,
+                       "I16": torch.int16, "I8": torch.int8, "U8": torch.uint8, "BOOL": torch.bool}
+
+
+def read_safetensors(model_dir, name="model.safetensors"):
+    """{tensor name: CPU tensor}: an 8-byte little-endian header length, a JSON header (name -> dtype, shape, data_offsets), the data."""
+    path = os.path.join(model_dir, name)
+    with open(path, "rb") as f:
+        header = json.loads(f.read(int.from_bytes(f.read(8), "little")))
+        start, size = f.tell(), os.path.getsize(path)
+        out = {}
+        for key, t in header.items():
+            if key == "__metadata__":
+                continue
+            lo, hi = t["data_offsets"]
+            dtype = _SAFETENSORS_DTYPES[t["dtype"]]
+            numel = 1
+            for n in t["shape"]:
+                numel *= n
+            if not (0 <= lo <= hi and start + hi <= size and hi - lo == numel * dtype.itemsize):
+                raise RuntimeError(f"{path}: {key} does not fit the file")
+            f.seek(start + lo)
+            data = bytearray(f.read(hi - lo))
+            out[key] = (torch.frombuffer(data, dtype=dtype) if numel else torch.empty(0, dtype=dtype)).view(t["shape"])
+    return out
 
 
 def find_last_step(checkpoint_dir):
@@ -43,6 +74,8 @@ def build_model(checkpoint_dir, step=None, device="cuda"):
     The reference evaluates a checkpoint with plain Linear modules (bf16 matmuls, checkpoint_manager.py:99-104); the path built
     here is the quantized one only, so a loaded model always runs its block linears and lm_head as e4m3 Float8Linear -- the
     numerics of the reference's --fp8 training forward, not of its bf16 evaluation."""
+    from .fp8 import convert_to_float8_training, fp8_module_filter
+    from .gpt import GPT, GPTConfig
     if step is None:
         step = find_last_step(checkpoint_dir)
     device = torch.device(device)

@@ -1,25 +1,13 @@
-// extern "C" surface of libnanochat_amd.so: argument validation, the thread-local error message and
-// thin forwarding into the launch functions.  Declarations and reference citations: include/nanochat_amd.h.
-#include <stdarg.h>
+// extern "C" surface of libnanochat_amd.so: argument validation and thin forwarding into the launch functions.  Declarations and reference citations: include/nanochat_amd.h.
 #include <stdio.h>
 #include "../../include/nanochat_amd.h"
 #include "nc_common.h"
 #include "nc_kernels.h"
 #include "nc_rope.h"
 
-static thread_local char g_error[512] = "";
-
-void nc_set_error(const char* fmt, ...) {
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(g_error, sizeof(g_error), fmt, ap);
-    va_end(ap);
-}
-
 extern "C" {
 
 int nc_abi_version(void) { return 2; }
-const char* nc_last_error(void) { return g_error; }
 
 int nc_fp8_quantize_tensorwise(const void* x, int x_dtype, int64_t n, uint8_t* out, float* scale_out, float* inv_scale_out,
                                uint32_t* amax_ws, int encoder, nc_stream_t stream) {

@@ -481,8 +481,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bl_kernel(const uint8_t* 
 }
 
 
-// Per-process caches of what never changes while the process lives: the number of CUs of a device, and which kernels have had their
-// dynamic LDS limit raised on which device (hipFuncSetAttribute costs microseconds per call, a launch-bound caller notices).
+// Per-process cache of what never changes while the process lives: which kernels have had their dynamic LDS limit raised on which device (hipFuncSetAttribute costs microseconds per call, a launch-bound caller notices).
 #include <atomic>
 namespace {
 constexpr int NC_GEMM_MAX_DEVICES = 64;
@@ -490,17 +489,7 @@ int current_device() {
     int dev = 0;
     return hipGetDevice(&dev) == hipSuccess && dev >= 0 && dev < NC_GEMM_MAX_DEVICES ? dev : 0;
 }
-int cu_count() {
-    static std::atomic<int> cached[NC_GEMM_MAX_DEVICES];
-    const int dev = current_device();
-    int cus = cached[dev].load(std::memory_order_relaxed);
-    if (cus == 0) {
-        cus = 256;
-        (void)hipDeviceGetAttribute(&cus, hipDeviceAttributeMultiprocessorCount, dev);
-        cached[dev].store(cus, std::memory_order_relaxed);
-    }
-    return cus;
-}
+int cu_count() { return nc_cu_count(); }
 // slot: one per kernel family that asks for dynamic LDS (the attribute is set for the instantiation actually launched, so the
 // cache is keyed by the function pointer as well)
 hipError_t reserve_lds(const void* fn, int bytes) {
@@ -525,8 +514,6 @@ hipError_t reserve_lds(const void* fn, int bytes) {
     return hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, bytes);      // table full: just set it
 }
 }  // namespace
-
-int nc_cu_count() { return cu_count(); }
 
 template <int BM, int BN, int WGM, int WGN, bool INTERLEAVE, int A_FMT, int OUT_KIND>
 static int launch_bl_as(const uint8_t* a, const uint8_t* b, const EpilogueArgs& ep, int M, int N, int K, hipStream_t s) {

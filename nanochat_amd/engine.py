@@ -65,12 +65,41 @@ def use_calculator(expr):
 
 
 # ------------------------------------------------------------------------------------------------
-class KVCache:
+class SequenceCache:
+    """Positions of the rows of a cache: per-row lengths in an int32 device tensor, with a host-side copy so that get_pos() does not
+    have to read the device tensor back every decode step.  What the rows hold is the subclass's: keys and values (KVCache), or
+    latents and recurrent states (StackCache).  The Engine uses: get_pos, advance / note_advanced (by the model), mark and rewind."""
+
+    def __init__(self, batch_size, seq_len, device):
+        self.batch_size = batch_size
+        self.max_seq_len = seq_len
+        self.cache_seqlens = torch.zeros(batch_size, dtype=torch.int32, device=device)
+        self._pos0 = 0          # host mirror of cache_seqlens[0]
+        self._pos_max = 0       # host mirror of cache_seqlens.max()
+
+    def get_pos(self):
+        return self._pos0
+
+    def advance(self, num_tokens):
+        self.cache_seqlens += num_tokens
+        self.note_advanced(num_tokens)
+
+    def note_advanced(self, num_tokens):
+        """The forward call advanced `cache_seqlens` on the device itself (the `advance` field of its cache descriptor): only the host
+        side follows."""
+        self._pos0 += num_tokens
+        self._pos_max += num_tokens
+
+    def mark(self):
+        """What rewind() needs to take back the forward that follows."""
+        return None
+
+
+class KVCache(SequenceCache):
     """Pre-allocated (n_layers, B, T, H, D) key and value tensors in FA3 layout, per-row lengths in an
     int32 tensor, and the previous token's normalised embedding for the smear gate (engine.py:82-137).
 
-    A host-side copy of the position is kept so that get_pos() does not have to read the device tensor
-    back every decode step; it is exact as long as positions change only through advance/reset/prefill
+    The host-side copy of the position is exact as long as positions change only through advance/reset/prefill
     (or set_seqlens for ragged batches, where it tracks row 0 like the reference's get_pos)."""
 
     def __init__(self, batch_size, num_heads, seq_len, head_dim, num_layers, device, dtype, prefill_from=None, share_prompt_reads=False):
@@ -84,8 +113,7 @@ class KVCache:
         forward reads it once for all rows in the layers that see most of it, instead of once per row; the tensors keep the reference's
         layout and contents.  The promise that goes with it: nobody writes into positions [0, shared_prefix_len) of k_cache / v_cache
         by hand (set shared_prefix_len = 0 first)."""
-        self.batch_size = batch_size
-        self.max_seq_len = seq_len
+        super().__init__(batch_size, seq_len, device)
         self.n_layers = num_layers
         self.n_heads = num_heads
         self.head_dim = head_dim
@@ -94,10 +122,7 @@ class KVCache:
         alloc = torch.empty if lazy else torch.zeros
         self.k_cache = alloc(shape, device=device, dtype=dtype)
         self.v_cache = alloc(shape, device=device, dtype=dtype)
-        self.cache_seqlens = torch.zeros(batch_size, dtype=torch.int32, device=device)
         self.prev_embedding = None
-        self._pos0 = 0          # host mirror of cache_seqlens[0]
-        self._pos_max = 0       # host mirror of cache_seqlens.max()
         self.share_prompt_reads = bool(share_prompt_reads)
         self.shared_prefix_len = 0      # positions [0, this) hold the same bytes in every row (set by prefill from a batch-1 cache)
         if prefill_from is not None:
@@ -114,21 +139,11 @@ class KVCache:
         self._pos0 = self._pos_max = 0
         self.shared_prefix_len = 0
 
-    def get_pos(self):
-        return self._pos0
-
     def get_layer_cache(self, layer_idx):
         return self.k_cache[layer_idx], self.v_cache[layer_idx]
 
-    def advance(self, num_tokens):
-        self.cache_seqlens += num_tokens
-        self._pos0 += num_tokens
-        self._pos_max += num_tokens
-
-    def note_advanced(self, num_tokens):
-        """The forward call advanced `cache_seqlens` on the device itself (nc_cache_desc.advance): only the host mirrors follow."""
-        self._pos0 += num_tokens
-        self._pos_max += num_tokens
+    def mark(self):
+        return self.prev_embedding
 
     def rewind(self, num_tokens, prev_embedding):
         """Take back the last advance (the appended rows stay in the tensors and are overwritten by the next
@@ -168,6 +183,84 @@ class KVCache:
         self.shared_prefix_len = n if (other.batch_size == 1 and self.batch_size > 1) else 0
         if other.prev_embedding is not None:
             self.prev_embedding = other.prev_embedding.expand(self.batch_size, -1, -1).clone()
+
+
+class StackCache(SequenceCache):
+    """Cache of a layer stack (nanochat_amd/stack.py): for every run of a latent-attention layer the latents of all tokens, for every
+    run of a recurrent layer one fp32 state per row.  A layer that runs several times has a slot for each of its runs.
+
+    `latents[slot]` [B, seq_len, latent width]; `states[i][slot]` [B, heads, dim, vdim], two buffers: a forward reads one and writes the
+    other, so a forward can be taken back.  A row at position 0 does not read its state: a slot of the batch is given back by
+    setting its position to zero."""
+
+    def __init__(self, latent_widths, state_shapes, dtype, batch_size, seq_len, device, prefill_from=None):
+        super().__init__(batch_size, seq_len, device)
+        self.dtype = dtype
+        # (zeros: the positions past a row's end enter products with weight zero, and must be finite there)
+        self.latents = [torch.zeros(batch_size, seq_len, w, device=device, dtype=dtype) for w in latent_widths]
+        self.states = [[torch.zeros(batch_size, *s, device=device, dtype=torch.float32) for s in state_shapes] for _ in range(2)]
+        self._current = 0                          # which of the two state buffers holds the states
+        self._host_pos = [0] * batch_size
+        self._last_tokens = 0                      # tokens of the last forward, which is the one rewind() can take back
+        if prefill_from is not None:
+            self.prefill(prefill_from)
+
+    def _positions_changed(self):
+        self._pos0, self._pos_max = self._host_pos[0], max(self._host_pos)
+        self._last_tokens = 0
+
+    def reset(self):
+        self.reset_rows(range(self.batch_size))
+
+    def reset_rows(self, rows):
+        """Give rows of the batch back: their next token is the first of a new sequence."""
+        for r in rows:
+            self.cache_seqlens[r] = 0
+            self._host_pos[r] = 0
+        self._positions_changed()
+
+    def state_buffers(self):
+        """(states to read, states to write) of the next forward."""
+        return self.states[self._current], self.states[self._current ^ 1]
+
+    def note_advanced(self, num_tokens):
+        super().note_advanced(num_tokens)
+        self._host_pos = [p + num_tokens for p in self._host_pos]
+        self._current ^= 1
+        self._last_tokens = num_tokens
+
+    def rewind(self, num_tokens, mark=None):
+        """Take back the last forward, which brought `num_tokens` tokens (their latents are overwritten by the next ones)."""
+        assert 0 < num_tokens == self._last_tokens, "only the last forward can be taken back"
+        self.cache_seqlens -= num_tokens
+        self._host_pos = [p - num_tokens for p in self._host_pos]
+        self._positions_changed()
+        self._current ^= 1
+
+    def load_row(self, row, other, other_row=0):
+        """Copy one sequence out of another cache of the same model into row `row` of this one."""
+        self._copy(other, other_row, 1, row, 1)
+        self.cache_seqlens[row] = other._host_pos[other_row]
+        self._host_pos[row] = other._host_pos[other_row]
+        self._positions_changed()
+
+    def prefill(self, other):
+        """Copy another cache's tokens and states into every row of this one (row by row, or its one row into all)."""
+        assert self._pos_max == 0, "Cannot prefill a non-empty cache"
+        assert other.batch_size in (1, self.batch_size)
+        self._copy(other, 0, other.batch_size, 0, self.batch_size)
+        self._host_pos = list(other._host_pos) if other.batch_size == self.batch_size else other._host_pos * self.batch_size
+        self.cache_seqlens.copy_(torch.tensor(self._host_pos, dtype=torch.int32))
+        self._positions_changed()
+
+    def _copy(self, other, src_row, src_rows, dst_row, dst_rows):
+        n = other._pos_max
+        assert n <= self.max_seq_len and self.dtype == other.dtype
+        assert [t.shape[2] for t in self.latents] == [t.shape[2] for t in other.latents]
+        for src, dst in zip(other.latents, self.latents):
+            ops.stack_cache_copy(src[src_row:src_row + src_rows], dst[dst_row:dst_row + dst_rows], n)
+        for src, dst in zip(other.state_buffers()[0], self.state_buffers()[0]):
+            ops.stack_cache_copy(src[src_row:src_row + src_rows], dst[dst_row:dst_row + dst_rows], src.shape[1])
 
 
 # ------------------------------------------------------------------------------------------------
@@ -246,6 +339,16 @@ class Engine:
             state.python_expr_tokens.append(token)
         return token, (0 if forced else 1)
 
+    def _new_cache(self, batch_size, seq_len, prefill_from=None, share_prompt_reads=False):
+        """A cache of the model's own kind (model.new_cache), or the KV cache that its configuration describes."""
+        make = getattr(self.model, "new_cache", None)
+        if make is not None:
+            return make(batch_size, seq_len, prefill_from=prefill_from, share_prompt_reads=share_prompt_reads)
+        cfg, device = self.model.config, self.model.get_device()
+        dtype = torch.bfloat16 if torch.device(device).type == "cuda" else COMPUTE_DTYPE
+        return KVCache(batch_size=batch_size, num_heads=cfg.n_kv_head, seq_len=seq_len, head_dim=cfg.n_embd // cfg.n_head, num_layers=cfg.n_layer,
+                       device=device, dtype=dtype, prefill_from=prefill_from, share_prompt_reads=share_prompt_reads)
+
     def _last_logits(self, ids, kv_cache):
         fast = getattr(self.model, "forward_last", None)
         if fast is not None:
@@ -253,28 +356,30 @@ class Engine:
         return self.model.forward(ids, kv_cache=kv_cache)[:, -1, :]
 
     @torch.inference_mode()
-    def generate(self, tokens, num_samples=1, max_tokens=None, temperature=1.0, top_k=None, seed=42, share_prompt_reads=False):
+    def generate(self, tokens, num_samples=1, max_tokens=None, temperature=1.0, top_k=None, seed=42, share_prompt_reads=False, prefill_chunk=None):
         """One batch-1 prefill, cache replicated to num_samples rows, then streamed decoding.
         Yields (token_column, token_masks) per step (engine.py:175-275).
 
         share_prompt_reads (not in the reference's signature, off by default): every row's cache starts with a copy of the same
-        prompt; with this set, the decode steps read that prompt once for all rows in the full-context layers (see KVCache)."""
+        prompt; with this set, the decode steps read that prompt once for all rows in the full-context layers (see KVCache).
+
+        prefill_chunk (not in the reference's signature): the prompt goes through the model in portions of at most this many tokens
+        (bounds the workspace of a long prompt); None: in one piece."""
         assert isinstance(tokens, list) and isinstance(tokens[0], int), "expecting list of ints"
         device = self.model.get_device()
-        dtype = torch.bfloat16 if torch.device(device).type == "cuda" else COMPUTE_DTYPE
         rng = torch.Generator(device=device)
         rng.manual_seed(seed)
         sp = _Specials(self.tokenizer)
 
-        cfg = self.model.config
-        geometry = dict(num_heads=cfg.n_kv_head, head_dim=cfg.n_embd // cfg.n_head, num_layers=cfg.n_layer)
-        kv_prefill = KVCache(batch_size=1, seq_len=len(tokens), device=device, dtype=dtype, **geometry)
-        ids = torch.tensor([tokens], dtype=torch.long, device=device)
-        logits = self._last_logits(ids, kv_prefill).expand(num_samples, -1)
+        kv_prefill = self._new_cache(1, len(tokens))
+        portion = len(tokens) if prefill_chunk is None else max(1, prefill_chunk)
+        for start in range(0, len(tokens), portion):
+            ids = torch.tensor([tokens[start:start + portion]], dtype=torch.long, device=device)
+            logits = self._last_logits(ids, kv_prefill)
+        logits = logits.expand(num_samples, -1)
 
-        hint = (len(tokens) + max_tokens) if max_tokens is not None else cfg.sequence_len
-        kv_decode = KVCache(batch_size=num_samples, seq_len=hint, device=device, dtype=dtype, prefill_from=kv_prefill,
-                            share_prompt_reads=share_prompt_reads, **geometry)
+        hint = (len(tokens) + max_tokens) if max_tokens is not None else max(self.model.config.sequence_len, len(tokens) + 1)
+        kv_decode = self._new_cache(num_samples, hint, prefill_from=kv_prefill, share_prompt_reads=share_prompt_reads)
         del kv_prefill
 
         rows = [RowState(tokens.copy()) for _ in range(num_samples)]
@@ -301,7 +406,7 @@ class Engine:
                 # active every one of the step's ~190 launches starts ~0.5 us later)
                 host_ids.copy_(sampled_dev[:, 0], non_blocking=True)
                 ids_ready.record()
-                prev_before = kv_decode.prev_embedding
+                before = kv_decode.mark()
                 logits_ahead = self._last_logits(sampled_dev, kv_decode)
                 ids_ready.synchronize()
                 sampled = host_ids.tolist()
@@ -318,7 +423,7 @@ class Engine:
                 logits = logits_ahead
                 continue
             if run_ahead:
-                kv_decode.rewind(1, prev_before)
+                kv_decode.rewind(1, before)
             # forced tokens come from the tokenizer, not from the sampler: refuse what the embedding table does not hold
             rows_in_table = getattr(self.model, "padded_vocab_size", None)
             if rows_in_table is not None and not all(0 <= t < rows_in_table for t in column):

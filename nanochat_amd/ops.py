@@ -475,3 +475,30 @@ def sample(logits, temperature, top_k, noise=None):
     rc = _lib.lib().nc_sample(_ptr(logits), B, V, logits.stride(0), float(temperature), k, _ptr(noise), _ptr(out), _stream())
     _lib.check(rc)
     return out
+
+
+# ----------------------------------------------------------------------------- layer stack
+STACK_DTYPES = {torch.bfloat16: 0, torch.float32: 1}
+STACK_PAD = 64
+
+
+def stack_cache_copy(src, dst, n):
+    """The first n entries (second axis) of every row of src into every row of dst; one row of src goes into all rows."""
+    _need_cuda(src, dst)
+    assert src.shape[2:] == dst.shape[2:] and src.dtype == dst.dtype and src[0].is_contiguous() and dst[0].is_contiguous()
+    es = src.element_size()
+    n_bytes = n * (src[0].numel() // src.shape[1]) * es
+    rc = _lib.stack_lib().nc_stack_cache_copy(_ptr(src), _ptr(dst), src.shape[0], dst.shape[0], src.stride(0) * es, dst.stride(0) * es, n_bytes, _stream())
+    _lib.check(rc, _lib.stack_lib())
+
+
+def stack_linear(a, w, kind=0, limit=0.0, kernel=0):
+    """a [M, K] w [N, K]^T in the storage type of both, 32-bit sums (nc_stack_linear).  kind: 0 plain, 1 tanh-form gelu, 2 clamped GLU of
+    interleaved (gate, up) rows of w, 3 float output; kernel: 0 choose, 1 the few-rows kernel, 2 the tiled one."""
+    _need_cuda(a, w)
+    (M, K), N = a.shape, w.shape[0]
+    assert w.shape[1] == K and a.dtype == w.dtype and a.is_contiguous() and w.is_contiguous()
+    out = torch.empty(M, N // 2 if kind == 2 else N, dtype=torch.float32 if kind == 3 else a.dtype, device=a.device)
+    rc = _lib.stack_lib().nc_stack_linear(STACK_DTYPES[a.dtype], _ptr(a), K, _ptr(w), _ptr(out), out.shape[1], M, N, K, kind, limit, kernel, _stream())
+    _lib.check(rc, _lib.stack_lib())
+    return out

@@ -82,11 +82,14 @@ class SequenceCache:
 
     def advance(self, num_tokens):
         self.cache_seqlens += num_tokens
-        self.note_advanced(num_tokens)
+        self._moved(num_tokens)
 
     def note_advanced(self, num_tokens):
         """The forward call advanced `cache_seqlens` on the device itself (the `advance` field of its cache descriptor): only the host
         side follows."""
+        self._moved(num_tokens)
+
+    def _moved(self, num_tokens):
         self._pos0 += num_tokens
         self._pos_max += num_tokens
 
@@ -223,8 +226,8 @@ class StackCache(SequenceCache):
         """(states to read, states to write) of the next forward."""
         return self.states[self._current], self.states[self._current ^ 1]
 
-    def note_advanced(self, num_tokens):
-        super().note_advanced(num_tokens)
+    def _moved(self, num_tokens):
+        super()._moved(num_tokens)
         self._host_pos = [p + num_tokens for p in self._host_pos]
         self._current ^= 1
         self._last_tokens = num_tokens

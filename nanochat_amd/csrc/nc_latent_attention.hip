@@ -182,13 +182,20 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(NcLatentGeom g, const 
         const bf16_t* src = q_lat + ((int64_t)b * rows + min(r0 + qr, rows - 1)) * rw;
         for (int c = qp; c < rw / 8; c += 16) *(uint4*)(lds_q + qr * pitch + c * 16) = *(const uint4*)(src + c * 8);
     }
-    const int skey = tid >> 2, spart = tid & 3;
+    // 64 cached rows are one contiguous run of memory, 256 pieces of 16 bytes at a time; `put` is where this thread's pieces go in LDS
     uint4 rk[PC];
+    int put[PC];
+#pragma unroll
+    for (int i = 0; i < PC; i++) {
+        const int idx = tid + 256 * i;
+        put[i] = idx / (4 * pieces) * pitch + idx % (4 * pieces) * 16;
+    }
     auto fetch = [&](int kb) {
-        const bf16_t* src = keys + (int64_t)min(kb + skey, k_end - 1) * rw + spart * 8;
+        const bf16_t* src = keys + (int64_t)kb * rw;
+        const int last = (k_end - kb) * 4 * pieces - 1;          // pieces past the last key re-read its last one (weight zero)
 #pragma unroll
         for (int i = 0; i < PC; i++)
-            if (i < pieces) rk[i] = nt_load16(src + i * 32);
+            if (i < pieces) rk[i] = nt_load16(src + min(tid + 256 * i, last) * 8);
     };
     v4f acc[NT];
 #pragma unroll
@@ -202,7 +209,7 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(NcLatentGeom g, const 
         __syncthreads();                    // everyone is done with the previous keys
 #pragma unroll
         for (int i = 0; i < PC; i++)
-            if (i < pieces) *(uint4*)(lds + skey * pitch + (spart + 4 * i) * 16) = rk[i];
+            if (i < pieces) *(uint4*)(lds + put[i]) = rk[i];
         __syncthreads();
         if (kb + KEYS < k_end) fetch(kb + KEYS);
         v4f s0 = v4f{0.f, 0.f, 0.f, 0.f}, s1 = s0;
@@ -273,21 +280,31 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(NcLatentGeom g, const 
     }
 }
 
+constexpr int MAX_SPLITS = 64;
 __global__ __launch_bounds__(128) void latent_combine_kernel(const float* __restrict__ partials, int splits, int rank_p, bf16_t* __restrict__ out) {
+    __shared__ float weight[MAX_SPLITS];
     const int64_t row = blockIdx.x;
-    const float* part = partials + row * splits * (rank_p + 4);
-    float mx = LA_M_FLOOR;
-    for (int s = 0; s < splits; s++) mx = fmaxf(mx, part[(int64_t)s * (rank_p + 4)]);
-    float l = 0.f;
-    for (int s = 0; s < splits; s++) l += part[(int64_t)s * (rank_p + 4) + 1] * __builtin_amdgcn_exp2f(part[(int64_t)s * (rank_p + 4)] - mx);
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const int stride = rank_p + 4;
+    const float* part = partials + row * splits * stride;
+    if (threadIdx.x < 64) {                     // lane = split
+        const bool in = (int)threadIdx.x < splits;
+        const float m = in ? part[(int64_t)threadIdx.x * stride] : LA_M_FLOOR, l = in ? part[(int64_t)threadIdx.x * stride + 1] : 0.f;
+        const float w = __builtin_amdgcn_exp2f(m - wave_max(m));
+        const float total = wave_sum(l * w);
+        weight[threadIdx.x] = total > 0.f ? w / total : 0.f;
+    }
+    __syncthreads();
     for (int c = 4 * threadIdx.x; c < rank_p; c += 512) {
         v4f a = v4f{0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < splits; s++) {
-            const float* q = part + (int64_t)s * (rank_p + 4);
-            a += *(const v4f*)(q + 4 + c) * __builtin_amdgcn_exp2f(q[0] - mx);
+        for (int s0 = 0; s0 < splits; s0 += 8) {
+            v4f p[8];
+#pragma unroll
+            for (int s = 0; s < 8; s++) p[s] = *(const v4f*)(part + (int64_t)min(s0 + s, splits - 1) * stride + 4 + c);
+#pragma unroll
+            for (int s = 0; s < 8; s++)
+                if (s0 + s < splits) a += p[s] * weight[s0 + s];
         }
-        st4_f32(out + row * rank_p + c, a * inv);
+        st4_f32(out + row * rank_p + c, a);
     }
 }
 
@@ -487,9 +504,10 @@ int mfma_variant(int dtype, const NcLatentGeom& g) {
 }
 int mfma_splits(const NcLatentGeom& g) {
     const int groups = (g.T * g.heads + 15) / 16, blocks = (g.pos_max + g.T + KEYS - 1) / KEYS;
-    int splits = (512 + g.B * groups - 1) / (g.B * groups);
+    // one workgroup per compute unit (their LDS holds one): all of them start and end together
+    int splits = nc_cu_count() / (g.B * groups);
     if (splits > blocks) splits = blocks;
-    return splits < 1 ? 1 : splits > 64 ? 64 : splits;
+    return splits < 1 ? 1 : splits > MAX_SPLITS ? MAX_SPLITS : splits;
 }
 int reserve_lds(const void* fn, int bytes) {
     if (bytes > 64 * 1024 && hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess)
@@ -507,7 +525,7 @@ int launch_mfma(const NcLatentGeom& g, const bf16_t* q, const bf16_t* cache, con
 template <int DN, int DR, int DV>
 int launch_expanded(const NcLatentGeom& g, const bf16_t* q, int ldq, const bf16_t* kv, int keys, const bf16_t* cache, const int32_t* seqlens, bf16_t* out,
                     int ldo, hipStream_t s) {
-    if ((int64_t)((g.T + 127) / 128) * g.heads * g.B >= 512)
+    if ((int64_t)((g.T + 127) / 128) * g.heads * g.B >= 200)
         hipLaunchKernelGGL((latent_expanded_kernel<DN, DR, DV, 4>), dim3((g.T + 127) / 128, g.heads, g.B), dim3(256), 0, s, g, q, ldq, kv, keys, cache,
                            seqlens, out, ldo);
     else
@@ -522,7 +540,7 @@ int nc_launch_latent_append(int dtype, const NcLatentGeom& g, void* proj, int ld
                             const int32_t* seqlens, void* cache, void* q_lat, hipStream_t s) {
     NC_CHECK_ARG(g.rot_dims % 2 == 0 && g.rot_dims <= g.rot_p && g.rank <= g.rank_p, "latent_append: rot_dims=%d rot_p=%d", g.rot_dims, g.rot_p);
     NC_CHECK_ARG(g.pos_max + g.T <= rope_len, "latent_append: position %d past the rotary table of %d", g.pos_max + g.T, rope_len);
-    NcStackProf prof(NC_CLS_ROWS, (double)g.B * g.T * (g.rank_p + g.rot_p * (2.0 + g.heads)) * (dtype ? 8 : 4), s);
+    NcProfScope prof(NC_CLS_ROWS, (double)g.B * g.T * (g.rank_p + g.rot_p * (2.0 + g.heads)) * (dtype ? 8 : 4), s);
     if (dtype)
         hipLaunchKernelGGL((latent_append_kernel<float>), dim3(g.B * g.T), dim3(128), 0, s, g, (float*)proj, ldp, norm_w, eps, rope, rope_len, seqlens,
                            (float*)cache, (float*)q_lat);
@@ -544,7 +562,7 @@ int nc_launch_latent_attention(int dtype, const NcLatentGeom& g, const void* q_l
                                void* partials, size_t partial_bytes, hipStream_t s) {
     const int rows = g.B * g.T * g.heads;
     // the cached rows are read once per batch row (bytes); what a key costs beyond that stays on the chip
-    NcStackProf prof(NC_CLS_LATENT, (double)g.B * (g.pos_max + g.T) * (g.rank_p + g.rot_p) * (dtype ? 4 : 2), s, g.T);
+    NcProfScope prof(NC_CLS_LATENT, (double)g.B * (g.pos_max + g.T) * (g.rank_p + g.rot_p) * (dtype ? 4 : 2), s, g.T);
     const int variant = mfma_variant(dtype, g);
     if (variant) {
         const int splits = mfma_splits(g);
@@ -581,7 +599,7 @@ int nc_launch_latent_expanded(const NcLatentGeom& g, const bf16_t* q, int ldq, c
     NC_CHECK_ARG(nc_latent_expanded_ok(0, g) && keys >= g.pos_max + g.T && keys <= g.Tmax, "latent_expanded: sizes not supported");
     const int dqk = g.dim_p + g.rot_p;
     // causal pairs: all earlier keys and half of the new ones
-    NcStackProf prof(NC_CLS_LATENT, 2.0 * g.B * g.heads * g.T * (g.pos_max + 0.5 * (g.T + 1)) * (dqk + g.vdim_p), s, g.T);
+    NcProfScope prof(NC_CLS_LATENT, 2.0 * g.B * g.heads * g.T * (g.pos_max + 0.5 * (g.T + 1)) * (dqk + g.vdim_p), s, g.T);
     NC_CHECK_ARG((int64_t)keys * g.heads * (g.dim_p + g.vdim_p) * 2 < (1ll << 31), "latent_expanded: %d keys past 2 GiB", keys);
 #define GO(N, R, V) launch_expanded<N, R, V>(g, q, ldq, kv, keys, cache, seqlens, out, ldo, s)
 #define GO_V(N, R) (g.vdim_p <= 64 ? GO(N, R, 64) : GO(N, R, 128))

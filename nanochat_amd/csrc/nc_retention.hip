@@ -231,8 +231,9 @@ __global__ __launch_bounds__(256) void retention_chunk_kv_kernel(NcRetentionGeom
     }
 }
 
-// The state in front of every chunk, as two bf16 terms over the place of KV_c (one word per element: hi, lo halves apart by DK * DV
-// elements), and the state behind the last one.  One thread per four elements of S^T [vdim][dim].
+// The state in front of every chunk, as two bf16 terms (hi, then lo DK * DV elements on), and the state behind the last one.  The terms are
+// laid out as the operand of S^T q reads them: 32 value rows x 16 dims are 64 lanes x 8 elements, lane = row % 32 + 32 (dim % 16 / 8).
+// One thread per four elements of S^T [vdim][dim].
 __global__ __launch_bounds__(256) void retention_scan_kernel(NcRetentionGeom g, const float* __restrict__ decay, const int32_t* __restrict__ seqlens,
                                                              const float* __restrict__ kv, bf16_t* __restrict__ prefix,
                                                              const float* __restrict__ state_in, float* __restrict__ state_out, int chunks, int C) {
@@ -249,7 +250,8 @@ __global__ __launch_bounds__(256) void retention_scan_kernel(NcRetentionGeom g, 
     const float full = exp2f((float)C * l2), tail = exp2f((float)(g.T - (chunks - 1) * C) * l2);
     const int64_t step = (int64_t)g.heads * DK * DV;
     const float* src = kv + (((int64_t)b * chunks) * g.heads + h) * DK * DV + e;
-    bf16_t* dst = prefix + 2 * ((((int64_t)b * chunks) * g.heads + h) * DK * DV) + e;
+    const int place = ((v / 32 * (DK / 16) + k / 16) * 64 + v % 32 + 32 * (k % 16 / 8)) * 8 + k % 8;
+    bf16_t* dst = prefix + 2 * ((((int64_t)b * chunks) * g.heads + h) * DK * DV) + place;
 #pragma unroll 4
     for (int c = 0; c < chunks; c++) {
         const v4f add = *(const v4f*)(src + c * step);
@@ -267,7 +269,7 @@ __global__ __launch_bounds__(256) void retention_scan_kernel(NcRetentionGeom g, 
 // The outputs of one chunk and head.  Four waves: C / 32 blocks of 32 queries x the value columns dealt to 4 / (C / 32) waves, each of which
 // computes the scores of its queries for itself.  Transposed like the attention kernels (a lane owns one query): S^T = K Q^T, O^T = V^T P^T.
 template <int DK, int DV, int C>
-__global__ __launch_bounds__(256) void retention_chunk_out_kernel(NcRetentionGeom g, const bf16_t* __restrict__ proj, int ldp, const float* __restrict__ decay,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void retention_chunk_out_kernel(NcRetentionGeom g, const bf16_t* __restrict__ proj, int ldp, const float* __restrict__ decay,
                                                                   const float* __restrict__ rope, int rope_len, const int32_t* __restrict__ seqlens,
                                                                   const bf16_t* __restrict__ prefix, int chunks, float eps, bf16_t* __restrict__ out, int ldo) {
     constexpr int QB = C / 32, VS = 4 / QB, NT = DV / 32 / VS, KP = DK * 2 + 16, VP = DV * 2 + 64;
@@ -314,10 +316,10 @@ __global__ __launch_bounds__(256) void retention_chunk_out_kernel(NcRetentionGeo
         const bf16_t* st = prefix + 2 * ((((int64_t)b * chunks + chunk) * g.heads + h) * DK * DV);
 #pragma unroll
         for (int d = 0; d < NT; d++) {
-            const bf16_t* srow = st + (int64_t)(32 * (vs * NT + d) + col) * DK + 8 * hl;
+            const bf16_t* srow = st + ((int64_t)(vs * NT + d) * (DK / 16) * 64 + lane) * 8;
 #pragma unroll
             for (int c = 0; c < DK / 16; c++) {
-                const v8bf sh = as_v8bf(*(const uint4*)(srow + 16 * c)), sl = as_v8bf(*(const uint4*)(srow + DK * DV + 16 * c));
+                const v8bf sh = as_v8bf(*(const uint4*)(srow + 512 * c)), sl = as_v8bf(*(const uint4*)(srow + DK * DV + 512 * c));
                 o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, qh[c], o[d], 0, 0, 0);
                 o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, ql[c], o[d], 0, 0, 0);
                 o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sl, qh[c], o[d], 0, 0, 0);
@@ -446,12 +448,12 @@ int nc_launch_retention(int dtype, const NcRetentionGeom& g, const void* proj, i
     const int C = chunk_size(dtype, g);
     if (!C) {
         // the state once in and once out (bytes); per token the projections
-        NcStackProf prof(NC_CLS_RETENTION, (double)g.B * g.heads * (8.0 * g.dim_p * g.vdim_p + (double)g.T * (2 * g.dim_p + 3 * g.vdim_p) * (dtype ? 4 : 2)), s, g.T);
+        NcProfScope prof(NC_CLS_RETENTION, (double)g.B * g.heads * (8.0 * g.dim_p * g.vdim_p + (double)g.T * (2 * g.dim_p + 3 * g.vdim_p) * (dtype ? 4 : 2)), s, g.T);
         return dtype ? launch_step<float>(g, (const float*)proj, ldp, decay, rope, rope_len, seqlens, state_in, state_out, eps, (float*)out, ldo, s)
                      : launch_step<bf16_t>(g, (const bf16_t*)proj, ldp, decay, rope, rope_len, seqlens, state_in, state_out, eps, (bf16_t*)out, ldo, s);
     }
     // state update and read-out 4 dim vdim flops per token and head, plus the pairs inside a chunk
-    NcStackProf prof(NC_CLS_RETENTION, (double)g.B * g.heads * g.T * (4.0 * g.dim * g.vdim + (double)C * (g.dim + g.vdim)), s, g.T);
+    NcProfScope prof(NC_CLS_RETENTION, (double)g.B * g.heads * g.T * (4.0 * g.dim * g.vdim + (double)C * (g.dim + g.vdim)), s, g.T);
     const bf16_t* p = (const bf16_t*)proj;
     bf16_t* o = (bf16_t*)out;
 #define CHUNKED(K, V, CC) \

@@ -6,18 +6,10 @@
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 #include "nc_common.h"
+#include "nc_kernels.h"
 
-// timing classes of nc_profile_*
+// timing classes of NcProfScope / nc_profile_*
 enum { NC_CLS_LATENT = 0, NC_CLS_LINEAR = 1, NC_CLS_RETENTION = 2, NC_CLS_ROWS = 3, NC_CLS_EXPERTS = 4 };
-
-int nc_prof_begin(int cls, double units, hipStream_t s, int64_t tag = 0);
-void nc_prof_end(int slot, hipStream_t s);
-struct NcStackProf {
-    int slot;
-    hipStream_t s;
-    NcStackProf(int cls, double units, hipStream_t st, int64_t tag = 0) : slot(nc_prof_begin(cls, units, st, tag)), s(st) {}
-    ~NcStackProf() { nc_prof_end(slot, s); }
-};
 
 // ---------------------------------------------------------------- element helpers
 template <typename T> __device__ __forceinline__ float ld_f32(const T* p);
@@ -71,7 +63,7 @@ struct NcLinear {
     NcSeg seg[4];
     int batch;                             // >= 1: how many (A, W, out) triples the strides (in elements) walk
     int64_t a_stride, w_stride, out_stride;
-    // groups: tile t of `tiles` is {group, first row, rows}; the weight of group g starts w_stride * g elements on; row r of A is
+    // groups: tile t of `tiles` is {group, first row, rows, first tile of the group, tiles of the group}; the weight of group g starts w_stride * g elements on; row r of A is
     // a_rows[r] / a_div (or r itself without a_rows), row r of the output is r
     const int32_t* tiles;
     const int32_t* n_tiles;
@@ -91,9 +83,10 @@ inline void nc_linear_seg(NcLinear& l, int end, int kind, void* out, int ld, flo
     l.seg[l.nseg++] = NcSeg{end, kind, out, ld, p0, p1};
 }
 #define NC_FEW_ROWS 64                     // up to here the few-rows kernel
+#define NC_TILE_WORDS 5
 #define NC_GROUP_TILE_FEW 16               // rows per group tile of the few-rows kernel (the tiled one takes 64 or 128)
 int nc_launch_linear_few(int dtype, const NcLinear& l, hipStream_t s, int cls = NC_CLS_LINEAR);
-int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls = NC_CLS_LINEAR);
+int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls = NC_CLS_LINEAR, int shape = 0);     // shape 0: choose
 // splits of the summed index over workgroups that fill the chip for a few-rows linear whose consumer adds partial sums
 int nc_linear_few_splits(int M, int N, int K);
 
@@ -131,7 +124,7 @@ struct NcRoute {
     int32_t* chosen;               // [M][top]
     int32_t* slot_of;              // [M][top]
     int32_t* perm;                 // [M * top]
-    int32_t* tiles;                // [max_tiles][3]
+    int32_t* tiles;                // [max_tiles][NC_TILE_WORDS], see NcLinear
     int32_t* n_tiles;
     int tile_rows, max_tiles;
 };

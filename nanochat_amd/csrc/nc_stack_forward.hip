@@ -52,7 +52,7 @@ bool expand(int dtype, const nc_stack_layer& l, const NcLatentGeom& g) {
 }
 int expert_tile_rows(const nc_stack_layer& l, int M) {
     const int per = M * l.top / l.experts;
-    return M <= NC_FEW_ROWS || per < 16 ? NC_GROUP_TILE_FEW : per < 192 ? 64 : 128;
+    return M <= NC_FEW_ROWS || per < 16 ? NC_GROUP_TILE_FEW : per < 128 ? 64 : 128;
 }
 int expert_max_tiles(const nc_stack_layer& l, int M, int tile_rows) {
     const int pairs = M * l.top;
@@ -113,7 +113,7 @@ Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_key
     w.chosen = (int32_t*)c.take(pairs * 4);
     w.slot_of = (int32_t*)c.take(pairs * 4);
     w.perm = (int32_t*)c.take(pairs * 4);
-    w.tiles = (int32_t*)c.take(tiles * 12);
+    w.tiles = (int32_t*)c.take(tiles * NC_TILE_WORDS * 4);
     w.n_tiles = (int32_t*)c.take(4);
     w.total = (c.off + 255) & ~(size_t)255;
     return w;
@@ -283,11 +283,12 @@ extern "C" int nc_stack_forward(const nc_stack_model* m, const nc_stack_cache* k
 
 extern "C" int nc_stack_linear(int dtype, const void* a, int64_t lda, const void* w, void* out, int ldc, int M, int N, int K, int kind, float limit,
                                int kernel, nc_stream_t stream) {
-    NC_CHECK_ARG(out && kind >= 0 && kind <= 3 && N % 16 == 0, "stack_linear: kind %d, N %d", kind, N);
+    NC_CHECK_ARG(out && kind >= 0 && kind <= 3 && N % 16 == 0 && kernel >= 0 && kernel <= 6, "stack_linear: kind %d, N %d", kind, N);
     NcLinear l = nc_linear(a, lda, w, M, N, K);
     nc_linear_seg(l, N, kind, out, ldc, limit);
     if (kernel == 0) return run_linear(dtype, l, (hipStream_t)stream);
-    return kernel == 1 ? nc_launch_linear_few(dtype, l, (hipStream_t)stream) : nc_launch_linear_tiled(dtype, l, (hipStream_t)stream);
+    if (kernel == 1) return nc_launch_linear_few(dtype, l, (hipStream_t)stream);
+    return nc_launch_linear_tiled(dtype, l, (hipStream_t)stream, NC_CLS_LINEAR, kernel - 2);
 }
 
 extern "C" int nc_stack_cache_copy(const void* src, void* dst, int src_rows, int dst_rows, int64_t src_row_bytes, int64_t dst_row_bytes, int64_t n_bytes,

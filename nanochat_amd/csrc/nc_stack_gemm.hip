@@ -33,6 +33,19 @@ template <> struct Mma<float> {
     }
 };
 
+// The same pair of fragments (32 bytes of K per lane), accumulated in place and kept in program order against every memory operation: the
+// builtin lets the register allocator pick another result tuple, which it repairs with copies in every K-step, and nothing would keep
+// the LDS reads of a step in front of the barrier that ends it. 
+template <typename T>
+__device__ __forceinline__ void mma_in_place(v4f& acc, const v4i& w, const v4i& a) {
+    if constexpr (sizeof(T) == 2) {
+        asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+a"(acc) : "v"(w), "v"(a) : "memory");
+    } else {
+#pragma unroll
+        for (int j = 0; j < 4; j++) asm volatile("v_mfma_f32_16x16x4_f32 %0, %1, %2, %0" : "+a"(acc) : "v"(w[j]), "v"(a[j]) : "memory");
+    }
+}
+
 // four consecutive columns n .. n+3 (n a multiple of 4, all in one segment) of output row `row`
 template <typename T>
 __device__ __forceinline__ void store_cols(const NcLinear& g, int64_t out_off, int row, int n, v4f v) {
@@ -81,7 +94,7 @@ struct Span {
 __device__ __forceinline__ bool find_span(const NcLinear& g, int y, int batch, int tile_rows, Span& sp) {
     if (g.tiles) {
         if (y >= *g.n_tiles) return false;
-        const int32_t* t = g.tiles + 3 * y;
+        const int32_t* t = g.tiles + NC_TILE_WORDS * y;
         sp = Span{t[1], t[2], 0, (int64_t)t[0] * g.w_stride, 0};
         return true;
     }
@@ -158,11 +171,11 @@ __global__ __launch_bounds__(256) void linear_few_kernel(NcLinear g) {
 }
 
 // ------------------------------------------------------------------------------------------------
-// BM x 128 outputs, four waves (2 x 2), K-steps of 128 bytes.  Operand tiles go from global memory straight into LDS, 1 KB (8 rows x 128
-// bytes) per load instruction; chunk c (16 bytes) of row r is kept at slot c ^ SWZ(r), the permutation being applied on the global
-// side, so that the fragment reads of 16 rows are free of bank conflicts.  Four stages: the loads of three steps are in flight while one
-// is multiplied.  Past the end of K the loads are issued all the same (into stages nobody reads any more), so that the barrier counts
-// the same number of loads in every step.
+// BM x BN outputs, WM x WN waves of 16-row, 16-column tiles, K-steps of 128 bytes.  Operand tiles go from global memory straight into LDS,
+// 1 KB (8 rows x 128 bytes) per load instruction; chunk c (16 bytes) of row r is kept at slot c ^ SWZ(r), the permutation being applied
+// on the global side, so that the fragment reads of 16 rows are free of bank conflicts.  A ring of STAGES: the loads of STAGES - 1 steps
+// are in flight while one is multiplied.  Past the end of K the loads are issued all the same (into stages nobody reads any more), so
+// that the barrier counts the same number of loads in every step.
 #define TILE_SWZ(row) (((row) & 7) ^ (((row) >> 3) & 1))
 #define TILE_OOB 0x80000000u       // a buffer offset past every descriptor: the load returns zeros
 #define TILE_GROUP_M 8
@@ -176,101 +189,128 @@ __device__ __forceinline__ void tile_order(int id, int tiles_m, int tiles_n, int
     tm = first + (lin % band) % rows, tn = (lin % band) / rows;
 }
 
-template <int A_P>
+// Grouped rows: every XCD gets a contiguous run of (group, column tile, row tile of the group), the row tiles innermost, so that a weight
+// tile is read by neighbours.  The launch covers the most tiles there can be; those past the actual count leave.
+__device__ __forceinline__ bool group_tile_order(const NcLinear& g, int id, int tiles_n, int& tm, int& tn) {
+    const int total = *g.n_tiles * tiles_n;
+    if (id >= total) return false;
+    const int xcd = id & 7, lin = xcd * (total >> 3) + min(xcd, total & 7) + (id >> 3);
+    const int32_t* t = g.tiles + NC_TILE_WORDS * (lin / tiles_n);
+    const int first = t[3], count = t[4], o = lin - first * tiles_n;
+    tm = first + o % count, tn = o / count;
+    return true;
+}
+
+template <int A_P, int W_P, int STRIDE>
 __device__ __forceinline__ void tile_fetch(const void* A, uint32_t a_bytes, const void* W, uint32_t w_bytes, uint8_t* st, int w_part,
                                            const uint32_t* vo_a, const uint32_t* vo_w, int k_off) {
     const __amdgpu_buffer_rsrc_t da = __builtin_amdgcn_make_buffer_rsrc((void*)A, 0, a_bytes, 0x00020000);
     const __amdgpu_buffer_rsrc_t dw = __builtin_amdgcn_make_buffer_rsrc((void*)W, 0, w_bytes, 0x00020000);
 #pragma unroll
-    for (int i = 0; i < A_P; i++) __builtin_amdgcn_raw_ptr_buffer_load_lds(da, (lds_ptr_t)(st + i * 4096), 16, vo_a[i], k_off, 0, 0);
+    for (int i = 0; i < A_P; i++) __builtin_amdgcn_raw_ptr_buffer_load_lds(da, (lds_ptr_t)(st + i * STRIDE), 16, vo_a[i], k_off, 0, 0);
 #pragma unroll
-    for (int i = 0; i < 4; i++) __builtin_amdgcn_raw_ptr_buffer_load_lds(dw, (lds_ptr_t)(st + w_part + i * 4096), 16, vo_w[i], k_off, 0, 0);
+    for (int i = 0; i < W_P; i++) __builtin_amdgcn_raw_ptr_buffer_load_lds(dw, (lds_ptr_t)(st + w_part + i * STRIDE), 16, vo_w[i], k_off, 0, 0);
 }
 
-template <typename T, int BM>
-__global__ __launch_bounds__(256) void linear_tiled_kernel(NcLinear g, int tiles_m, int tiles_n, uint32_t a_bytes) {
-    constexpr int WTM = BM / 32, STAGE = (BM + 128) * 128, A_P = BM / 32, LOADS = A_P + 4;
-    // s_waitcnt vmcnt(2 * LOADS), other counters untouched: the loads of the two youngest steps may still be in flight
-    constexpr int WAIT2 = 0x0F70 | ((2 * LOADS) & 15) | (((2 * LOADS) >> 4) << 14);
+template <typename T, int BM, int BN, int WM, int WN, int STAGES>
+__global__ __launch_bounds__(64 * WM * WN) void linear_tiled_kernel(NcLinear g, int tiles_m, int tiles_n, uint32_t a_bytes) {
+    constexpr int NW = WM * WN, WTM = BM / WM / 16, WTN = BN / WN / 16, STAGE = (BM + BN) * 128, A_P = BM / 8 / NW, W_P = BN / 8 / NW;
+    // s_waitcnt vmcnt(loads of the STAGES - 2 youngest steps), other counters untouched
+    constexpr int FLIGHT = (STAGES - 2) * (A_P + W_P), WAIT = 0x0F70 | (FLIGHT & 15) | ((FLIGHT >> 4) << 14);
+    static_assert(A_P >= 1 && W_P >= 1 && NW % 2 == 0, "waves");
     extern __shared__ __align__(16) uint8_t lds[];
     int tm, tn;
-    if (g.tiles) tm = (int)blockIdx.x / tiles_n, tn = (int)blockIdx.x % tiles_n;
-    else tile_order(blockIdx.x, tiles_m, tiles_n, tm, tn);
+    if (g.tiles) {
+        if (!group_tile_order(g, blockIdx.x, tiles_n, tm, tn)) return;
+    } else {
+        tile_order(blockIdx.x, tiles_m, tiles_n, tm, tn);
+    }
     Span sp;
     if (!find_span(g, tm, blockIdx.y, BM, sp)) return;
-    const int n0 = tn * 128;
+    const int n0 = tn * BN;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int wm = wave >> 1, wn = wave & 1, frow = lane & 15, piece = lane >> 4;
-    // staging: this lane's row inside an 8-row block, and the global chunk that belongs in its LDS slot
+    const int wm = wave / WN, wn = wave % WN, frow = lane & 15, piece = lane >> 4;
+    // staging: piece i of this wave is the 1 KB block (wave + NW i) of its operand's part of the stage; this lane's row inside an 8-row
+    // block, and the global chunk that belongs in its LDS slot
     const int sub = lane >> 3, gch = (lane & 7) ^ sub ^ (wave & 1);
     const int rd_lo = frow * 128 + (((2 * piece) ^ TILE_SWZ(frow)) << 4), rd_hi = frow * 128 + (((2 * piece + 1) ^ TILE_SWZ(frow)) << 4);
     const uint32_t row_a = (uint32_t)(g.lda * sizeof(T)), row_w = (uint32_t)(g.K * sizeof(T));
     const T* const A = (const T*)g.a + sp.a_off;
     const T* const W = (const T*)g.w + sp.w_off;
-    uint32_t vo_a[A_P], vo_w[4];
+    uint32_t vo_a[A_P], vo_w[W_P];
 #pragma unroll
     for (int i = 0; i < A_P; i++) {
-        const int r = 8 * wave + 32 * i + sub;
+        const int r = 8 * (wave + NW * i) + sub;
         vo_a[i] = r < sp.rows ? (uint32_t)a_row(g, sp.row0 + r) * row_a + gch * 16 : TILE_OOB;
     }
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const int r = n0 + 8 * wave + 32 * i + sub;
+    for (int i = 0; i < W_P; i++) {
+        const int r = n0 + 8 * (wave + NW * i) + sub;
         vo_w[i] = r < g.N ? (uint32_t)r * row_w + gch * 16 : TILE_OOB;
     }
     const int ksteps = row_w / 128;
-    v4f acc[WTM][4];
+    v4f acc[WTM][WTN];
 #pragma unroll
     for (int i = 0; i < WTM; i++)
 #pragma unroll
-        for (int j = 0; j < 4; j++) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
-    auto fetch = [&](int t) {
-        tile_fetch<A_P>(A, a_bytes, W, (uint32_t)g.N * row_w, lds + (t & 3) * STAGE + wave * 1024, BM * 128, vo_a, vo_w, t < ksteps ? t * 128 : 0);
+        for (int j = 0; j < WTN; j++) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
+    auto fetch = [&](int t, int stage) {
+        tile_fetch<A_P, W_P, NW * 1024>(A, a_bytes, W, (uint32_t)g.N * row_w, lds + stage * STAGE + wave * 1024, BM * 128, vo_a, vo_w,
+                                        t < ksteps ? t * 128 : 0);
     };
-    auto compute = [&](int t) {
-        const uint8_t* a = lds + (t & 3) * STAGE + wm * (BM / 2) * 128;
-        const uint8_t* w = lds + (t & 3) * STAGE + BM * 128 + wn * 64 * 128;
-#pragma unroll
-        for (int half = 0; half < 2; half++) {
-            const int rd = half ? rd_hi : rd_lo;
-            v4i af[WTM], wf[4];
-#pragma unroll
-            for (int i = 0; i < WTM; i++) af[i] = *(const v4i*)(a + i * 2048 + rd);
-#pragma unroll
-            for (int j = 0; j < 4; j++) wf[j] = *(const v4i*)(w + j * 2048 + rd);
-#pragma unroll
-            for (int j = 0; j < 4; j++)
-#pragma unroll
-                for (int i = 0; i < WTM; i++) acc[i][j] = Mma<T>::run(wf[j], af[i], acc[i][j]);
-        }
-    };
-    fetch(0);
-    fetch(1);
-    fetch(2);
-    asm volatile("" ::: "memory");
-    __builtin_amdgcn_s_waitcnt(WAIT2);
-    __builtin_amdgcn_s_barrier();
-    asm volatile("" ::: "memory");
-    for (int kt = 0; kt < ksteps; kt++) {
-        fetch(kt + 3);                       // into the stage that was read in step kt - 1: everyone is past the barrier that ended it
-        compute(kt);
+    auto meet = [&]() {
         asm volatile("" ::: "memory");
-        __builtin_amdgcn_s_waitcnt(WAIT2);   // the operands of step kt + 1 have landed (this wave's share; the barrier says everybody's)
+        __builtin_amdgcn_s_waitcnt(WAIT);    // the operands of the next step have landed (this wave's share; the barrier says everybody's)
         __builtin_amdgcn_s_barrier();
         asm volatile("" ::: "memory");
+    };
+#pragma unroll
+    for (int i = 0; i < STAGES - 1; i++) fetch(i, i);
+    meet();
+    int cur = 0, nxt = STAGES - 1;
+    for (int kt = 0; kt < ksteps; kt++) {
+        const uint8_t* a = lds + cur * STAGE + wm * (BM / WM) * 128;
+        const uint8_t* w = lds + cur * STAGE + BM * 128 + wn * (BN / WN) * 128;
+        v4i al[WTM], ah[WTM], wl[2], wh[2];
+        wl[0] = *(const v4i*)(w + rd_lo);
+#pragma unroll
+        for (int i = 0; i < WTM; i++) al[i] = *(const v4i*)(a + i * 2048 + rd_lo);
+        wh[0] = *(const v4i*)(w + rd_hi);
+#pragma unroll
+        for (int i = 0; i < WTM; i++) ah[i] = *(const v4i*)(a + i * 2048 + rd_hi);
+        fetch(kt + STAGES - 1, nxt);         // into the stage read in step kt - 1: everyone is past the barrier that ended it
+#pragma unroll
+        for (int j = 0; j < WTN; j++) {
+            if (j + 1 < WTN) {               // one group ahead of its use
+                wl[(j + 1) & 1] = *(const v4i*)(w + (j + 1) * 2048 + rd_lo);
+                wh[(j + 1) & 1] = *(const v4i*)(w + (j + 1) * 2048 + rd_hi);
+            }
+#pragma unroll
+            for (int i = 0; i < WTM; i++) mma_in_place<T>(acc[i][j], wl[j & 1], al[i]);
+#pragma unroll
+            for (int i = 0; i < WTM; i++) mma_in_place<T>(acc[i][j], wh[j & 1], ah[i]);
+        }
+        meet();
+        cur = cur + 1 == STAGES ? 0 : cur + 1;
+        nxt = nxt + 1 == STAGES ? 0 : nxt + 1;
     }
     // the loads past the end of K are still landing: they must be done before the workgroup gives its LDS back
     asm volatile("" ::: "memory");
     __builtin_amdgcn_s_waitcnt(0x0F70);
     __builtin_amdgcn_s_barrier();
-    asm volatile("" ::: "memory");
+    // (the last products: the compiler does not see that an asm statement wrote the accumulators late)
+    asm volatile("s_nop 15\n\ts_nop 15" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < WTM; i++)
+#pragma unroll
+        for (int j = 0; j < WTN; j++) asm volatile("" : "+a"(acc[i][j]));
 #pragma unroll
     for (int i = 0; i < WTM; i++) {
-        const int m = wm * (BM / 2) + 16 * i + frow;
+        const int m = wm * (BM / WM) + 16 * i + frow;
         if (m >= sp.rows) continue;
 #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const int n = n0 + wn * 64 + 16 * j + 4 * piece;
+        for (int j = 0; j < WTN; j++) {
+            const int n = n0 + wn * (BN / WN) + 16 * j + 4 * piece;
             if (n < g.N) store_cols<T>(g, sp.out_off, sp.row0 + m, n, acc[i][j]);
         }
     }
@@ -306,22 +346,31 @@ int launch_few_t(const NcLinear& l, hipStream_t s) {
     if (l.tiles) return l.N >= 2048 ? launch_few<T, 1, 2>(l, l.max_tiles, s) : launch_few<T, 1, 1>(l, l.max_tiles, s);
     if (l.M <= 16) return (int64_t)l.N * l.splits * l.batch >= 16384 ? launch_few<T, 1, 2>(l, 1, s) : launch_few<T, 1, 1>(l, 1, s);
     if (l.M <= 32) return launch_few<T, 2, 2>(l, 1, s);
-    return launch_few<T, 4, 4>(l, (l.M + 63) / 64, s);
+    // (64 rows, K = 2048: N = 32768 54 us with four column tiles per workgroup against 66 with two, N = 7808 32 against 19)
+    return l.N >= 16384 ? launch_few<T, 4, 4>(l, (l.M + 63) / 64, s) : launch_few<T, 4, 2>(l, (l.M + 63) / 64, s);
 }
-template <typename T, int BM>
+template <typename T, int BM, int BN, int WM, int WN, int STAGES>
 int launch_tiled(const NcLinear& l, hipStream_t s) {
     static std::atomic<uint64_t> done{0};
-    constexpr int LDS = (BM + 128) * 128 * 4;
-    const void* fn = (const void*)linear_tiled_kernel<T, BM>;
+    constexpr int LDS = (BM + BN) * 128 * STAGES;
+    const void* fn = (const void*)linear_tiled_kernel<T, BM, BN, WM, WN, STAGES>;
     if (int rc = reserve_dynamic_lds(fn, LDS, done)) return rc;
-    const int tm = l.tiles ? l.max_tiles : (l.M + BM - 1) / BM, tn = (l.N + 127) / 128;
+    const int tm = l.tiles ? l.max_tiles : (l.M + BM - 1) / BM, tn = (l.N + BN - 1) / BN;
     // rows of A this launch may reach: all of them (a gathered row index is below M / a_div)
     const int64_t a_rows = l.a_rows ? (l.M + l.a_div - 1) / l.a_div : l.M;
     const int64_t a_bytes = ((a_rows - 1) * l.lda + l.K) * (int64_t)sizeof(T);
     NC_CHECK_ARG(a_bytes < (1ll << 31) && (int64_t)l.N * l.K * (int64_t)sizeof(T) < (1ll << 31), "linear: operand past 2 GiB");
-    hipLaunchKernelGGL((linear_tiled_kernel<T, BM>), dim3(tm * tn, l.batch), dim3(256), LDS, s, l, tm, tn, (uint32_t)a_bytes);
+    hipLaunchKernelGGL((linear_tiled_kernel<T, BM, BN, WM, WN, STAGES>), dim3(tm * tn, l.batch), dim3(64 * WM * WN), LDS, s, l, tm, tn, (uint32_t)a_bytes);
     NC_CHECK_LAUNCH("linear_tiled");
     return 0;
+}
+// tile shapes: 1 = 64 x 128, 2 = 128 x 128, 3 = 256 x 256, 4 = 128 x 256
+template <typename T>
+int launch_tiled_shape(const NcLinear& l, int shape, hipStream_t s) {
+    if (shape == 1) return launch_tiled<T, 64, 128, 2, 2, 3>(l, s);
+    if (shape == 2) return launch_tiled<T, 128, 128, 2, 2, 2>(l, s);
+    if (shape == 3) return launch_tiled<T, 256, 256, 4, 2, 2>(l, s);
+    return launch_tiled<T, 128, 256, 2, 4, 3>(l, s);
 }
 
 double linear_units(const NcLinear& l, int dtype, bool few) {
@@ -332,7 +381,7 @@ int64_t linear_tag(const NcLinear& l) { return ((int64_t)l.N << 32) | (uint32_t)
 }  // namespace
 
 int nc_linear_few_splits(int M, int N, int K) {
-    const int nb = M <= 16 ? 16 : M <= 32 ? 32 : 64;
+    const int nb = M <= 16 ? 16 : 32;
     const int wgs = (N + nb - 1) / nb;
     int splits = 1;
     while (splits < 8 && wgs * splits < 384 && K / (splits * 2) >= 256) splits *= 2;
@@ -343,17 +392,20 @@ int nc_launch_linear_few(int dtype, const NcLinear& l, hipStream_t s, int cls) {
     if (int rc = check_linear(l, dtype)) return rc;
     NC_CHECK_ARG(!l.tiles || l.tile_rows == NC_GROUP_TILE_FEW, "linear: group tiles of %d rows", l.tile_rows);
     NC_CHECK_ARG(l.splits >= 1 && (l.splits == 1 || l.partials), "linear: split sums need a buffer");
-    NcStackProf prof(cls, linear_units(l, dtype, true), s, linear_tag(l));
+    NcProfScope prof(cls, linear_units(l, dtype, true), s, linear_tag(l));
     return dtype ? launch_few_t<float>(l, s) : launch_few_t<bf16_t>(l, s);
 }
 
-int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls) {
+int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls, int shape) {
     if (int rc = check_linear(l, dtype)) return rc;
     NC_CHECK_ARG(!l.partials && l.K % 64 == 0, "linear: the tiled kernel takes whole K-steps and finishes its sums");
-    NcStackProf prof(cls, linear_units(l, dtype, false), s, linear_tag(l));
-    // a launch that would leave compute units without a tile takes the lower tile
-    const int64_t tiles128 = (int64_t)((l.M + 127) / 128) * ((l.N + 127) / 128) * l.batch;
-    if (l.tiles) NC_CHECK_ARG(l.tile_rows == 64 || l.tile_rows == 128, "linear: group tiles of %d rows", l.tile_rows);
-    if (l.tiles ? l.tile_rows == 64 : tiles128 < 256) return dtype ? launch_tiled<float, 64>(l, s) : launch_tiled<bf16_t, 64>(l, s);
-    return dtype ? launch_tiled<float, 128>(l, s) : launch_tiled<bf16_t, 128>(l, s);
+    NcProfScope prof(cls, linear_units(l, dtype, false), s, linear_tag(l));
+    if (!shape) {
+        // the widest tile unless it leaves compute units without one (measured at 1792 rows: 858 against 679 TFLOP/s at N = 12352, 551
+        // against 717 at N = 2048, where the launch has 112 or 448 tiles)
+        const int64_t wide = (int64_t)((l.M + 127) / 128) * ((l.N + 255) / 256) * l.batch;
+        shape = l.tiles ? (l.tile_rows == 64 ? 1 : 4) : wide < 200 ? 1 : 4;
+    }
+    if (l.tiles) NC_CHECK_ARG(l.tile_rows == (shape == 1 ? 64 : shape == 3 ? 256 : 128), "linear: group tiles of %d rows", l.tile_rows);
+    return dtype ? launch_tiled_shape<float>(l, shape, s) : launch_tiled_shape<bf16_t>(l, shape, s);
 }

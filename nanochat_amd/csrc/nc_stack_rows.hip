@@ -56,45 +56,91 @@ __global__ __launch_bounds__(ROW_THREADS) void stack_embed_kernel(const int64_t*
     layer_norm_row<T, STEPS>(v, norm_w, eps, width, width_p, h + m * width_p, red);
 }
 
+// (every loop over splits and choices asks for its loads in batches, all of a batch before the first sum: a few rows' worth of these
+// kernels lasts as long as its longest chain of dependent loads)
 template <typename T, int STEPS>
 __global__ __launch_bounds__(ROW_THREADS) void stack_row_add_kernel(NcRowAdd a, float eps, int M, int width, int width_p) {
+    constexpr int BATCH = 8;
     __shared__ float red[ROW_THREADS / 64];
     const int64_t m = a.rows ? a.rows[blockIdx.x] : (int)blockIdx.x;
     v4f v[STEPS];
 #pragma unroll
     for (int i = 0; i < STEPS; i++) {
         const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS);
-        v[i] = v4f{0.f, 0.f, 0.f, 0.f};
-        if (c >= width_p) continue;
-        v4f x = *(const v4f*)(a.x + m * width_p + c);
-        if (a.partials) {
-            v4f p = *(const v4f*)(a.partials + m * width_p + c);
-            for (int s = 1; s < a.splits; s++) p += *(const v4f*)(a.partials + ((int64_t)s * M + m) * width_p + c);
-            x += p;
-        }
-        if (a.expert_out) {
-            v4f y = v4f{0.f, 0.f, 0.f, 0.f};
-            for (int k = 0; k < a.top; k++) {
-                const int64_t slot = a.slot_of[m * a.top + k];
-                y += ld4_f32((const T*)a.expert_out + slot * width_p + c) * a.slot_w[m * a.top + k];
+        v[i] = c < width_p ? *(const v4f*)(a.x + m * width_p + c) : v4f{0.f, 0.f, 0.f, 0.f};
+    }
+    if (a.partials) {
+#pragma unroll
+        for (int i = 0; i < STEPS; i++) {
+            const int c = min(4 * ((int)threadIdx.x + i * ROW_THREADS), width_p - 4);
+            v4f p[BATCH], sum = v4f{0.f, 0.f, 0.f, 0.f};
+            for (int s0 = 0; s0 < a.splits; s0 += BATCH) {
+#pragma unroll
+                for (int s = 0; s < BATCH; s++) p[s] = *(const v4f*)(a.partials + ((int64_t)min(s0 + s, a.splits - 1) * M + m) * width_p + c);
+#pragma unroll
+                for (int s = 0; s < BATCH; s++)
+                    if (s0 + s < a.splits) sum += p[s];
             }
-            x += y;
+            v[i] += sum;
         }
-        if (a.tap) *(v4f*)(a.tap + m * width_p + c) = x;
-        if (a.x0) x += *(const v4f*)(a.x0 + m * width_p + c);
-        if (a.step) x += *(const v4f*)(a.step + c);
-        if (!a.rows) *(v4f*)(a.x + m * width_p + c) = x;
-        v[i] = x;
+    }
+    if (a.expert_out) {
+        v4f sum[STEPS];
+#pragma unroll
+        for (int i = 0; i < STEPS; i++) sum[i] = v4f{0.f, 0.f, 0.f, 0.f};
+        for (int k0 = 0; k0 < a.top; k0 += BATCH) {
+            int64_t slot[BATCH];
+            float w[BATCH];
+#pragma unroll
+            for (int k = 0; k < BATCH; k++) {
+                const int64_t p = m * a.top + min(k0 + k, a.top - 1);
+                slot[k] = a.slot_of[p];
+                w[k] = a.slot_w[p];
+            }
+#pragma unroll
+            for (int i = 0; i < STEPS; i++) {
+                const int c = min(4 * ((int)threadIdx.x + i * ROW_THREADS), width_p - 4);
+                v4f y[BATCH];
+#pragma unroll
+                for (int k = 0; k < BATCH; k++) y[k] = ld4_f32((const T*)a.expert_out + slot[k] * width_p + c);
+#pragma unroll
+                for (int k = 0; k < BATCH; k++)
+                    if (k0 + k < a.top) sum[i] += y[k] * w[k];
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < STEPS; i++) v[i] += sum[i];
+    }
+#pragma unroll
+    for (int i = 0; i < STEPS; i++) {
+        const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS);
+        if (c >= width_p) {
+            v[i] = v4f{0.f, 0.f, 0.f, 0.f};
+            continue;
+        }
+        if (a.tap) *(v4f*)(a.tap + m * width_p + c) = v[i];
+        if (a.x0) v[i] += *(const v4f*)(a.x0 + m * width_p + c);
+        if (a.step) v[i] += *(const v4f*)(a.step + c);
+        if (!a.rows) *(v4f*)(a.x + m * width_p + c) = v[i];
     }
     if (a.h) layer_norm_row<T, STEPS>(v, a.norm_w, eps, width, width_p, (T*)a.h + (int64_t)blockIdx.x * width_p, red);
     if (a.bump && threadIdx.x == 0 && (int)blockIdx.x % a.tokens_per_row == a.tokens_per_row - 1) a.bump[(int)blockIdx.x / a.tokens_per_row] += a.bump_by;
 }
 
 // ------------------------------------------------------------------------------------------------ expert choice
-// One wave per row: lane l holds the scores of experts l, l + 64, ...; ties go to the lower index.
+// One wave per row: lane l holds the scores of experts l, l + 64, ...; ties go to the lowest lane.
 constexpr int ROUTE_MAX_EXPERTS = 1024;
-__device__ __forceinline__ void choose_experts(const NcRoute& r, int m, int lane) {
-    constexpr int PER = ROUTE_MAX_EXPERTS / 64;
+// maximum over the wave: inside rows of 16 lanes without leaving the registers
+__device__ __forceinline__ float row_wave_max(float v) {
+    v = fmaxf(v, dpp_f32<0x128>(v));
+    v = fmaxf(v, dpp_f32<0x124>(v));
+    v = fmaxf(v, dpp_f32<0x122>(v));
+    v = fmaxf(v, dpp_f32<0x121>(v));
+    v = fmaxf(v, __shfl_xor(v, 16));
+    return fmaxf(v, __shfl_xor(v, 32));
+}
+template <int PER>
+__device__ __forceinline__ void choose_experts_of(const NcRoute& r, int m, int lane) {
     float s[PER];
     const float* z = r.logits + (int64_t)m * r.ld;
     float mx = -3.0e38f;
@@ -104,7 +150,7 @@ __device__ __forceinline__ void choose_experts(const NcRoute& r, int m, int lane
         s[i] = e < r.experts ? z[e] : -3.0e38f;
         mx = fmaxf(mx, s[i]);
     }
-    mx = wave_max(mx);
+    mx = row_wave_max(mx);
     float sum = 0.f;
 #pragma unroll
     for (int i = 0; i < PER; i++) {
@@ -120,12 +166,10 @@ __device__ __forceinline__ void choose_experts(const NcRoute& r, int m, int lane
 #pragma unroll
         for (int i = 0; i < PER; i++)
             if (s[i] > best) best = s[i], at = lane + 64 * i;
-#pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float v2 = __shfl_xor(best, o);
-            const int a2 = __shfl_xor(at, o);
-            if (v2 > best || (v2 == best && a2 < at)) best = v2, at = a2;
-        }
+        // (a row of NaN scores chooses experts 0, 1, ..: `best` keeps its start value)
+        const float top = row_wave_max(best);
+        at = __builtin_amdgcn_readlane(at, __ffsll((unsigned long long)__builtin_amdgcn_ballot_w64(best == top)) - 1);
+        best = top;
         const float score = best / sum;
         chosen_sum += score;
         if (lane == k) mine = score;
@@ -135,6 +179,12 @@ __device__ __forceinline__ void choose_experts(const NcRoute& r, int m, int lane
             if (at == lane + 64 * i) s[i] = -1.5f;
     }
     if (lane < r.top) r.slot_w[m * r.top + lane] = mine / (chosen_sum + 1e-20f);
+}
+
+__device__ __forceinline__ void choose_experts(const NcRoute& r, int m, int lane) {
+    if (r.experts <= 64) choose_experts_of<1>(r, m, lane);
+    else if (r.experts <= 256) choose_experts_of<4>(r, m, lane);
+    else choose_experts_of<ROUTE_MAX_EXPERTS / 64>(r, m, lane);
 }
 
 __global__ __launch_bounds__(256) void route_choose_kernel(NcRoute r, int M) {
@@ -170,8 +220,8 @@ __global__ __launch_bounds__(1024) void route_sort_kernel(NcRoute r, int M) {
                 const int row0 = rows_before + cs - c, tile0 = tiles_before + ts - t;
                 start[e] = row0;
                 for (int i = 0; i < t; i++) {
-                    int32_t* tile = r.tiles + 3 * (tile0 + i);
-                    tile[0] = e, tile[1] = row0 + i * r.tile_rows, tile[2] = min(r.tile_rows, c - i * r.tile_rows);
+                    int32_t* tile = r.tiles + NC_TILE_WORDS * (tile0 + i);
+                    tile[0] = e, tile[1] = row0 + i * r.tile_rows, tile[2] = min(r.tile_rows, c - i * r.tile_rows), tile[3] = tile0, tile[4] = t;
                 }
             }
             rows_before += __shfl(cs, 63), tiles_before += __shfl(ts, 63);
@@ -208,7 +258,7 @@ __global__ __launch_bounds__(256) void stack_cache_copy_kernel(const uint8_t* __
 int nc_launch_stack_embed(int dtype, const int64_t* idx, const void* embed, float scale, const float* step, int vocab, float* x, float* x0,
                           const float* norm_w, float eps, void* h, int M, int width, int width_p, hipStream_t s) {
     NC_CHECK_ARG(width_p % 4 == 0 && width <= width_p && width_p <= 8192, "stack_embed: width %d", width_p);
-    NcStackProf prof(NC_CLS_ROWS, (double)M * width_p * 8, s);
+    NcProfScope prof(NC_CLS_ROWS, (double)M * width_p * 8, s);
 #define CALL(S)                                                                                                                                \
     if (dtype) hipLaunchKernelGGL((stack_embed_kernel<float, S>), dim3(M), dim3(ROW_THREADS), 0, s, idx, (const float*)embed, scale, step, vocab, \
                                   x, x0, norm_w, eps, (float*)h, width, width_p);                                                              \
@@ -223,7 +273,7 @@ int nc_launch_stack_embed(int dtype, const int64_t* idx, const void* embed, floa
 int nc_launch_stack_row_add(int dtype, const NcRowAdd& a, float eps, int M, int n_rows, int width, int width_p, hipStream_t s) {
     NC_CHECK_ARG(width_p % 4 == 0 && width <= width_p && width_p <= 8192, "stack_row_add: width %d", width_p);
     if (n_rows == 0) return 0;
-    NcStackProf prof(NC_CLS_ROWS, (double)n_rows * width_p * (8 + (dtype ? 4 : 2) + 4.0 * (a.partials ? a.splits : 0) + (a.expert_out ? 2.0 * a.top : 0)), s);
+    NcProfScope prof(NC_CLS_ROWS, (double)n_rows * width_p * (8 + (dtype ? 4 : 2) + 4.0 * (a.partials ? a.splits : 0) + (a.expert_out ? 2.0 * a.top : 0)), s);
 #define CALL(S)                                                                                                                  \
     if (dtype) hipLaunchKernelGGL((stack_row_add_kernel<float, S>), dim3(n_rows), dim3(ROW_THREADS), 0, s, a, eps, M, width, width_p); \
     else hipLaunchKernelGGL((stack_row_add_kernel<bf16_t, S>), dim3(n_rows), dim3(ROW_THREADS), 0, s, a, eps, M, width, width_p)
@@ -236,7 +286,7 @@ int nc_launch_stack_row_add(int dtype, const NcRowAdd& a, float eps, int M, int 
 int nc_launch_stack_route(const NcRoute& r, int M, hipStream_t s) {
     NC_CHECK_ARG(r.experts >= 1 && r.experts <= ROUTE_MAX_EXPERTS && r.top >= 1 && r.top <= 64 && r.top <= r.experts, "route: %d of %d experts", r.top,
                  r.experts);
-    NcStackProf prof(NC_CLS_ROWS, (double)M * r.experts * 4, s);
+    NcProfScope prof(NC_CLS_ROWS, (double)M * r.experts * 4, s);
     if (M <= 64) {
         hipLaunchKernelGGL((route_sort_kernel<true>), dim3(1), dim3(1024), 0, s, r, M);
     } else {
@@ -252,7 +302,7 @@ int nc_launch_stack_cache_copy(const void* src, void* dst, int src_rows, int dst
     NC_CHECK_ARG(src && dst && (src_rows == 1 || src_rows == dst_rows) && dst_rows > 0, "stack_cache_copy: bad rows");
     NC_CHECK_ARG(bytes % 16 == 0 && src_stride % 16 == 0 && dst_stride % 16 == 0, "stack_cache_copy: sizes must be multiples of 16 bytes");
     if (bytes == 0) return 0;
-    NcStackProf prof(NC_CLS_ROWS, 2.0 * bytes * dst_rows, s);
+    NcProfScope prof(NC_CLS_ROWS, 2.0 * bytes * dst_rows, s);
     const int64_t pieces = bytes / 16;
     const int gx = (int)(pieces / 1024 < 1 ? 1 : pieces / 1024 > 512 ? 512 : pieces / 1024);
     hipLaunchKernelGGL(stack_cache_copy_kernel, dim3(gx, dst_rows), dim3(256), 0, s, (const uint8_t*)src, (uint8_t*)dst, src_rows, src_stride, dst_stride,

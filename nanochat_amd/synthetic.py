@@ -53,6 +53,39 @@ def random_init_model(cfg, device, seed=0):
     return model
 
 
+def palilix_config(width, heads, rank=512, experts=64, top=6, expert_ff=1024, vocab=32768, groups=1):
+    """A Palilix configuration with the proportions of an ordinary model of this width: `groups` times (latent attention + dense,
+    retention + experts twice, latent attention + experts), heads of 128, no repeated layers."""
+    head = width // heads
+    moe = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "router": {"experts": experts, "top": top}, "shared": {"ff": 2 * expert_ff, "limit": 7.0}}
+    lat = {"heads": heads, "dim": head, "rot_dim": head // 2, "vdim": head, "kv_rank": rank, "scale": (1.5 * head) ** -0.5,
+           "rot": {"base": 10000.0, "dims": head // 2}}
+    ret = {"heads": heads, "dim": head, "vdim": head, "decay": [1 - 2.0 ** -(5 + 6 * i / max(1, heads - 1)) for i in range(heads)],
+           "rot": {"base": 10000.0, "dims": head}}
+    group = [{"type": "latent_attention", "mixer": lat, "mlp": {"kind": "dense", "ff": 4 * width}}, {"type": "retention", "mixer": ret, "mlp": moe},
+             {"type": "retention", "mixer": ret, "mlp": moe}, {"type": "latent_attention", "mixer": lat, "mlp": moe}]
+    return {"architecture": "Palilix", "embedding": {"scale": 1.0}, "layers": group * groups, "logit_scale": 1.0, "logit_softcap": 30.0,
+            "norm": {"eps": 1e-6}, "vocab": vocab, "width": width}
+
+
+def random_stack_model(cls, cfg, device, dtype=torch.bfloat16, seed=0):
+    """A LayerStack design (its class and configuration) with random bf16 weights drawn on the device."""
+    g = torch.Generator(device=device).manual_seed(seed)
+    with torch.device("meta"):
+        model = cls.from_config(cfg, dtype)
+    tensors = {}
+    for name, shape in model.tensor_shapes(model.config).items():
+        t = torch.empty(shape, dtype=torch.bfloat16, device=device)
+        if name == "embed" or name == "loop.step":
+            t.normal_(0.0, 1.0, generator=g)
+        elif len(shape) == 1:
+            t.fill_(1.0)
+        else:
+            t.normal_(0.0, shape[-1] ** -0.5, generator=g)
+        tensors[name] = t
+    return model.load_tensors(tensors, device).eval()
+
+
 class SyntheticTokenizer:
     """encode_special / get_bos_token_id / encode / decode: the Engine's whole view of a tokenizer (engine.py:186-192).
     The specials sit outside the vocabulary, so sampling from a random model never ends a row early."""

@@ -48,9 +48,9 @@ CASES = {
     "large_heads": config([(latent(heads=1, dim=160, rot_dim=96, vdim=144, kv_rank=680, scale=0.07), dense(ff=96)),
                            (retention(heads=1, dim=288, vdim=264, rot_dims=288), None)], width=128, vocab=64, loop=(0, 2, 2)),
     # the whole stack looped, one head, every expert chosen, no softcap, a decay of exactly 1
-    "ones": config([(latent(heads=1, dim=32, rot_dim=32, vdim=32, kv_rank=64, scale=1.0), moe(experts=4, top=4, ff=64, limit=0.5, shared=(64, 0.5))),
+    "ones": config([(latent(heads=1, dim=32, rot_dim=32, vdim=32, kv_rank=64, scale=0.15), moe(experts=4, top=4, ff=64, limit=0.5, shared=(64, 0.5))),
                     (retention(heads=3, dim=64, vdim=64, rot_dims=64, decay=[1.0, 0.25, 0.5]), moe(experts=1, top=1, ff=16, limit=1.0))],
-                   width=64, vocab=48, loop=(0, 2, 2), softcap=None, scale=1.0, logit_scale=1.0),
+                   width=64, vocab=48, loop=(0, 2, 2), softcap=None, scale=5.0, logit_scale=1.0),
 }
 
 

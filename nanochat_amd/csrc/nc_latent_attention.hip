@@ -11,6 +11,7 @@
 //                    the form for many query rows, where dim + rot + vdim per key and head is less work than 2 rank + rot.
 // Scores, softmax and sums are fp32.  Where the weights meet the bf16 values on the matrix cores they go in as two bf16 terms (the
 // rounded weight and what rounding left), so that the product sees them to 16 bits.
+#include <atomic>
 #include "nc_stack.h"
 
 typedef __bf16 v8bf __attribute__((ext_vector_type(8)));
@@ -149,135 +150,151 @@ __global__ __launch_bounds__(256) void latent_simple_kernel(NcLatentGeom g, cons
 }
 
 // ------------------------------------------------------------------------------------------------ latent space, matrix cores
-// A workgroup takes 16 query rows (row = token * heads + head of one batch row) and a share of the keys, 64 keys at a time through LDS:
-//   scores   wave w multiplies keys 16 w .. 16 w + 15 with all 16 queries (S^T = K Q^T), and leaves them in LDS;
-//   softmax  every wave reads all 64 x 16 scores (lane = one query, 16 of the keys), so the running maximum and sum need no exchange
-//            between waves, and has the weights in the layout of the second product's operand;
-//   sums     wave w adds the columns 16 (w + 4 n) .. + 15 of the latent: O^T += C^T P^T, C^T through the transposing LDS read.
+// A workgroup of eight waves takes 16 query rows (row = token * heads + head of one batch row) and a share of the keys, 64 keys at a time
+// through LDS:
+//   scores   wave w multiplies keys 16 (w % 4) .. + 15 with all 16 queries over one half of the row (S^T = K Q^T), sums into LDS;
+//   softmax  wave w takes queries 2 w and 2 w + 1 (32 lanes each, two keys per lane): running maximum, weights as two bf16 terms and the
+//            factor of the sums so far into LDS;
+//   sums     wave w adds the columns 16 (w + 8 n) .. + 15 of the latent: O^T += C^T P^T, C^T through the transposing LDS read.
 // The rows of the next 64 keys are in flight in registers meanwhile.
-constexpr int KEYS = 64, SB_PITCH = KEYS + 4;
+constexpr int KEYS = 64, SB_PITCH = KEYS + 4, P_PITCH = KEYS * 2 + 16, MFMA_WAVES = 8, MFMA_THREADS = 64 * MFMA_WAVES;
+constexpr int MFMA_SMALL_LDS = 2 * 16 * SB_PITCH * 4 + 2 * 16 * P_PITCH + 2 * 16 * 4;      // scores, weights, factors and sums
 template <int NT, int PC>
-__global__ __launch_bounds__(256) void latent_mfma_kernel(NcLatentGeom g, const bf16_t* __restrict__ q_lat, const bf16_t* __restrict__ cache,
-                                                          const int32_t* __restrict__ seqlens, bf16_t* __restrict__ out, float* __restrict__ partials,
-                                                          int splits, int groups) {
+__global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom g, const bf16_t* __restrict__ q_lat, const bf16_t* __restrict__ cache,
+                                                                   const int32_t* __restrict__ seqlens, bf16_t* __restrict__ out,
+                                                                   float* __restrict__ partials, int splits, int groups) {
     extern __shared__ __align__(16) uint8_t lds[];
     const int rw = g.rank_p + g.rot_p, pitch = rw * 2 + 16, pieces = rw / 32;
     uint8_t* const lds_q = lds + KEYS * pitch;
-    float* const sb = (float*)(lds_q + 16 * pitch);
+    float* const sb = (float*)(lds_q + 16 * pitch);                                    // [half of the row][query][key]
+    uint8_t* const pb = (uint8_t*)(sb + 2 * 16 * SB_PITCH);                            // [hi, lo][query][key] bf16
+    float* const factor = (float*)(pb + 2 * 16 * P_PITCH);                             // [query]: of the sums so far
+    float* const sums = factor + 16;                                                   // [query]: of the weights, at the end
     const int group = (int)blockIdx.x % groups, split = (int)blockIdx.x / groups, b = blockIdx.y;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int col = lane & 15, quad = lane >> 4;
+    const int col = lane & 15, quad = lane >> 4, ktile = wave & 3, half = wave >> 2;
     const int rows = g.T * g.heads, r0 = group * 16;
-    const int r = min(r0 + col, rows - 1);
     const int pos0 = seqlens[b];
-    const int limit = pos0 + r / g.heads;                                              // last key this lane's query sees
     const int per = ((g.pos_max + g.T + KEYS - 1) / KEYS + splits - 1) / splits * KEYS;
     const int k_begin = split * per;
     const int k_end = min(min(k_begin + per, pos0 + min(r0 + 15, rows - 1) / g.heads + 1), g.Tmax);      // exclusive
     const bf16_t* const keys = cache + (int64_t)b * g.Tmax * rw;
     const float scale2 = g.scale * LOG2E;
 
-    {   // the queries: thread = (row, piece of 16 bytes)
-        const int qr = tid >> 4, qp = tid & 15;
-        const bf16_t* src = q_lat + ((int64_t)b * rows + min(r0 + qr, rows - 1)) * rw;
-        for (int c = qp; c < rw / 8; c += 16) *(uint4*)(lds_q + qr * pitch + c * 16) = *(const uint4*)(src + c * 8);
-    }
-    // 64 cached rows are one contiguous run of memory, 256 pieces of 16 bytes at a time; `put` is where this thread's pieces go in LDS
+    // 64 cached rows are one contiguous run of memory, 512 pieces of 16 bytes at a time; `put` is where this thread's pieces go in LDS
+    const int total = KEYS * 4 * pieces;
     uint4 rk[PC];
     int put[PC];
 #pragma unroll
     for (int i = 0; i < PC; i++) {
-        const int idx = tid + 256 * i;
-        put[i] = idx / (4 * pieces) * pitch + idx % (4 * pieces) * 16;
+        const int idx = tid + MFMA_THREADS * i;
+        put[i] = idx < total ? idx / (4 * pieces) * pitch + idx % (4 * pieces) * 16 : -1;
     }
     auto fetch = [&](int kb) {
         const bf16_t* src = keys + (int64_t)kb * rw;
         const int last = (k_end - kb) * 4 * pieces - 1;          // pieces past the last key re-read its last one (weight zero)
 #pragma unroll
         for (int i = 0; i < PC; i++)
-            if (i < pieces) rk[i] = nt_load16(src + min(tid + 256 * i, last) * 8);
+            if (MFMA_THREADS * i < total) rk[i] = nt_load16(src + min(tid + MFMA_THREADS * i, last) * 8);
     };
+    if (k_begin < k_end) fetch(k_begin);
+    {   // the queries: thread = (row, piece of 16 bytes)
+        const int qr = tid >> 5, qp = tid & 31;
+        const bf16_t* src = q_lat + ((int64_t)b * rows + min(r0 + qr, rows - 1)) * rw;
+        for (int c = qp; c < rw / 8; c += 32) *(uint4*)(lds_q + qr * pitch + c * 16) = *(const uint4*)(src + c * 8);
+    }
     v4f acc[NT];
 #pragma unroll
     for (int n = 0; n < NT; n++) acc[n] = v4f{0.f, 0.f, 0.f, 0.f};
+    // softmax: this lane's query row, its last visible key, and its two keys of a block
+    const int srow = 2 * wave + (lane >> 5), skey = 2 * (lane & 31);
+    const int limit = pos0 + min(r0 + srow, rows - 1) / g.heads;
     float m_run = LA_M_FLOOR, l_run = 0.f;
-    const int ntiles = g.rank_p / 64;
+    const int ntiles = g.rank_p / 16;
     const lds_u8_t tr = (lds_u8_t)lds + (8 * quad + (col >> 2)) * pitch + (16 * wave + 4 * (lane & 3)) * 2;
+    const int c_begin = half ? (pieces + 1) / 2 : 0, c_end = half ? pieces : (pieces + 1) / 2;
+    const uint8_t* const kp = lds + (16 * ktile + col) * pitch + quad * 16;
+    const uint8_t* const qp = lds_q + col * pitch + quad * 16;
 
-    if (k_begin < k_end) fetch(k_begin);
     for (int kb = k_begin; kb < k_end; kb += KEYS) {
-        __syncthreads();                    // everyone is done with the previous keys
+        __syncthreads();                    // everyone is done with the previous keys and weights
 #pragma unroll
         for (int i = 0; i < PC; i++)
-            if (i < pieces) *(uint4*)(lds + put[i]) = rk[i];
+            if (MFMA_THREADS * i < total && put[i] >= 0) *(uint4*)(lds + put[i]) = rk[i];
         __syncthreads();
         if (kb + KEYS < k_end) fetch(kb + KEYS);
-        v4f s0 = v4f{0.f, 0.f, 0.f, 0.f}, s1 = s0;
-        const uint8_t* kp = lds + (16 * wave + col) * pitch + quad * 16;
-        const uint8_t* qp = lds_q + col * pitch + quad * 16;
-        int c = 0;
-        for (; c + 2 <= pieces; c += 2) {
-            s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_v8bf(*(const uint4*)(kp + c * 64)), as_v8bf(*(const uint4*)(qp + c * 64)), s0, 0, 0, 0);
-            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_v8bf(*(const uint4*)(kp + c * 64 + 64)), as_v8bf(*(const uint4*)(qp + c * 64 + 64)), s1, 0, 0, 0);
+        v4f s[2] = {v4f{0.f, 0.f, 0.f, 0.f}, v4f{0.f, 0.f, 0.f, 0.f}};
+        int c = c_begin;
+        for (; c + 4 <= c_end; c += 4) {
+            v8bf kf[4], qf[4];
+#pragma unroll
+            for (int u = 0; u < 4; u++) kf[u] = as_v8bf(*(const uint4*)(kp + (c + u) * 64)), qf[u] = as_v8bf(*(const uint4*)(qp + (c + u) * 64));
+#pragma unroll
+            for (int u = 0; u < 4; u++) s[u & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[u], qf[u], s[u & 1], 0, 0, 0);
         }
-        if (c < pieces)
-            s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_v8bf(*(const uint4*)(kp + c * 64)), as_v8bf(*(const uint4*)(qp + c * 64)), s0, 0, 0, 0);
-        s0 = (s0 + s1) * scale2;
-        *(v4f*)(sb + col * SB_PITCH + 16 * wave + 4 * quad) = s0;
+        for (; c < c_end; c++)
+            s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_v8bf(*(const uint4*)(kp + c * 64)), as_v8bf(*(const uint4*)(qp + c * 64)), s[0], 0, 0, 0);
+        *(v4f*)(sb + (16 * half + col) * SB_PITCH + 16 * ktile + 4 * quad) = (s[0] + s[1]) * scale2;
         __syncthreads();
-        float p[16], mx = LA_MASKED;
-#pragma unroll
-        for (int h = 0; h < 4; h++) {
-            const v4f v = *(const v4f*)(sb + col * SB_PITCH + 32 * (h >> 1) + 8 * quad + 4 * (h & 1));
-#pragma unroll
-            for (int j = 0; j < 4; j++) {
-                const int key = kb + 32 * (h >> 1) + 8 * quad + 4 * (h & 1) + j;
-                p[4 * h + j] = key <= limit && key < k_end ? v[j] : LA_MASKED;
-                mx = fmaxf(mx, p[4 * h + j]);
-            }
+        {
+            const float2 s0 = *(const float2*)(sb + srow * SB_PITCH + skey), s1 = *(const float2*)(sb + (16 + srow) * SB_PITCH + skey);
+            const int key = kb + skey, last = min(limit, k_end - 1);
+            const float pa = key <= last ? s0.x + s1.x : LA_MASKED, pc = key + 1 <= last ? s0.y + s1.y : LA_MASKED;
+            float mx = fmaxf(pa, pc);
+            mx = fmaxf(mx, dpp_f32<0x128>(mx));
+            mx = fmaxf(mx, dpp_f32<0x124>(mx));
+            mx = fmaxf(mx, dpp_f32<0x122>(mx));
+            mx = fmaxf(mx, dpp_f32<0x121>(mx));
+            mx = fmaxf(mx, __shfl_xor(mx, 16));
+            const float m_new = fmaxf(m_run, mx), corr = __builtin_amdgcn_exp2f(m_run - m_new);
+            const float wa = __builtin_amdgcn_exp2f(pa - m_new), wc = __builtin_amdgcn_exp2f(pc - m_new);
+            m_run = m_new;
+            l_run = l_run * corr + (wa + wc);
+            const uint32_t hi = pack_bf16(wa, wc);
+            *(uint32_t*)(pb + srow * P_PITCH + skey * 2) = hi;
+            *(uint32_t*)(pb + (16 + srow) * P_PITCH + skey * 2) = pack_bf16(wa - bf16_lo(hi), wc - bf16_hi(hi));
+            if ((lane & 31) == 0) factor[srow] = corr;
         }
-        mx = fmaxf(mx, __shfl_xor(mx, 16));
-        mx = fmaxf(mx, __shfl_xor(mx, 32));
-        const float m_new = fmaxf(m_run, mx), corr = __builtin_amdgcn_exp2f(m_run - m_new);
-        m_run = m_new;
-        l_run *= corr;
+        __syncthreads();
+        const float corr = factor[col];
         v8bf hi[2], lo[2];
 #pragma unroll
-        for (int j = 0; j < 16; j++) {
-            const float w = __builtin_amdgcn_exp2f(p[j] - m_new);
-            l_run += w;
-            __bf16 h, l;
-            split_bf16(w, h, l);
-            hi[j >> 3][j & 7] = h, lo[j >> 3][j & 7] = l;
+        for (int h = 0; h < 2; h++) {
+            hi[h] = as_v8bf(*(const uint4*)(pb + col * P_PITCH + (32 * h + 8 * quad) * 2));
+            lo[h] = as_v8bf(*(const uint4*)(pb + (16 + col) * P_PITCH + (32 * h + 8 * quad) * 2));
         }
 #pragma unroll
-        for (int n = 0; n < NT; n++) {
-            if (n >= ntiles) break;
-            acc[n] *= corr;
-#pragma unroll
-            for (int h = 0; h < 2; h++) {
-                const v8bf cf = tr_read8(tr + 32 * h * pitch + 128 * n, 4 * pitch);
-                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, hi[h], acc[n], 0, 0, 0);
-                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, lo[h], acc[n], 0, 0, 0);
+        for (int n = 0; n < NT; n++)
+            if (wave + MFMA_WAVES * n < ntiles) {
+                acc[n] *= corr;
+                const v8bf c0 = tr_read8(tr + 256 * n, 4 * pitch), c1 = tr_read8(tr + 32 * pitch + 256 * n, 4 * pitch);
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, hi[0], acc[n], 0, 0, 0);
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, lo[0], acc[n], 0, 0, 0);
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c1, hi[1], acc[n], 0, 0, 0);
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c1, lo[1], acc[n], 0, 0, 0);
             }
+    }
+    l_run = row16_sum(l_run);
+    l_run += __shfl_xor(l_run, 16);
+    if ((lane & 31) == 0) {
+        sums[srow] = l_run;
+        if (splits > 1 && r0 + srow < rows) {
+            float* part = partials + (((int64_t)b * rows + r0 + srow) * splits + split) * (g.rank_p + 4);
+            part[0] = m_run, part[1] = l_run;
         }
     }
-    float l_tot = l_run + __shfl_xor(l_run, 16);
-    l_tot += __shfl_xor(l_tot, 32);
+    __syncthreads();
     if (r0 + col >= rows) return;
-    const int64_t row = (int64_t)b * rows + r;
-    if (splits == 1) {
-        const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
+    const int64_t row = (int64_t)b * rows + r0 + col;
+    const float inv = sums[col] > 0.f ? 1.0f / sums[col] : 0.f;
+    float* part = partials + (row * splits + split) * (g.rank_p + 4) + 4;
 #pragma unroll
-        for (int n = 0; n < NT; n++)
-            if (n < ntiles) st4_f32(out + row * g.rank_p + 16 * (wave + 4 * n) + 4 * quad, acc[n] * inv);
-    } else {
-        float* part = partials + (row * splits + split) * (g.rank_p + 4);
-        if (wave == 0 && quad == 0) part[0] = m_run, part[1] = l_tot;
-#pragma unroll
-        for (int n = 0; n < NT; n++)
-            if (n < ntiles) *(v4f*)(part + 4 + 16 * (wave + 4 * n) + 4 * quad) = acc[n];
-    }
+    for (int n = 0; n < NT; n++)
+        if (wave + MFMA_WAVES * n < ntiles) {
+            const int c = 16 * (wave + MFMA_WAVES * n) + 4 * quad;
+            if (splits == 1) st4_f32(out + row * g.rank_p + c, acc[n] * inv);
+            else *(v4f*)(part + c) = acc[n];
+        }
 }
 
 constexpr int MAX_SPLITS = 64;
@@ -491,15 +508,14 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(2, 2)))
 // the matrix-core kernel's variant for these sizes (0: none), and how many workgroups share the keys of 16 query rows
 int mfma_lds_bytes(const NcLatentGeom& g) {
     const int pitch = (g.rank_p + g.rot_p) * 2 + 16;
-    return (KEYS + 16) * pitch + 16 * SB_PITCH * 4;
+    return (KEYS + 16) * pitch + MFMA_SMALL_LDS;
 }
 int mfma_variant(int dtype, const NcLatentGeom& g) {
     const int pieces = (g.rank_p + g.rot_p) / 32;
     if (dtype != 0 || mfma_lds_bytes(g) > 160 * 1024) return 0;
-    if (g.rank_p <= 64 && pieces <= 6) return 1;
-    if (g.rank_p <= 128 && pieces <= 8) return 2;
-    if (g.rank_p <= 256 && pieces <= 12) return 4;
-    if (g.rank_p <= 512 && pieces <= 20) return 8;
+    if (g.rank_p <= 128 && pieces <= 8) return 1;
+    if (g.rank_p <= 256 && pieces <= 12) return 2;
+    if (g.rank_p <= 512 && pieces <= 20) return 4;
     return 0;
 }
 int mfma_splits(const NcLatentGeom& g) {
@@ -509,16 +525,21 @@ int mfma_splits(const NcLatentGeom& g) {
     if (splits > blocks) splits = blocks;
     return splits < 1 ? 1 : splits > MAX_SPLITS ? MAX_SPLITS : splits;
 }
-int reserve_lds(const void* fn, int bytes) {
-    if (bytes > 64 * 1024 && hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess)
+int reserve_lds(const void* fn, int bytes, std::atomic<uint64_t>& done) {
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev > 63) dev = 0;
+    if (bytes <= 64 * 1024 || (done.load(std::memory_order_relaxed) >> dev & 1)) return 0;
+    if (hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess)
         NC_FAIL(-2, "latent attention: %d bytes of LDS refused", bytes);
+    done.fetch_or(1ull << dev, std::memory_order_relaxed);
     return 0;
 }
 template <int NT, int PC>
 int launch_mfma(const NcLatentGeom& g, const bf16_t* q, const bf16_t* cache, const int32_t* seqlens, bf16_t* out, float* partials, int splits, hipStream_t s) {
     const int groups = (g.T * g.heads + 15) / 16, bytes = mfma_lds_bytes(g);
-    if (int rc = reserve_lds((const void*)latent_mfma_kernel<NT, PC>, bytes)) return rc;
-    hipLaunchKernelGGL((latent_mfma_kernel<NT, PC>), dim3(groups * splits, g.B), dim3(256), bytes, s, g, q, cache, seqlens, out, partials, splits, groups);
+    static std::atomic<uint64_t> done{0};
+    if (int rc = reserve_lds((const void*)latent_mfma_kernel<NT, PC>, bytes, done)) return rc;
+    hipLaunchKernelGGL((latent_mfma_kernel<NT, PC>), dim3(groups * splits, g.B), dim3(MFMA_THREADS), bytes, s, g, q, cache, seqlens, out, partials, splits, groups);
     NC_CHECK_LAUNCH("latent_mfma");
     return 0;
 }
@@ -570,10 +591,9 @@ int nc_launch_latent_attention(int dtype, const NcLatentGeom& g, const void* q_l
         const bf16_t *q = (const bf16_t*)q_lat, *c = (const bf16_t*)cache;
         bf16_t* o = (bf16_t*)out_lat;
         float* p = (float*)partials;
-        int rc = variant == 1   ? launch_mfma<1, 6>(g, q, c, seqlens, o, p, splits, s)
-                 : variant == 2 ? launch_mfma<2, 8>(g, q, c, seqlens, o, p, splits, s)
-                 : variant == 4 ? launch_mfma<4, 12>(g, q, c, seqlens, o, p, splits, s)
-                                : launch_mfma<8, 20>(g, q, c, seqlens, o, p, splits, s);
+        const int rc = variant == 1   ? launch_mfma<1, 4>(g, q, c, seqlens, o, p, splits, s)
+                       : variant == 2 ? launch_mfma<2, 6>(g, q, c, seqlens, o, p, splits, s)
+                                      : launch_mfma<4, 10>(g, q, c, seqlens, o, p, splits, s);
         if (rc) return rc;
         if (splits > 1) {
             hipLaunchKernelGGL(latent_combine_kernel, dim3(rows), dim3(128), 0, s, p, splits, g.rank_p, o);

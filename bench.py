@@ -1,6 +1,7 @@
 """Decode throughput of the FP8 + KV-cache path on one MI355X, at the headline shape.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W]
+    python bench.py --palilix                 (another workload: the Palilix design beside the GPT, see nanochat_amd/stack_bench.py)
 
 Workload (the headline decode configuration, whatever K and W are): nanochat d26 (n_embd 1664, 13 heads, head_dim 128,
 26 layers, vocab 32768, window pattern SSSL), bf16 weights with FP8 linears, random init seed 2; one prompt of 1792 random
@@ -478,6 +479,9 @@ def main():
     ap.add_argument("--copy-probe-mib", type=int, default=0,
                     help="after the decode steps, run an elementwise pass that reads and writes this many MiB "
                          "(a kernel of known traffic to scale hardware byte counters with)")
+    ap.add_argument("--palilix", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the Palilix design at widths 2048 and 4096, "
+                         "beside the FP8 GPT of equal width and layers, every kind of kernel against its roofline")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (decode would shard by batch row, one independent copy per GPU). "
@@ -489,6 +493,14 @@ def main():
     device = torch.device("cuda:0")
     torch.cuda.set_device(device)
 
+    if args.palilix:
+        from nanochat_amd import stack_bench
+        r = stack_bench.run(device)
+        print(json.dumps({"metric": "palilix decode tokens/sec @ width 2048, 8 layers, bs64 ctx2048", "unit": "tokens/s", "n_gpus": 1,
+                          "value": r["width 2048"]["palilix"]["decode"][64]["tokens_per_s"], "higher_is_better": True, "vs_baseline": None,
+                          "dtype": "bf16 (linears, latents), fp32 (residual, scores, states)", "data": "synthetic: random token ids, random weights",
+                          "config": {"context": stack_bench.CONTEXT, "prefill_tokens": list(stack_bench.PREFILL)}, "results": r}))
+        return
     K, W = args.steps, max(1, args.warmup)
     assert 1 <= K and W + K + 1 <= NEW_TOKENS, f"warmup + steps must leave at least one of the {NEW_TOKENS} new tokens for the profiled steps"
     P = max(1, min(args.profile_steps, NEW_TOKENS - W - K))       # what the 256 new tokens leave room for

@@ -150,15 +150,16 @@ __global__ __launch_bounds__(256) void latent_simple_kernel(NcLatentGeom g, cons
 }
 
 // ------------------------------------------------------------------------------------------------ latent space, matrix cores
-// A workgroup of eight waves takes 16 query rows (row = token * heads + head of one batch row) and a share of the keys, 64 keys at a time
+// A workgroup of eight waves takes 16 query rows (row = token * heads + head of one batch row) and a share of the keys, 32 keys at a time
 // through LDS:
-//   scores   wave w multiplies keys 16 (w % 4) .. + 15 with all 16 queries over one half of the row (S^T = K Q^T), sums into LDS;
-//   softmax  wave w takes queries 2 w and 2 w + 1 (32 lanes each, two keys per lane): running maximum, weights as two bf16 terms and the
-//            factor of the sums so far into LDS;
+//   scores   wave w multiplies keys 16 (w % 2) .. + 15 with all 16 queries over one quarter of the row (S^T = K Q^T), sums into LDS;
+//   softmax  wave w takes queries 2 w and 2 w + 1 (32 lanes each, lane = key): running maximum, weights as two bf16 terms and the factor
+//            of the sums so far into LDS;
 //   sums     wave w adds the columns 16 (w + 8 n) .. + 15 of the latent: O^T += C^T P^T, C^T through the transposing LDS read.
-// The rows of the next 64 keys are in flight in registers meanwhile.
-constexpr int KEYS = 64, SB_PITCH = KEYS + 4, P_PITCH = KEYS * 2 + 16, MFMA_WAVES = 8, MFMA_THREADS = 64 * MFMA_WAVES;
-constexpr int MFMA_SMALL_LDS = 2 * 16 * SB_PITCH * 4 + 2 * 16 * P_PITCH + 2 * 16 * 4;      // scores, weights, factors and sums
+// The rows of the next 32 keys are in flight in registers meanwhile, and two workgroups share a compute unit: a block is a chain of short
+// phases with a barrier behind each, and one workgroup works while the other waits.
+constexpr int KEYS = 32, SB_PITCH = KEYS + 4, P_PITCH = KEYS * 2 + 16, MFMA_WAVES = 8, MFMA_THREADS = 64 * MFMA_WAVES;
+constexpr int MFMA_SMALL_LDS = 4 * 16 * SB_PITCH * 4 + 2 * 16 * P_PITCH + 2 * 16 * 4;      // scores, weights, factors and sums
 template <int NT, int PC>
 __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom g, const bf16_t* __restrict__ q_lat, const bf16_t* __restrict__ cache,
                                                                    const int32_t* __restrict__ seqlens, bf16_t* __restrict__ out,
@@ -166,13 +167,17 @@ __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom 
     extern __shared__ __align__(16) uint8_t lds[];
     const int rw = g.rank_p + g.rot_p, pitch = rw * 2 + 16, pieces = rw / 32;
     uint8_t* const lds_q = lds + KEYS * pitch;
-    float* const sb = (float*)(lds_q + 16 * pitch);                                    // [half of the row][query][key]
-    uint8_t* const pb = (uint8_t*)(sb + 2 * 16 * SB_PITCH);                            // [hi, lo][query][key] bf16
+    float* const sb = (float*)(lds_q + 16 * pitch);                                    // [quarter of the row][query][key]
+    uint8_t* const pb = (uint8_t*)(sb + 4 * 16 * SB_PITCH);                            // [hi, lo][query][key] bf16
     float* const factor = (float*)(pb + 2 * 16 * P_PITCH);                             // [query]: of the sums so far
     float* const sums = factor + 16;                                                   // [query]: of the weights, at the end
-    const int group = (int)blockIdx.x % groups, split = (int)blockIdx.x / groups, b = blockIdx.y;
+    // workgroups that read the same keys for other query rows follow each other on one XCD (dealt in turn by the linear index), so that
+    // the keys come out of its L2 the second time
+    const int slot = (int)blockIdx.x >> 3, group = slot % groups, unit = slot / groups * 8 + ((int)blockIdx.x & 7);
+    const int b = unit / splits, split = unit % splits;
+    if (b >= g.B) return;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int col = lane & 15, quad = lane >> 4, ktile = wave & 3, half = wave >> 2;
+    const int col = lane & 15, quad = lane >> 4, ktile = wave & 1, quarter = wave >> 1;
     const int rows = g.T * g.heads, r0 = group * 16;
     const int pos0 = seqlens[b];
     const int per = ((g.pos_max + g.T + KEYS - 1) / KEYS + splits - 1) / splits * KEYS;
@@ -181,7 +186,7 @@ __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom 
     const bf16_t* const keys = cache + (int64_t)b * g.Tmax * rw;
     const float scale2 = g.scale * LOG2E;
 
-    // 64 cached rows are one contiguous run of memory, 512 pieces of 16 bytes at a time; `put` is where this thread's pieces go in LDS
+    // 32 cached rows are one contiguous run of memory, 512 pieces of 16 bytes at a time; `put` is where this thread's pieces go in LDS
     const int total = KEYS * 4 * pieces;
     uint4 rk[PC];
     int put[PC];
@@ -195,7 +200,10 @@ __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom 
         const int last = (k_end - kb) * 4 * pieces - 1;          // pieces past the last key re-read its last one (weight zero)
 #pragma unroll
         for (int i = 0; i < PC; i++)
-            if (MFMA_THREADS * i < total) rk[i] = nt_load16(src + min(tid + MFMA_THREADS * i, last) * 8);
+            if (MFMA_THREADS * i < total) {
+                const bf16_t* piece = src + min(tid + MFMA_THREADS * i, last) * 8;
+                rk[i] = groups == 1 ? nt_load16(piece) : *(const uint4*)piece;
+            }
     };
     if (k_begin < k_end) fetch(k_begin);
     {   // the queries: thread = (row, piece of 16 bytes)
@@ -206,13 +214,13 @@ __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom 
     v4f acc[NT];
 #pragma unroll
     for (int n = 0; n < NT; n++) acc[n] = v4f{0.f, 0.f, 0.f, 0.f};
-    // softmax: this lane's query row, its last visible key, and its two keys of a block
-    const int srow = 2 * wave + (lane >> 5), skey = 2 * (lane & 31);
+    // softmax: this lane's query row, its last visible key, and its key of a block
+    const int srow = 2 * wave + (lane >> 5), skey = lane & 31;
     const int limit = pos0 + min(r0 + srow, rows - 1) / g.heads;
     float m_run = LA_M_FLOOR, l_run = 0.f;
     const int ntiles = g.rank_p / 16;
     const lds_u8_t tr = (lds_u8_t)lds + (8 * quad + (col >> 2)) * pitch + (16 * wave + 4 * (lane & 3)) * 2;
-    const int c_begin = half ? (pieces + 1) / 2 : 0, c_end = half ? pieces : (pieces + 1) / 2;
+    const int c_begin = pieces * quarter / 4, c_end = pieces * (quarter + 1) / 4;
     const uint8_t* const kp = lds + (16 * ktile + col) * pitch + quad * 16;
     const uint8_t* const qp = lds_q + col * pitch + quad * 16;
 
@@ -234,44 +242,37 @@ __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom 
         }
         for (; c < c_end; c++)
             s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_v8bf(*(const uint4*)(kp + c * 64)), as_v8bf(*(const uint4*)(qp + c * 64)), s[0], 0, 0, 0);
-        *(v4f*)(sb + (16 * half + col) * SB_PITCH + 16 * ktile + 4 * quad) = (s[0] + s[1]) * scale2;
+        *(v4f*)(sb + (16 * quarter + col) * SB_PITCH + 16 * ktile + 4 * quad) = (s[0] + s[1]) * scale2;
         __syncthreads();
         {
-            const float2 s0 = *(const float2*)(sb + srow * SB_PITCH + skey), s1 = *(const float2*)(sb + (16 + srow) * SB_PITCH + skey);
-            const int key = kb + skey, last = min(limit, k_end - 1);
-            const float pa = key <= last ? s0.x + s1.x : LA_MASKED, pc = key + 1 <= last ? s0.y + s1.y : LA_MASKED;
-            float mx = fmaxf(pa, pc);
+            const float* sp = sb + srow * SB_PITCH + skey;
+            const float sum = (sp[0] + sp[16 * SB_PITCH]) + (sp[32 * SB_PITCH] + sp[48 * SB_PITCH]);
+            const float sc = kb + skey <= min(limit, k_end - 1) ? sum : LA_MASKED;
+            float mx = sc;
             mx = fmaxf(mx, dpp_f32<0x128>(mx));
             mx = fmaxf(mx, dpp_f32<0x124>(mx));
             mx = fmaxf(mx, dpp_f32<0x122>(mx));
             mx = fmaxf(mx, dpp_f32<0x121>(mx));
             mx = fmaxf(mx, __shfl_xor(mx, 16));
             const float m_new = fmaxf(m_run, mx), corr = __builtin_amdgcn_exp2f(m_run - m_new);
-            const float wa = __builtin_amdgcn_exp2f(pa - m_new), wc = __builtin_amdgcn_exp2f(pc - m_new);
+            const float w = __builtin_amdgcn_exp2f(sc - m_new);
             m_run = m_new;
-            l_run = l_run * corr + (wa + wc);
-            const uint32_t hi = pack_bf16(wa, wc);
-            *(uint32_t*)(pb + srow * P_PITCH + skey * 2) = hi;
-            *(uint32_t*)(pb + (16 + srow) * P_PITCH + skey * 2) = pack_bf16(wa - bf16_lo(hi), wc - bf16_hi(hi));
+            l_run = l_run * corr + w;
+            const bf16_t hi = f32_to_bf16(w);
+            *(bf16_t*)(pb + srow * P_PITCH + skey * 2) = hi;
+            *(bf16_t*)(pb + (16 + srow) * P_PITCH + skey * 2) = f32_to_bf16(w - bf16_to_f32(hi));
             if ((lane & 31) == 0) factor[srow] = corr;
         }
         __syncthreads();
         const float corr = factor[col];
-        v8bf hi[2], lo[2];
-#pragma unroll
-        for (int h = 0; h < 2; h++) {
-            hi[h] = as_v8bf(*(const uint4*)(pb + col * P_PITCH + (32 * h + 8 * quad) * 2));
-            lo[h] = as_v8bf(*(const uint4*)(pb + (16 + col) * P_PITCH + (32 * h + 8 * quad) * 2));
-        }
+        const v8bf hi = as_v8bf(*(const uint4*)(pb + col * P_PITCH + 16 * quad)), lo = as_v8bf(*(const uint4*)(pb + (16 + col) * P_PITCH + 16 * quad));
 #pragma unroll
         for (int n = 0; n < NT; n++)
             if (wave + MFMA_WAVES * n < ntiles) {
+                const v8bf c0 = tr_read8(tr + 256 * n, 4 * pitch);
                 acc[n] *= corr;
-                const v8bf c0 = tr_read8(tr + 256 * n, 4 * pitch), c1 = tr_read8(tr + 32 * pitch + 256 * n, 4 * pitch);
-                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, hi[0], acc[n], 0, 0, 0);
-                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, lo[0], acc[n], 0, 0, 0);
-                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c1, hi[1], acc[n], 0, 0, 0);
-                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c1, lo[1], acc[n], 0, 0, 0);
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, hi, acc[n], 0, 0, 0);
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, lo, acc[n], 0, 0, 0);
             }
     }
     l_run = row16_sum(l_run);
@@ -297,13 +298,13 @@ __global__ __launch_bounds__(MFMA_THREADS) void latent_mfma_kernel(NcLatentGeom 
         }
 }
 
-constexpr int MAX_SPLITS = 64;
+constexpr int MAX_SPLITS = 32;
 __global__ __launch_bounds__(128) void latent_combine_kernel(const float* __restrict__ partials, int splits, int rank_p, bf16_t* __restrict__ out) {
-    __shared__ float weight[MAX_SPLITS];
+    __shared__ float weight[64];
     const int64_t row = blockIdx.x;
     const int stride = rank_p + 4;
     const float* part = partials + row * splits * stride;
-    if (threadIdx.x < 64) {                     // lane = split
+    if (threadIdx.x < 64) {                     // lane = split (MAX_SPLITS <= 64)
         const bool in = (int)threadIdx.x < splits;
         const float m = in ? part[(int64_t)threadIdx.x * stride] : LA_M_FLOOR, l = in ? part[(int64_t)threadIdx.x * stride + 1] : 0.f;
         const float w = __builtin_amdgcn_exp2f(m - wave_max(m));
@@ -520,8 +521,9 @@ int mfma_variant(int dtype, const NcLatentGeom& g) {
 }
 int mfma_splits(const NcLatentGeom& g) {
     const int groups = (g.T * g.heads + 15) / 16, blocks = (g.pos_max + g.T + KEYS - 1) / KEYS;
-    // one workgroup per compute unit (their LDS holds one): all of them start and end together
-    int splits = nc_cu_count() / (g.B * groups);
+    // two workgroups per compute unit (what their LDS holds): all of them start and end together.  More than 32 shares cost more to merge
+    // than they save (2016 keys, 16 heads: 17 us with 24 or 32 shares of one row's keys, 19 with 64)
+    int splits = 2 * nc_cu_count() / (g.B * groups);
     if (splits > blocks) splits = blocks;
     return splits < 1 ? 1 : splits > MAX_SPLITS ? MAX_SPLITS : splits;
 }
@@ -539,7 +541,7 @@ int launch_mfma(const NcLatentGeom& g, const bf16_t* q, const bf16_t* cache, con
     const int groups = (g.T * g.heads + 15) / 16, bytes = mfma_lds_bytes(g);
     static std::atomic<uint64_t> done{0};
     if (int rc = reserve_lds((const void*)latent_mfma_kernel<NT, PC>, bytes, done)) return rc;
-    hipLaunchKernelGGL((latent_mfma_kernel<NT, PC>), dim3(groups * splits, g.B), dim3(MFMA_THREADS), bytes, s, g, q, cache, seqlens, out, partials, splits, groups);
+    hipLaunchKernelGGL((latent_mfma_kernel<NT, PC>), dim3((splits * g.B + 7) / 8 * 8 * groups), dim3(MFMA_THREADS), bytes, s, g, q, cache, seqlens, out, partials, splits, groups);
     NC_CHECK_LAUNCH("latent_mfma");
     return 0;
 }
@@ -591,9 +593,9 @@ int nc_launch_latent_attention(int dtype, const NcLatentGeom& g, const void* q_l
         const bf16_t *q = (const bf16_t*)q_lat, *c = (const bf16_t*)cache;
         bf16_t* o = (bf16_t*)out_lat;
         float* p = (float*)partials;
-        const int rc = variant == 1   ? launch_mfma<1, 4>(g, q, c, seqlens, o, p, splits, s)
-                       : variant == 2 ? launch_mfma<2, 6>(g, q, c, seqlens, o, p, splits, s)
-                                      : launch_mfma<4, 10>(g, q, c, seqlens, o, p, splits, s);
+        const int rc = variant == 1   ? launch_mfma<1, 2>(g, q, c, seqlens, o, p, splits, s)
+                       : variant == 2 ? launch_mfma<2, 3>(g, q, c, seqlens, o, p, splits, s)
+                                      : launch_mfma<4, 5>(g, q, c, seqlens, o, p, splits, s);
         if (rc) return rc;
         if (splits > 1) {
             hipLaunchKernelGGL(latent_combine_kernel, dim3(rows), dim3(128), 0, s, p, splits, g.rank_p, o);

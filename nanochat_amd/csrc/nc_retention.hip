@@ -452,8 +452,9 @@ int nc_launch_retention(int dtype, const NcRetentionGeom& g, const void* proj, i
         return dtype ? launch_step<float>(g, (const float*)proj, ldp, decay, rope, rope_len, seqlens, state_in, state_out, eps, (float*)out, ldo, s)
                      : launch_step<bf16_t>(g, (const bf16_t*)proj, ldp, decay, rope, rope_len, seqlens, state_in, state_out, eps, (bf16_t*)out, ldo, s);
     }
-    // state update and read-out 4 dim vdim flops per token and head, plus the pairs inside a chunk
-    NcProfScope prof(NC_CLS_RETENTION, (double)g.B * g.heads * g.T * (4.0 * g.dim * g.vdim + (double)C * (g.dim + g.vdim)), s, g.T);
+    // bytes: the projections in, the outputs, and four passes over the chunks' states (written, scanned in and out, read)
+    NcProfScope prof(NC_CLS_RETENTION, (double)g.B * g.heads * (g.T * (2.0 * g.dim_p + 3.0 * g.vdim_p) * 2 + 16.0 * ((g.T + C - 1) / C) * g.dim_p * g.vdim_p), s,
+                     g.T);
     const bf16_t* p = (const bf16_t*)proj;
     bf16_t* o = (bf16_t*)out;
 #define CHUNKED(K, V, CC) \

@@ -33,17 +33,14 @@ template <> struct Mma<float> {
     }
 };
 
-// The same pair of fragments (32 bytes of K per lane), accumulated in place and kept in program order against every memory operation: the
-// builtin lets the register allocator pick another result tuple, which it repairs with copies in every K-step, and nothing would keep
-// the LDS reads of a step in front of the barrier that ends it. 
+// One instruction of the same, accumulated in place and kept in program order against every memory operation: the builtin lets the register
+// allocator pick another result tuple, which it repairs with copies in every K-step, and nothing would keep the LDS reads of a step in
+// front of the barrier that ends it.  PARTS instructions make up 16 bytes; the caller puts other accumulators between them.
+template <typename T> constexpr int MMA_PARTS = sizeof(T) == 2 ? 1 : 4;
 template <typename T>
-__device__ __forceinline__ void mma_in_place(v4f& acc, const v4i& w, const v4i& a) {
-    if constexpr (sizeof(T) == 2) {
-        asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+a"(acc) : "v"(w), "v"(a) : "memory");
-    } else {
-#pragma unroll
-        for (int j = 0; j < 4; j++) asm volatile("v_mfma_f32_16x16x4_f32 %0, %1, %2, %0" : "+a"(acc) : "v"(w[j]), "v"(a[j]) : "memory");
-    }
+__device__ __forceinline__ void mma_in_place(v4f& acc, const v4i& w, const v4i& a, int part) {
+    if constexpr (sizeof(T) == 2) asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+a"(acc) : "v"(w), "v"(a) : "memory");
+    else asm volatile("v_mfma_f32_16x16x4_f32 %0, %1, %2, %0" : "+a"(acc) : "v"(w[part]), "v"(a[part]) : "memory");
 }
 
 // four consecutive columns n .. n+3 (n a multiple of 4, all in one segment) of output row `row`
@@ -286,9 +283,13 @@ __global__ __launch_bounds__(64 * WM * WN) void linear_tiled_kernel(NcLinear g, 
                 wh[(j + 1) & 1] = *(const v4i*)(w + (j + 1) * 2048 + rd_hi);
             }
 #pragma unroll
-            for (int i = 0; i < WTM; i++) mma_in_place<T>(acc[i][j], wl[j & 1], al[i]);
+            for (int p = 0; p < MMA_PARTS<T>; p++)
 #pragma unroll
-            for (int i = 0; i < WTM; i++) mma_in_place<T>(acc[i][j], wh[j & 1], ah[i]);
+                for (int i = 0; i < WTM; i++) mma_in_place<T>(acc[i][j], wl[j & 1], al[i], p);
+#pragma unroll
+            for (int p = 0; p < MMA_PARTS<T>; p++)
+#pragma unroll
+                for (int i = 0; i < WTM; i++) mma_in_place<T>(acc[i][j], wh[j & 1], ah[i], p);
         }
         meet();
         cur = cur + 1 == STAGES ? 0 : cur + 1;

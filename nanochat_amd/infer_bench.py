@@ -5,6 +5,7 @@ what the architecture costs, and -- as the very last line of stdout -- one JSON 
 
     python -m nanochat_amd.infer_bench --depth 26                      # random weights of the d26 shape
     python -m nanochat_amd.infer_bench --checkpoint-dir DIR [--step N] # a nanochat checkpoint
+    python -m nanochat_amd.infer_bench --model DIR [--dtype float32]   # any folder the model registry knows (config.json)
 
 Accounting follows the reference (scripts/infer_bench.py:51-53,130-138,215-222): a decode step moves the stored
 weights plus batch * kv_read_bytes(context_mid); MBU is that over the median step time over the peak bandwidth;
@@ -33,6 +34,9 @@ def weight_bytes(model):
 def streamed_weight_bytes(model):
     """What a decode step reads: e4m3 payloads of the FP8 linears, bf16 for the remaining small matrices.  Embedding
     tables are gathered (a few rows per step) and not counted."""
+    own = getattr(model, "streamed_weight_bytes", None)          # a model with another plan counts for itself
+    if own is not None:
+        return own()
     from .fp8 import Float8Linear
     fp8 = {id(m.weight) for m in model._fp8_modules() if isinstance(m, Float8Linear)}
     total = 0
@@ -96,6 +100,8 @@ def bench_generate(engine, prompt_tokens, batch_size, decode_tokens, temperature
 def main(argv=None):
     ap = argparse.ArgumentParser(description="Inference benchmark (MI355X, FP8 linears, KV-cache decode)")
     ap.add_argument("--checkpoint-dir", type=str, default=None, help="nanochat checkpoint directory (model_*.pt, meta_*.json)")
+    ap.add_argument("--model", type=str, default=None, help="folder of a model with a config.json (the registry chooses the class)")
+    ap.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16", help="storage type of a --model")
     ap.add_argument("-s", "--step", type=int, default=None, help="checkpoint step (default: last)")
     ap.add_argument("--depth", type=int, default=26, help="without a checkpoint: random weights of this depth")
     ap.add_argument("--window-pattern", type=str, default="SSSL")
@@ -112,9 +118,9 @@ def main(argv=None):
     device = torch.device("cuda:0")
     torch.cuda.set_device(device)
 
-    if args.checkpoint_dir:
-        from .checkpoint import build_model
-        model, meta = build_model(args.checkpoint_dir, args.step, device)
+    if args.checkpoint_dir or args.model:
+        from .registry import load_model
+        model, meta = load_model(args.model or args.checkpoint_dir, getattr(torch, args.dtype), device, step=args.step)
         source, step, model_config = "checkpoint", meta.get("step"), meta["model_config"]
     else:
         cfg = config_for_depth(args.depth, window_pattern=args.window_pattern, n_kv_head=args.n_kv_head)
@@ -137,14 +143,16 @@ def main(argv=None):
 
     bar = "=" * 100
     print(bar)
-    print(f"Model: {source} | depth {config.n_layer}, dim {config.n_embd}, heads {config.n_head}, kv heads {config.n_kv_head}")
+    shape = model.describe() if hasattr(model, "describe") else (f"depth {config.n_layer}, dim {config.n_embd}, heads {config.n_head}, "
+                                                                 f"kv heads {config.n_kv_head}")
+    print(f"Model: {source} | {shape}")
     print(f"GPU: {device_name} | peak bandwidth {peak_bw / 1e12:.2f} TB/s | peak compute {peak_flops / 1e12:.0f} TFLOPS "
           f"(fp8 dense {PEAK_FP8_FLOPS / 1e12:.0f}) | VRAM {total_vram / 2**30:.0f} GiB")
     param_dtypes = ", ".join(f"{n:,} {name}" for name, n in sorted(card["param_dtypes"].items()))
     print(f"Parameters: {card['num_params']:,} ({param_dtypes}) | weight bytes as stored: {w_bytes / 2**20:.0f} MiB | streamed per "
-          f"decode step {w_stream / 2**20:.0f} MiB (e4m3 linears)")
-    print(f"KV cache: {card['kv_bytes_per_token']:,} bytes/token stored | {kv_read:,} bytes read/step at context {context_mid} "
-          f"(window pattern {config.window_pattern})")
+          f"decode step {w_stream / 2**20:.0f} MiB")
+    print(f"KV cache: {card['kv_bytes_per_token']:,} bytes/token stored | {kv_read:,} bytes read/step at context {context_mid}"
+          + (f" (window pattern {config.window_pattern})" if hasattr(config, "window_pattern") else ""))
     print(f"Theoretical decode ceiling at batch 1: {card['ceiling_bs1_tok_per_sec']:,.0f} tok/s ({card['ceiling_bs1_streamed_tok_per_sec']:,.0f} "
           f"on the bytes really streamed) | max ~{card['max_full_context_rows']:,} full-context rows in VRAM")
     print(bar)

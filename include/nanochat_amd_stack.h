@@ -104,7 +104,7 @@ int nc_stack_forward(const nc_stack_model* model /*host*/, const nc_stack_cache*
 
 /* out[M,N] (T, leading dimension ldc) = A[M,K] W[N,K]^T; kind 0 plain, 1 tanh-form gelu, 2 clamped GLU of interleaved (gate, up)
  * columns (N/2 outputs), 3 float output.  kernel: 0 choose, 1 the few-rows kernel, 2 the tiled kernel,
- * 3 .. 6 the tiled kernel with tiles of 64 x 128, 128 x 128, 256 x 256, 128 x 256.  K a multiple of 64, N of 16. */
+ * 3, 4 the tiled kernel with tiles of 64 x 128, 128 x 256.  K a multiple of 64, N of 16. */
 int nc_stack_linear(int dtype, const void* a, int64_t lda, const void* w, void* out, int ldc, int M, int N, int K, int kind, float limit,
                     int kernel, nc_stream_t stream);
 

@@ -283,7 +283,7 @@ extern "C" int nc_stack_forward(const nc_stack_model* m, const nc_stack_cache* k
 
 extern "C" int nc_stack_linear(int dtype, const void* a, int64_t lda, const void* w, void* out, int ldc, int M, int N, int K, int kind, float limit,
                                int kernel, nc_stream_t stream) {
-    NC_CHECK_ARG(out && kind >= 0 && kind <= 3 && N % 16 == 0 && kernel >= 0 && kernel <= 6, "stack_linear: kind %d, N %d", kind, N);
+    NC_CHECK_ARG(out && kind >= 0 && kind <= 3 && N % 16 == 0 && kernel >= 0 && kernel <= 4, "stack_linear: kind %d, N %d", kind, N);
     NcLinear l = nc_linear(a, lda, w, M, N, K);
     nc_linear_seg(l, N, kind, out, ldc, limit);
     if (kernel == 0) return run_linear(dtype, l, (hipStream_t)stream);

@@ -6,7 +6,7 @@
 //
 //   linear_few_kernel    up to 64 rows (decode): the weight is streamed once, K is dealt to the four waves of a workgroup (and, where a
 //                        consumer adds partial sums, to several workgroups); no LDS in the loop.
-//   linear_tiled_kernel  more rows: BM x 128 tiles, operands straight into a ring of four LDS stages.
+//   linear_tiled_kernel  more rows: 64 x 128 or 128 x 256 tiles, operands straight into a ring of three LDS stages.
 //
 // A stacked weight is several matrices that read the same input; the epilogue sends each run of output columns its own way (store,
 // gelu, clamped GLU, router logits, residual add, soft-capped logits).  Rows can be grouped by weight (experts).
@@ -365,13 +365,11 @@ int launch_tiled(const NcLinear& l, hipStream_t s) {
     NC_CHECK_LAUNCH("linear_tiled");
     return 0;
 }
-// tile shapes: 1 = 64 x 128, 2 = 128 x 128, 3 = 256 x 256, 4 = 128 x 256
+// tile shapes: 1 = 64 x 128 (two workgroups per compute unit), 2 = 128 x 256.  Measured and not kept: 128 x 128 in two stages (711 to 848
+// TFLOP/s where 128 x 256 has 833 to 870), 256 x 256 in two stages (598 to 690).
 template <typename T>
 int launch_tiled_shape(const NcLinear& l, int shape, hipStream_t s) {
-    if (shape == 1) return launch_tiled<T, 64, 128, 2, 2, 3>(l, s);
-    if (shape == 2) return launch_tiled<T, 128, 128, 2, 2, 2>(l, s);
-    if (shape == 3) return launch_tiled<T, 256, 256, 4, 2, 2>(l, s);
-    return launch_tiled<T, 128, 256, 2, 4, 3>(l, s);
+    return shape == 1 ? launch_tiled<T, 64, 128, 2, 2, 3>(l, s) : launch_tiled<T, 128, 256, 2, 4, 3>(l, s);
 }
 
 double linear_units(const NcLinear& l, int dtype, bool few) {
@@ -405,8 +403,8 @@ int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls,
         // the widest tile unless it leaves compute units without one (measured at 1792 rows: 858 against 679 TFLOP/s at N = 12352, 551
         // against 717 at N = 2048, where the launch has 112 or 448 tiles)
         const int64_t wide = (int64_t)((l.M + 127) / 128) * ((l.N + 255) / 256) * l.batch;
-        shape = l.tiles ? (l.tile_rows == 64 ? 1 : 4) : wide < 200 ? 1 : 4;
+        shape = l.tiles ? (l.tile_rows == 64 ? 1 : 2) : wide < 200 ? 1 : 2;
     }
-    if (l.tiles) NC_CHECK_ARG(l.tile_rows == (shape == 1 ? 64 : shape == 3 ? 256 : 128), "linear: group tiles of %d rows", l.tile_rows);
+    if (l.tiles) NC_CHECK_ARG(l.tile_rows == (shape == 1 ? 64 : 128), "linear: group tiles of %d rows", l.tile_rows);
     return dtype ? launch_tiled_shape<float>(l, shape, s) : launch_tiled_shape<bf16_t>(l, shape, s);
 }

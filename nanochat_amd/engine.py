@@ -4,6 +4,7 @@
 Device work (model forward, sampling on GPU logits) goes to the HIP kernels; this file is host logic:
 cache bookkeeping, the per-row tool-use state machine and the streaming generator protocol.
 """
+import ctypes
 import signal
 import warnings
 from collections import deque
@@ -202,6 +203,7 @@ class StackCache(SequenceCache):
         # (zeros: the positions past a row's end enter products with weight zero, and must be finite there)
         self.latents = [torch.zeros(batch_size, seq_len, w, device=device, dtype=dtype) for w in latent_widths]
         self.states = [[torch.zeros(batch_size, *s, device=device, dtype=torch.float32) for s in state_shapes] for _ in range(2)]
+        self._pointers = None
         self._current = 0                          # which of the two state buffers holds the states
         self._host_pos = [0] * batch_size
         self._last_tokens = 0                      # tokens of the last forward, which is the one rewind() can take back
@@ -225,6 +227,13 @@ class StackCache(SequenceCache):
     def state_buffers(self):
         """(states to read, states to write) of the next forward."""
         return self.states[self._current], self.states[self._current ^ 1]
+
+    def pointers(self):
+        """Arrays of device pointers: latents, states to read, states to write (the tensors of a cache never move)."""
+        if self._pointers is None:
+            lat, a, b = ((ctypes.c_void_p * max(1, len(ts)))(*(t.data_ptr() for t in ts)) for ts in (self.latents, *self.states))
+            self._pointers = ((lat, a, b), (lat, b, a))
+        return self._pointers[self._current]
 
     def _moved(self, num_tokens):
         super()._moved(num_tokens)

@@ -494,7 +494,7 @@ def stack_cache_copy(src, dst, n):
 
 def stack_linear(a, w, kind=0, limit=0.0, kernel=0):
     """a [M, K] w [N, K]^T in the storage type of both, 32-bit sums (nc_stack_linear).  kind: 0 plain, 1 tanh-form gelu, 2 clamped GLU of
-    interleaved (gate, up) rows of w, 3 float output; kernel: 0 choose, 1 the few-rows kernel, 2 the tiled one."""
+    interleaved (gate, up) rows of w, 3 float output; kernel: 0 choose, 1 the few-rows kernel, 2 the tiled one (3, 4: its 64 x 128, 128 x 256 tiles)."""
     _need_cuda(a, w)
     (M, K), N = a.shape, w.shape[0]
     assert w.shape[1] == K and a.dtype == w.dtype and a.is_contiguous() and w.is_contiguous()

@@ -211,13 +211,16 @@ class Experts:
             out |= {f"{name}.gate": (n, width), f"{name}.up": (n, width), f"{name}.down": (width, n)}
         return out
 
+    def stacked(self):
+        """{name of one parameter: the tensors it holds, one per expert}."""
+        return {f"experts.{part}": [f"e{i}.{part}" for i in range(self.experts)] for part in ("gate", "up", "down")}
+
     def pack(self, w, width_p):
         router = padded(w["router"], self.router_cols, width_p)
         e1 = torch.empty(self.experts, 2 * self.expert_ff_p, width_p, dtype=router.dtype, device=router.device)
-        e2 = torch.empty(self.experts, width_p, self.expert_ff_p, dtype=router.dtype, device=router.device)
         for i in range(self.experts):
-            e1[i] = interleaved(w[f"e{i}.gate"], w[f"e{i}.up"], self.expert_ff_p, width_p)
-            e2[i] = padded(w[f"e{i}.down"], width_p, self.expert_ff_p)
+            e1[i] = interleaved(w["experts.gate"][i], w["experts.up"][i], self.expert_ff_p, width_p)
+        e2 = padded(w["experts.down"], self.experts, width_p, self.expert_ff_p)
         first = last = None
         if self.shared_ff:
             first = interleaved(w["shared.gate"], w["shared.up"], self.ff_p, width_p)
@@ -281,9 +284,14 @@ class LayerStack(nn.Module):
         self.dtype = dtype
         self.width_p = round_up(config.n_embd, PAD)
         self.run_list = config.runs()
-        # parameters under their tensor names ('.' is not allowed in a parameter's name)
-        self.tensors = nn.ParameterDict({name.replace(".", "/"): nn.Parameter(torch.empty(shape), requires_grad=False)
-                                         for name, shape in self.tensor_shapes(config).items()})
+        # parameters under their tensor names ('.' is not allowed in a parameter's name); an expert layer's tensors of one kind are one
+        # parameter, with one row of it per tensor
+        shapes = self.tensor_shapes(config)
+        self._stacks = {f"l{i}.mlp.{k}": [f"l{i}.mlp.{n}" for n in names] for i, layer in enumerate(config.layers) if isinstance(layer.ff, Experts)
+                        for k, names in layer.ff.stacked().items()}
+        inside = {n for names in self._stacks.values() for n in names}
+        held = {k: s for k, s in shapes.items() if k not in inside} | {k: (len(names), *shapes[names[0]]) for k, names in self._stacks.items()}
+        self.tensors = nn.ParameterDict({k.replace(".", "/"): nn.Parameter(torch.empty(s), requires_grad=False) for k, s in held.items()})
         self._plan = None
         self._plan_key = None
         self._rope = {}
@@ -304,8 +312,16 @@ class LayerStack(nn.Module):
                 out |= {f"l{i}.mlp.{k}": s for k, s in layer.ff.tensors(W).items()}
         return out | {"final.norm": (W,), "head": (config.vocab_size, W)}
 
-    def named_tensors(self):
+    def held_tensors(self):
+        """{name: parameter} as the model holds them (experts of a layer together)."""
         return {k.replace("/", "."): p for k, p in self.tensors.items()}
+
+    def named_tensors(self):
+        """{tensor name: tensor} as in a weight file; an expert's is a view of its layer's parameter."""
+        out = {}
+        for name, p in self.held_tensors().items():
+            out |= dict(zip(self._stacks[name], p.unbind(0))) if name in self._stacks else {name: p}
+        return out
 
     def load_tensors(self, tensors, device):
         """Take the weights by name, in the dtype they come in; names and shapes must be exactly the model's."""
@@ -316,7 +332,9 @@ class LayerStack(nn.Module):
         for name, shape in want.items():
             if tuple(tensors[name].shape) != tuple(shape):
                 raise RuntimeError(f"{name}: shape {tuple(tensors[name].shape)} in the file, {tuple(shape)} in the model")
-            self.tensors[name.replace(".", "/")] = nn.Parameter(tensors[name].to(device), requires_grad=False)
+        for name in self.held_tensors():
+            t = torch.stack([tensors[n] for n in self._stacks[name]]) if name in self._stacks else tensors[name]
+            self.tensors[name.replace(".", "/")] = nn.Parameter(t.to(device), requires_grad=False)
         self.invalidate_plan()
         return self
 
@@ -394,7 +412,7 @@ class LayerStack(nn.Module):
         dev = self.get_device()
         if dev.type != "cuda":
             raise RuntimeError("the layer stack runs on the GPU only: load the model on cuda (there is no CPU fallback)")
-        w = {k: p.detach() for k, p in self.named_tensors().items()}
+        w = {k: p.detach() for k, p in self.held_tensors().items()}
         keep = []
 
         def own(t, dtype):
@@ -493,10 +511,8 @@ class LayerStack(nn.Module):
         n_logits = B * T if rows is None else rows.numel()
         logits = torch.empty(n_logits, self.config.vocab_size, dtype=torch.float32, device=idx.device)
         tap = torch.empty(len(self.run_list), B, T, self.width_p, dtype=torch.float32, device=idx.device) if taps else None
-        state_in, state_out = kv_cache.state_buffers()
-        pointers = [(C.c_void_p * max(1, len(ts)))(*(t.data_ptr() for t in ts)) for ts in (kv_cache.latents, state_in, state_out)]
         cd = _lib.StackCacheDesc()
-        cd.latents, cd.state_in, cd.state_out = pointers
+        cd.latents, cd.state_in, cd.state_out = kv_cache.pointers()
         cd.cache_seqlens = kv_cache.cache_seqlens.data_ptr()
         cd.batch, cd.max_seq_len, cd.pos_max = B, kv_cache.max_seq_len, pos_max
         cd.advance = T if rows is None else 0

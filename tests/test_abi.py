@@ -2,6 +2,7 @@
 import ctypes
 import os
 import re
+from concurrent.futures import ThreadPoolExecutor
 
 from nanochat_amd import _lib
 
@@ -65,10 +66,18 @@ def test_hot_kernels_use_no_scratch_memory():
            "nc_gemm.hip": {"gemm_dl_kernel": 0, "gemm_dlp_kernel": 64},
            "nc_attention_prefill.hip": {"attn_prefill_kernel": 0},
            "nc_quantize.hip": {"amax_kernel": 0, "convert_kernel": 0, "transpose_u8_kernel": 0},
-           "nc_sample.hip": {"sample_kernel": 0}}
-    for src, kernels in hot.items():
+           "nc_sample.hip": {"sample_kernel": 0},
+           "nc_stack_gemm.hip": {"linear_few_kernel": 0, "linear_tiled_kernel": 0},
+           "nc_latent_attention.hip": {"latent_mfma_kernel": 0, "latent_expanded_kernel": 0, "latent_combine_kernel": 0, "latent_append_kernel": 0},
+           "nc_stack_rows.hip": {"stack_row_add_kernel": 0, "route_sort_kernel": 0}}
+
+    def compile_remarks(src):
         cmd = ["hipcc", *nb.FLAGS, "-Rpass-analysis=kernel-resource-usage", "-c", os.path.join(nb.CSRC, src), "-o", os.devnull]
-        r = subprocess.run(cmd, capture_output=True, text=True)
+        return subprocess.run(cmd, capture_output=True, text=True)
+    with ThreadPoolExecutor(max_workers=6) as ex:
+        remarks = dict(zip(hot, ex.map(compile_remarks, hot)))
+    for src, kernels in hot.items():
+        r = remarks[src]
         assert r.returncode == 0, r.stderr[-2000:]
         name, seen = None, set()
         for line in r.stderr.splitlines():

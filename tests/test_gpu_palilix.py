@@ -90,7 +90,7 @@ def test_linear_kernels(dtype, kind):
             want = ref.gelu_tanh(want)
         elif kind == 2:
             want = ref.clamped_glu(want[:, 0::2], want[:, 1::2], 0.6)
-        for kernel in (1, 2, 3, 4, 5, 6):
+        for kernel in (1, 2, 3, 4):
             got = ops.stack_linear(a.to(DEV), w.to(DEV), kind=kind, limit=0.6, kernel=kernel).cpu()
             tol = 1e-2 if got.dtype == torch.bfloat16 else 2e-5
             assert torch.allclose(got.double(), want, rtol=tol, atol=tol), (M, N, K, kernel, (got.double() - want).abs().max().item())

@@ -119,7 +119,10 @@ def test_weight_file_reader(tmp_path):
 def test_weights_must_fit_the_model():
     cfg = CASES["odd"]
     w = weights(cfg)
-    meta_model(cfg).load_tensors(w, "cpu")
+    model = meta_model(cfg).load_tensors(w, "cpu")
+    assert {k: t for k, t in model.named_tensors().items()}.keys() == w.keys()
+    assert all(torch.equal(t, w[k]) for k, t in model.named_tensors().items())
+    assert model.held_tensors()["l0.mlp.experts.down"].shape == (7, cfg["width"], 40)
     for change in (lambda d: d.pop("head"), lambda d: d.update(more=torch.zeros(1)), lambda d: d.update(head=torch.zeros(2, 2))):
         bad = dict(w)
         change(bad)
@@ -158,7 +161,9 @@ def test_packed_matrices_are_the_weights_in_padded_places():
     o = torch.randn(4, ret.heads, ret.vdim, dtype=torch.float64)
     assert torch.allclose(torch.nn.functional.pad(o, (0, ret.vdim_p - ret.vdim)).view(4, -1) @ cols.T, o.view(4, -1) @ m["o"].T)
     ff = sc.layers[0].ff
-    router, first, last, more = ff.pack(ref.sub(w, "l0.mlp."), 128)
+    held = ref.sub(w, "l0.mlp.")
+    held |= {k: torch.stack([held[n] for n in names]) for k, names in ff.stacked().items()}
+    router, first, last, more = ff.pack(held, 128)
     hp = torch.nn.functional.pad(h, (0, 128 - cfg["width"]))
     both = hp @ first.T
     act = ref.clamped_glu(both[:, 0::2], both[:, 1::2], ff.shared_limit)

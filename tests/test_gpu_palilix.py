@@ -128,7 +128,7 @@ MECHANISMS = {
     "latent": mechanism(latent()),
     "latent, peaked scores": mechanism(latent(heads=2, dim=32, rot_dim=32, vdim=32, kv_rank=64, scale=1.5)),
     "retention": mechanism(retention()),
-    "retention, slow decay": mechanism(retention(heads=2, dim=64, vdim=64, rot_dims=32, decay=[0.99951171875, 0.9990234375])),
+    "retention, slow decay": mechanism(retention(heads=2, dim=64, vdim=64, rot_dims=32, decay=[0.9993, 0.9985])),
     "retention, nothing kept and all kept": mechanism(retention(heads=2, dim=64, vdim=64, rot_dims=32, decay=[0.0, 1.0])),
     "dense": mechanism(retention(heads=1, dim=16, vdim=16, rot_dims=8), dense()),
     "experts": mechanism(retention(heads=1, dim=16, vdim=16, rot_dims=8), moe(experts=33, top=5)),
@@ -202,7 +202,7 @@ def test_keys_at_the_borders_of_the_kernels_blocks(dtype):
     """One key stands out for one query: the query's answer is that key's value.  Every place where a block of keys, a portion or a share
     of the keys begins or ends is visited, in prompts, in portions and in decoding."""
     say(f"keys that stand out, {dtype}")
-    cfg = mechanism(latent(heads=2, dim=32, rot_dim=32, vdim=32, kv_rank=64, scale=0.3, base=1e6))
+    cfg = mechanism(latent(heads=2, dim=32, rot_dim=32, vdim=32, kv_rank=64, scale=0.3, base=2e5))
     w = weights(cfg, seed=5)
     # token 0 asks for token 1: their embeddings are opposite, and a query's unrotated part is minus the unrotated key of its own token
     W = cfg["width"]

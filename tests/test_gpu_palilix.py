@@ -407,6 +407,17 @@ def test_greedy_generation_through_the_engine(tmp_path):
     assert runs[0] == runs[1] and len({tuple(r) for r in runs[0]}) > 1
 
 
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_harness_on_a_model_folder(tmp_path, capsys, dtype):
+    say(f"infer_bench --model, {dtype}")
+    from nanochat_amd import infer_bench
+    write_model(tmp_path, CASES["wide"], case_weights("wide"))
+    infer_bench.main(["--model", str(tmp_path), "--dtype", dtype, "--prompt-tokens", "40", "--decode-tokens", "6", "--batch-sizes", "1,3"])
+    card = json.loads(capsys.readouterr().out.strip().splitlines()[-1])
+    assert card["model_config"] == CASES["wide"] and [s["batch_size"] for s in card["sweep"]] == [1, 3]
+    assert card["kv_bytes_per_token"] == (512 + 64) * (2 if dtype == "bfloat16" else 4)
+
+
 class ForcingTokenizer(SyntheticTokenizer):
     """Every sequence meets the tool-use tokens at once: <|python_start|> is whatever the model likes to say, so that the state machine
     forces tokens of its own and the step run ahead is taken back."""

@@ -49,27 +49,38 @@ class CacheDesc(C.Structure):
                 ("shared_prefix", C.c_int), ("uniform_pos", C.c_int), ("advance", C.c_int)]
 
 
+STACK_MAX_MIXERS = 2
+
+
+class StackMixer(C.Structure):
+    _fields_ = ([(n, C.c_int) for n in ("kind", "cols", "out", "heads", "dim", "dim_p", "vdim", "vdim_p", "rot_dim", "rot_p", "rank", "rank_p", "rot_dims")]
+                + [(n, C.c_float) for n in ("score_scale", "out_scale")]
+                + [(n, C.c_int) for n in ("silu_qkv", "gate", "kv_heads", "window", "keep_first", "inner", "inner_p", "state", "state_p", "taps", "dt_rank",
+                                          "dt_rank_p")]
+                + [(n, C.c_void_p) for n in ("kv_norm_w", "w_uk_t", "w_ukv", "decay", "rope", "qkv_bias", "q_norm_w", "k_norm_w", "sink", "out_norm_w", "conv_w",
+                                             "conv_b", "w_x", "w_dt", "w_dt_t", "dt_b", "a_log2", "skip")])
+
+
 class StackLayer(C.Structure):
-    _fields_ = ([(n, C.c_int) for n in ("mixer", "ff", "heads", "dim", "dim_p", "vdim", "vdim_p", "rot_dim", "rot_p", "rank", "rank_p", "rot_dims")]
-                + [("score_scale", C.c_float)]
-                + [(n, C.c_int) for n in ("mix_cols", "router_cols", "ff_cols", "n_in", "mix_out", "ff_p", "k_out")]
+    _fields_ = ([(n, C.c_int) for n in ("block", "n_mixers", "ff", "mix_cols", "router_cols", "ff_cols", "n_in", "mix_out", "ff_p", "k_out")]
                 + [("ff_limit", C.c_float), ("experts", C.c_int), ("top", C.c_int), ("expert_ff_p", C.c_int), ("expert_limit", C.c_float)]
-                + [(n, C.c_void_p) for n in ("norm_w", "w_in", "w_out", "kv_norm_w", "w_uk_t", "w_ukv", "decay", "rope", "w_e1", "w_e2")])
+                + [(n, C.c_void_p) for n in ("norm_w", "norm2_w", "w_in", "w_out", "w_ff_in", "w_ff_out", "w_e1", "w_e2")]
+                + [("mix", StackMixer * STACK_MAX_MIXERS)])
 
 
 class StackRun(C.Structure):
-    _fields_ = [("layer", C.c_int), ("slot", C.c_int), ("add_embedding", C.c_int), ("step", C.c_int)]
+    _fields_ = [("layer", C.c_int), ("slot", C.c_int * STACK_MAX_MIXERS), ("add_embedding", C.c_int), ("step", C.c_int)]
 
 
 class StackModel(C.Structure):
-    _fields_ = ([(n, C.c_int) for n in ("dtype", "width", "width_p", "vocab", "rope_len", "n_layers", "n_runs", "max_k_out")]
+    _fields_ = ([(n, C.c_int) for n in ("dtype", "width", "width_p", "vocab", "rope_len", "n_layers", "n_runs", "max_k_out", "norm")]
                 + [(n, C.c_float) for n in ("eps", "embed_scale", "logit_scale", "logit_softcap")]
                 + [(n, C.c_void_p) for n in ("embed", "head", "final_norm_w", "steps")]
                 + [("layers", C.POINTER(StackLayer)), ("runs", C.POINTER(StackRun))])
 
 
 class StackCacheDesc(C.Structure):
-    _fields_ = [("latents", C.POINTER(C.c_void_p)), ("state_in", C.POINTER(C.c_void_p)), ("state_out", C.POINTER(C.c_void_p)),
+    _fields_ = [("rows", C.POINTER(C.c_void_p)), ("state_in", C.POINTER(C.c_void_p)), ("state_out", C.POINTER(C.c_void_p)),
                 ("cache_seqlens", C.c_void_p), ("batch", C.c_int), ("max_seq_len", C.c_int), ("pos_max", C.c_int), ("advance", C.c_int)]
 
 

@@ -21,7 +21,7 @@ OBJ_DIR = os.path.join(HERE, "_build")
 SOURCES = ["nc_api.hip", "nc_host.hip", "nc_quantize.hip", "nc_gemm.hip", "nc_elementwise.hip", "nc_attention.hip", "nc_attention_prefill.hip",
            "nc_sample.hip", "nc_forward.hip", "nc_profile.hip", "nc_gemm_decode.hip"]
 STACK_SOURCES = ["nc_stack_forward.hip", "nc_host.hip", "nc_stack_gemm.hip", "nc_stack_rows.hip", "nc_latent_attention.hip", "nc_retention.hip",
-                 "nc_profile.hip"]
+                 "nc_window_attention.hip", "nc_selective_scan.hip", "nc_profile.hip"]
 TARGETS = {"gpt": ("libnanochat_amd.so", SOURCES), "stack": ("libnanochat_amd_stack.so", STACK_SOURCES)}
 LIB_PATH = os.path.join(HERE, TARGETS["gpt"][0])
 

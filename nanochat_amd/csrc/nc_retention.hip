@@ -1,6 +1,8 @@
-// Retention: linear attention with one fixed decay per head.  q and k turn with the position, k is scaled, and per head
+// Retention: linear attention with one fixed decay per head.  q and k turn with the position (or not at all), k is scaled, and per head
 //
 //     S_t = decay S_(t-1) + k_t v_t^T   (dim x vdim, fp32),     o_t = S_t^T q_t,     y_t = o_t / rms(o_t) * silu(gate_t)
+//
+// or o_t itself, in fp32, where a design norms all heads together.
 //
 // Two forms:
 //   step     token by token, the state in registers (decode, short portions, 32-bit);
@@ -113,7 +115,9 @@ __global__ __launch_bounds__(NTHR) void retention_step_kernel(NcRetentionGeom g,
             const float ss = wave_sum((y[0] * y[0] + y[1] * y[1]) + (y[2] * y[2] + y[3] * y[3]));
             const float inv = 1.0f / sqrtf(ss / (float)g.vdim + eps);
             const int c = h * g.vdim_p + 4 * tid;
-            if (tid < VG) {
+            if (g.raw) {
+                if (tid < VG) *(v4f*)(g.raw + m * g.heads * g.vdim_p + c) = y;
+            } else if (tid < VG) {
                 const v4f z = ld4_f32(gate + 4 * tid);
                 v4f r;
 #pragma unroll
@@ -166,6 +170,10 @@ __global__ __launch_bounds__(256) void retention_plain_kernel(NcRetentionGeom g,
         }
         const float inv = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)g.vdim + eps);
         for (int c = tid; c < g.vdim_p; c += 256) {
+            if (g.raw) {
+                g.raw[(m * g.heads + h) * g.vdim_p + c] = os[c];
+                continue;
+            }
             const float z = ld_f32(gate + c);
             st_f32(out + m * ldo + h * g.vdim_p + c, os[c] * inv * (z * sigmoid_f32(z)));
         }
@@ -362,6 +370,16 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void r
                 o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, ph[c2], o[d], 0, 0, 0);
                 o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pl[c2], o[d], 0, 0, 0);
             }
+    }
+    if (g.raw) {                               // (uniform)
+        if (i >= n) return;
+        float* row = g.raw + (((int64_t)b * g.T + t0 + i) * g.heads + h) * DV;
+#pragma unroll
+        for (int d = 0; d < NT; d++)
+#pragma unroll
+            for (int g4 = 0; g4 < 4; g4++)
+                *(v4f*)(row + 32 * (vs * NT + d) + 8 * g4 + 4 * hl) = v4f{o[d][4 * g4], o[d][4 * g4 + 1], o[d][4 * g4 + 2], o[d][4 * g4 + 3]};
+        return;
     }
     float ss = 0.f;
 #pragma unroll

@@ -1,0 +1,228 @@
+// Selective scan: a causal convolution per channel, then per channel c and state n a linear recurrence whose step comes from the token,
+//
+//     S[c,n] <- exp(dt_c A[c,n]) S[c,n] + dt_c u_c B_n,     y_c = (sum_n S[c,n] C_n + D_c u_c) silu(z_c)
+//
+// with dt (softplus done by the linear that makes it), B and C per token.  State fp32, kept [state_p + taps - 1][inner_p] per sequence: the
+// recurrent state, then the last inputs of the convolution.  A row at position 0 starts from zero and does not read its state.
+//
+// A channel's states are dealt to LG lanes, SP to each, in registers: lane = part * (64 / LG) + channel, so that neighbours read
+// neighbouring channels.  Tokens go TB at a time: their B and C through LDS (every channel reads the same ones), a lane's own dt, u and z
+// into registers ahead of their use.
+//   one pass    decode and short portions: the tokens one after the other
+//   chunked     long portions: every chunk's own sums from a zero state side by side, a scan over the chunks
+//               S <- exp(A sum dt) S + own sums, then every chunk again from its true start, with outputs
+// A is kept times log2(e), so that a decay is one exp2.
+#include "nc_stack.h"
+
+namespace {
+constexpr int TB = 8;
+enum { SCAN_WHOLE = 0, SCAN_SUMS = 1, SCAN_OUT = 2 };
+
+template <typename T>
+__global__ __launch_bounds__(256) void scan_conv_kernel(NcScanGeom g, const T* __restrict__ x, int ldx, const float* __restrict__ w, const float* __restrict__ bias,
+                                                        const int32_t* __restrict__ seqlens, const float* __restrict__ state_in, float* __restrict__ state_out,
+                                                        T* __restrict__ u) {
+    const int c = 4 * ((int)blockIdx.x * 256 + (int)threadIdx.x), t = blockIdx.y, b = blockIdx.z;
+    if (c >= g.inner_p) return;
+    const int old = g.taps - 1;
+    const bool fresh = seqlens[b] == 0;
+    const int64_t so = ((int64_t)b * (g.state_p + old) + g.state_p) * g.inner_p + c;
+    // input of token tt of this portion; earlier ones come out of the state, oldest first
+    auto input = [&](int tt) -> v4f {
+        if (tt >= 0) return ld4_f32(x + ((int64_t)b * g.T + tt) * ldx + c);
+        if (fresh) return v4f{0.f, 0.f, 0.f, 0.f};
+        return *(const v4f*)(state_in + so + (int64_t)(old + tt) * g.inner_p);
+    };
+    v4f y = v4f{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < g.taps; i++) y += *(const v4f*)(w + (int64_t)i * g.inner_p + c) * input(t - old + i);
+    y += *(const v4f*)(bias + c);
+    st4_f32(u + ((int64_t)b * g.T + t) * g.inner_p + c, v4f{silu_f32(y[0]), silu_f32(y[1]), silu_f32(y[2]), silu_f32(y[3])});
+    if (t == g.T - 1)
+        for (int j = 0; j < old; j++) *(v4f*)(state_out + so + (int64_t)j * g.inner_p) = input(g.T - old + j);
+}
+
+// MODE WHOLE: all tokens from the stored state, outputs, state out.  SUMS: one chunk from zero, its end and its sum of dt into `ends` /
+// `sum_dt`.  OUT: one chunk from its start in `ends`, outputs; the last chunk stores the state.
+template <typename T, int SP, int MODE>
+__global__ __launch_bounds__(256) void scan_kernel(NcScanGeom g, int lg, const T* __restrict__ u, const float* __restrict__ dt, const float* __restrict__ bc,
+                                                   const float* __restrict__ a_log2, const float* __restrict__ skip, const T* __restrict__ z, int ldz,
+                                                   const int32_t* __restrict__ seqlens, const float* __restrict__ state_in, float* __restrict__ state_out,
+                                                   T* __restrict__ out, int ldo, float* __restrict__ ends, float* __restrict__ sum_dt, int chunks, int chunk_len) {
+    extern __shared__ __align__(16) float lds[];            // [TB][2][state_p]: B, C
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, cw = 64 / lg, part = lane / cw;
+    const int c_at = ((int)blockIdx.x * 4 + wave) * cw + lane % cw, c = min(c_at, g.inner_p - 1);
+    const bool mine = c_at < g.inner_p;
+    const int chunk = MODE == SCAN_WHOLE ? 0 : (int)blockIdx.y, b = blockIdx.z;
+    const int t_begin = MODE == SCAN_WHOLE ? 0 : chunk * chunk_len, t_end = MODE == SCAN_WHOLE ? g.T : min(g.T, t_begin + chunk_len);
+    const int64_t row0 = (int64_t)b * g.T, plane = (int64_t)g.state_p * g.inner_p;
+    const int64_t st = (int64_t)b * (g.state_p + g.taps - 1) * g.inner_p + (int64_t)part * SP * g.inner_p + c;
+    const int bc_cols = nc_scan_bc_cols(g.state_p);
+    float a[SP], S[SP];
+#pragma unroll
+    for (int i = 0; i < SP; i++) a[i] = a_log2[(int64_t)(part * SP + i) * g.inner_p + c];
+    if (MODE == SCAN_SUMS || (chunk == 0 && seqlens[b] == 0)) {
+#pragma unroll
+        for (int i = 0; i < SP; i++) S[i] = 0.f;
+    } else {
+        const float* src = MODE == SCAN_OUT && chunk > 0 ? ends + ((int64_t)b * (chunks - 1) + chunk - 1) * plane + (int64_t)part * SP * g.inner_p + c : state_in + st;
+#pragma unroll
+        for (int i = 0; i < SP; i++) S[i] = src[(int64_t)i * g.inner_p];
+    }
+    const float d = MODE == SCAN_SUMS ? 0.f : skip[c];
+    float total = 0.f;
+    for (int t0 = t_begin; t0 < t_end; t0 += TB) {
+        float dv[TB], uv[TB], zv[TB];
+#pragma unroll
+        for (int j = 0; j < TB; j++) {
+            const int64_t row = row0 + min(t0 + j, t_end - 1);
+            dv[j] = dt[row * g.inner_p + c];
+            uv[j] = ld_f32(u + row * g.inner_p + c);
+            zv[j] = MODE == SCAN_SUMS ? 0.f : ld_f32(z + row * ldz + c);
+        }
+        __syncthreads();
+        for (int i = 4 * threadIdx.x; i < TB * 2 * g.state_p; i += 1024) {
+            const int j = i / (2 * g.state_p), k = i % (2 * g.state_p), which = k / g.state_p;
+            *(v4f*)(lds + i) = *(const v4f*)(bc + (row0 + min(t0 + j, t_end - 1)) * 2 * bc_cols + which * bc_cols + k - which * g.state_p);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < TB; j++) {
+            if (t0 + j >= t_end) break;                     // uniform
+            const float* bj = lds + j * 2 * g.state_p + part * SP;
+            const float* cj = bj + g.state_p;
+            const float du = dv[j] * uv[j];
+            float y = 0.f;
+            if (MODE == SCAN_SUMS) total += dv[j];
+#pragma unroll
+            for (int i = 0; i < SP; i += 4) {
+                const v4f bv = *(const v4f*)(bj + i), cv = MODE == SCAN_SUMS ? v4f{0.f, 0.f, 0.f, 0.f} : *(const v4f*)(cj + i);
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    S[i + r] = fmaf(__builtin_amdgcn_exp2f(dv[j] * a[i + r]), S[i + r], du * bv[r]);
+                    if (MODE != SCAN_SUMS) y = fmaf(S[i + r], cv[r], y);
+                }
+            }
+            if (MODE != SCAN_SUMS) {
+                for (int o = cw; o < 64; o <<= 1) y += __shfl_xor(y, o);
+                y = fmaf(d, uv[j], y) * silu_f32(zv[j]) * g.out_scale;
+                if (part == 0 && mine) st_f32(out + (row0 + t0 + j) * ldo + c, y);
+            }
+        }
+    }
+    if (!mine) return;
+    if (MODE == SCAN_SUMS) {
+        float* dst = ends + ((int64_t)b * (chunks - 1) + chunk) * plane + (int64_t)part * SP * g.inner_p + c;
+#pragma unroll
+        for (int i = 0; i < SP; i++) dst[(int64_t)i * g.inner_p] = S[i];
+        if (part == 0) sum_dt[((int64_t)b * (chunks - 1) + chunk) * g.inner_p + c] = total;
+    } else if (MODE == SCAN_WHOLE || chunk == chunks - 1) {
+#pragma unroll
+        for (int i = 0; i < SP; i++) state_out[st + (int64_t)i * g.inner_p] = S[i];
+    }
+}
+
+// Every chunk's end from a zero state becomes the true start of the next chunk, in place.  One thread per four channels of one state.
+__global__ __launch_bounds__(256) void scan_chunks_kernel(NcScanGeom g, const float* __restrict__ a_log2, const int32_t* __restrict__ seqlens,
+                                                          const float* __restrict__ state_in, float* __restrict__ ends, const float* __restrict__ sum_dt, int chunks) {
+    const int c = 4 * ((int)blockIdx.x * 256 + (int)threadIdx.x), n = blockIdx.y, b = blockIdx.z;
+    if (c >= g.inner_p) return;
+    const int64_t plane = (int64_t)g.state_p * g.inner_p;
+    const v4f a = *(const v4f*)(a_log2 + (int64_t)n * g.inner_p + c);
+    v4f S = v4f{0.f, 0.f, 0.f, 0.f};
+    if (seqlens[b] > 0) S = *(const v4f*)(state_in + ((int64_t)b * (g.state_p + g.taps - 1) + n) * g.inner_p + c);
+    float* e = ends + (int64_t)b * (chunks - 1) * plane + (int64_t)n * g.inner_p + c;
+    const float* sd = sum_dt + (int64_t)b * (chunks - 1) * g.inner_p + c;
+    constexpr int AHEAD = 8;
+    for (int k0 = 0; k0 < chunks - 1; k0 += AHEAD) {
+        v4f own[AHEAD], s[AHEAD];
+#pragma unroll
+        for (int j = 0; j < AHEAD; j++) {
+            const int k = min(k0 + j, chunks - 2);
+            own[j] = *(const v4f*)(e + k * plane), s[j] = *(const v4f*)(sd + (int64_t)k * g.inner_p);
+        }
+#pragma unroll
+        for (int j = 0; j < AHEAD; j++) {
+            if (k0 + j >= chunks - 1) break;
+#pragma unroll
+            for (int r = 0; r < 4; r++) S[r] = fmaf(__builtin_amdgcn_exp2f(a[r] * s[j][r]), S[r], own[j][r]);
+            *(v4f*)(e + (k0 + j) * plane) = S;
+        }
+    }
+}
+
+constexpr int CHUNK = 64, CHUNK_MIN_TOKENS = 96;
+int chunk_count(const NcScanGeom& g) { return g.T < CHUNK_MIN_TOKENS ? 1 : (g.T + CHUNK - 1) / CHUNK; }
+// states per lane and lanes per channel (0: not such a size)
+bool lanes_of(int state_p, int& sp, int& lg) {
+    for (int s : {16, 12, 8, 4}) {
+        const int l = state_p / s;
+        if (state_p % s == 0 && (l & (l - 1)) == 0 && l >= 1 && l <= 16) {
+            sp = s, lg = l;
+            return true;
+        }
+    }
+    return false;
+}
+
+template <typename T, int SP>
+int launch_scan(const NcScanGeom& g, int lg, const T* u, const float* dt, const float* bc, const float* a_log2, const float* skip, const T* z, int ldz,
+                const int32_t* seqlens, const float* state_in, float* state_out, T* out, int ldo, void* workspace, hipStream_t s) {
+    const int chunks = chunk_count(g), xs = (g.inner_p + 4 * (64 / lg) - 1) / (4 * (64 / lg)), bytes = TB * 2 * g.state_p * 4;
+    if (chunks == 1) {
+        hipLaunchKernelGGL((scan_kernel<T, SP, SCAN_WHOLE>), dim3(xs, 1, g.B), dim3(256), bytes, s, g, lg, u, dt, bc, a_log2, skip, z, ldz, seqlens, state_in, state_out,
+                           out, ldo, nullptr, nullptr, 1, 0);
+        NC_CHECK_LAUNCH("scan");
+        return 0;
+    }
+    float* ends = (float*)workspace;
+    float* sum_dt = ends + (int64_t)g.B * (chunks - 1) * g.state_p * g.inner_p;
+    hipLaunchKernelGGL((scan_kernel<T, SP, SCAN_SUMS>), dim3(xs, chunks - 1, g.B), dim3(256), bytes, s, g, lg, u, dt, bc, a_log2, skip, z, ldz, seqlens, state_in,
+                       state_out, out, ldo, ends, sum_dt, chunks, CHUNK);
+    hipLaunchKernelGGL(scan_chunks_kernel, dim3((g.inner_p + 1023) / 1024, g.state_p, g.B), dim3(256), 0, s, g, a_log2, seqlens, state_in, ends, sum_dt, chunks);
+    hipLaunchKernelGGL((scan_kernel<T, SP, SCAN_OUT>), dim3(xs, chunks, g.B), dim3(256), bytes, s, g, lg, u, dt, bc, a_log2, skip, z, ldz, seqlens, state_in, state_out,
+                       out, ldo, ends, sum_dt, chunks, CHUNK);
+    NC_CHECK_LAUNCH("scan_chunked");
+    return 0;
+}
+}  // namespace
+
+int nc_launch_scan_conv(int dtype, const NcScanGeom& g, const void* x, int ldx, const float* w, const float* b, const int32_t* seqlens, const float* state_in,
+                        float* state_out, void* u, hipStream_t s) {
+    NC_CHECK_ARG(x && w && b && u && state_in != state_out && g.taps >= 1 && g.inner_p % 4 == 0 && ldx % 4 == 0, "scan_conv: %d taps, %d channels", g.taps, g.inner_p);
+    NC_CHECK_ARG(g.T <= 65535 && g.B <= 65535, "scan_conv: %d tokens in one portion", g.T);
+    NcProfScope prof(NC_CLS_ROWS, (double)g.B * g.T * g.inner_p * (dtype ? 8 : 4), s);
+    const dim3 grid((g.inner_p + 1023) / 1024, g.T, g.B);
+    if (dtype)
+        hipLaunchKernelGGL((scan_conv_kernel<float>), grid, dim3(256), 0, s, g, (const float*)x, ldx, w, b, seqlens, state_in, state_out, (float*)u);
+    else
+        hipLaunchKernelGGL((scan_conv_kernel<bf16_t>), grid, dim3(256), 0, s, g, (const bf16_t*)x, ldx, w, b, seqlens, state_in, state_out, (bf16_t*)u);
+    NC_CHECK_LAUNCH("scan_conv");
+    return 0;
+}
+
+size_t nc_scan_workspace_bytes(const NcScanGeom& g) {
+    const int chunks = chunk_count(g);
+    return chunks > 1 ? (size_t)g.B * (chunks - 1) * (g.state_p + 1) * g.inner_p * sizeof(float) : 0;
+}
+
+int nc_launch_scan(int dtype, const NcScanGeom& g, const void* u, const float* dt, const float* bc, const float* a_log2, const float* skip, const void* z, int ldz,
+                   const int32_t* seqlens, const float* state_in, float* state_out, void* out, int ldo, void* workspace, hipStream_t s) {
+    int sp = 0, lg = 0;
+    NC_CHECK_ARG(lanes_of(g.state_p, sp, lg) && g.state <= g.state_p, "scan: %d states per channel in %d", g.state, g.state_p);
+    NC_CHECK_ARG(u && dt && bc && a_log2 && skip && z && out && state_in != state_out, "scan: null operand");
+    NC_CHECK_ARG(g.T <= 65535 * CHUNK && g.B <= 65535, "scan: %d tokens in one portion", g.T);
+    // state in and out once; per token the projections and the result (bytes)
+    NcProfScope prof(NC_CLS_SCAN, (double)g.B * (8.0 * g.state * g.inner_p + (double)g.T * g.inner_p * (4 + (dtype ? 12 : 6))), s, g.T);
+#define GO(SP)                                                                                                                                           \
+    (dtype ? launch_scan<float, SP>(g, lg, (const float*)u, dt, bc, a_log2, skip, (const float*)z, ldz, seqlens, state_in, state_out, (float*)out, ldo,   \
+                                    workspace, s)                                                                                                         \
+           : launch_scan<bf16_t, SP>(g, lg, (const bf16_t*)u, dt, bc, a_log2, skip, (const bf16_t*)z, ldz, seqlens, state_in, state_out, (bf16_t*)out, ldo, \
+                                     workspace, s))
+    switch (sp) {
+        case 16: return GO(16);
+        case 12: return GO(12);
+        case 8: return GO(8);
+        default: return GO(4);
+    }
+#undef GO
+}

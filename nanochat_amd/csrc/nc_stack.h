@@ -9,7 +9,7 @@
 #include "nc_kernels.h"
 
 // timing classes of NcProfScope / nc_profile_*
-enum { NC_CLS_LATENT = 0, NC_CLS_LINEAR = 1, NC_CLS_RETENTION = 2, NC_CLS_ROWS = 3, NC_CLS_EXPERTS = 4 };
+enum { NC_CLS_LATENT = 0, NC_CLS_LINEAR = 1, NC_CLS_RETENTION = 2, NC_CLS_ROWS = 3, NC_CLS_EXPERTS = 4, NC_CLS_WINDOW = 5, NC_CLS_SCAN = 6 };
 
 // ---------------------------------------------------------------- element helpers
 template <typename T> __device__ __forceinline__ float ld_f32(const T* p);
@@ -30,6 +30,8 @@ __device__ __forceinline__ float gelu_tanh_f32(float z) {
     return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
 // gate and up of one unit -> its activation, both clamped: the gate from above, up on both sides
 __device__ __forceinline__ float clamped_glu_f32(float gate, float up, float limit) {
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
@@ -45,6 +47,9 @@ enum NcSegKind {
     NC_SEG_F32 = 3,        // float
     NC_SEG_RESIDUAL = 4,   // float, added to what is there
     NC_SEG_LOGITS = 5,     // float, p0 * v, then p1 * tanh(. / p1) if p1 > 0; bounds checked column by column
+    NC_SEG_SILU = 6,       // T, silu
+    NC_SEG_SWIGLU = 7,     // T, silu(gate) * up of interleaved columns (gate, up): half as many outputs
+    NC_SEG_SOFTPLUS = 8,   // float, softplus(v + bias)
 };
 struct NcSeg {
     int end;               // exclusive last column (of the stacked weight) of this run
@@ -52,6 +57,7 @@ struct NcSeg {
     void* out;             // output column 0 of the run
     int ld;                // elements between output rows
     float p0, p1;          // GLU: p0 = limit
+    const float* bias;     // SOFTPLUS: per output column of the run
 };
 // The rows a linear works on: M rows of A; or, per batch, the same M with strides; or groups of rows, one group per weight (experts).
 struct NcLinear {
@@ -79,8 +85,8 @@ inline NcLinear nc_linear(const void* a, int64_t lda, const void* w, int M, int 
     l.a = a, l.lda = lda, l.w = w, l.M = M, l.N = N, l.K = K, l.batch = 1, l.a_div = 1, l.splits = 1;
     return l;
 }
-inline void nc_linear_seg(NcLinear& l, int end, int kind, void* out, int ld, float p0 = 0.f, float p1 = 0.f) {
-    l.seg[l.nseg++] = NcSeg{end, kind, out, ld, p0, p1};
+inline void nc_linear_seg(NcLinear& l, int end, int kind, void* out, int ld, float p0 = 0.f, float p1 = 0.f, const float* bias = nullptr) {
+    l.seg[l.nseg++] = NcSeg{end, kind, out, ld, p0, p1, bias};
 }
 #define NC_FEW_ROWS 64                     // up to here the few-rows kernel
 #define NC_TILE_WORDS 5
@@ -91,11 +97,13 @@ int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls 
 int nc_linear_few_splits(int M, int N, int K);
 
 // ---------------------------------------------------------------- row kernels (nc_stack_rows.hip)
-// x = embedding rows * scale (+ step); h = layer_norm(x)
+// What the rows that leave for the next linear are: layer norm or RMS norm of x times a weight, or x itself in the storage type.
+enum NcRowNorm { NC_ROW_LAYER_NORM = 0, NC_ROW_RMS_NORM = 1, NC_ROW_COPY = 2 };
+// x = embedding rows * scale (+ step); h = norm(x)
 int nc_launch_stack_embed(int dtype, const int64_t* idx, const void* embed, float scale, const float* step, int vocab, float* x, float* x0,
-                          const float* norm_w, float eps, void* h, int M, int width, int width_p, hipStream_t s);
-// x += partial sums + weighted expert rows; tap = x; x += x0 + step; h = layer_norm(x).  Rows may be a selection (`rows`: which row of x
-// is normalised into row i of h); then x itself is not stored.
+                          int norm, const float* norm_w, float eps, void* h, int M, int width, int width_p, hipStream_t s);
+// y = partial sums + weighted expert rows; x += y, or (post_norm_w) x += rms_norm(y) * post_norm_w; tap = x; x += x0 + step; h = norm(x).
+// Rows may be a selection (`rows`: which row of x is normalised into row i of h); then x itself is not stored.
 struct NcRowAdd {
     float* x;
     const float* partials;         // [splits][M][width_p] or null
@@ -104,9 +112,11 @@ struct NcRowAdd {
     const int32_t* slot_of;        // [M][top]
     const float* slot_w;           // [M][top]
     int top;
+    const float* post_norm_w;      // or null
     float* tap;                    // [M][width_p] or null
     const float* x0;               // or null
     const float* step;             // or null
+    int norm;                      // NcRowNorm of h
     const float* norm_w;
     void* h;
     const int32_t* rows;           // selection or null
@@ -157,9 +167,44 @@ struct NcRetentionGeom {
     int heads, dim, dim_p, vdim, vdim_p, rot_dims;
     float k_scale;
     int B, T;
+    float* raw;                    // fp32 [B*T][heads * vdim_p]: the heads' outputs as they are go here instead of into `out`; or null
 };
 // proj: q | k | v | gate; out: normed per head, times silu(gate)
 size_t nc_retention_workspace_bytes(int dtype, const NcRetentionGeom& g);
 int nc_launch_retention(int dtype, const NcRetentionGeom& g, const void* proj, int ldp, const float* decay, const float* rope, int rope_len,
                         const int32_t* seqlens, const float* state_in, float* state_out, float eps, void* out, int ldo, void* workspace,
                         hipStream_t s);
+// out = rms_norm(raw row, over `count` values of its `cols`) * w * sigmoid(gate) * scale
+int nc_launch_joint_gate(int dtype, const float* raw, int cols, int count, const void* gate, int ldg, const float* w, float eps, float scale, void* out,
+                         int ldo, int M, hipStream_t s);
+
+// ---------------------------------------------------------------- window attention (nc_window_attention.hip)
+struct NcWindowGeom {
+    int heads, kv_heads, dim, dim_p, vdim_p, rot_dims;
+    int window, keep_first;        // query i sees key j <= i if i - j < window or j < keep_first
+    float scale, out_scale;
+    int B, T, Tmax, pos_max;
+};
+// New tokens: bias, norm over the whole projection, rotation; queries in place, keys and values into the cache.
+int nc_launch_window_append(int dtype, const NcWindowGeom& g, void* proj, int ldp, const float* bias, const float* q_norm_w, const float* k_norm_w, float eps,
+                            const float* rope, int rope_len, const int32_t* seqlens, void* cache, hipStream_t s);
+size_t nc_window_partial_bytes(int dtype, const NcWindowGeom& g);
+int nc_launch_window_attention(int dtype, const NcWindowGeom& g, const void* q, int ldq, const void* cache, const float* sink, const int32_t* seqlens, void* out,
+                               int ldo, void* partials, size_t partial_bytes, hipStream_t s);
+
+// ---------------------------------------------------------------- selective scan (nc_selective_scan.hip)
+struct NcScanGeom {
+    int inner, inner_p, state, state_p, taps, dt_rank_p;
+    float out_scale;
+    int B, T;
+};
+__host__ __device__ inline int nc_scan_bc_cols(int state_p) { return (state_p + 15) / 16 * 16; }      // columns of B (and of C) in the projected rows
+// u = silu(causal convolution of x); the convolution's part of the state moves on
+int nc_launch_scan_conv(int dtype, const NcScanGeom& g, const void* x, int ldx, const float* w, const float* b, const int32_t* seqlens, const float* state_in,
+                        float* state_out, void* u, hipStream_t s);
+// the recurrence and what follows it: out = (sum_n S C + skip u) * silu(z) * scale.  dt fp32 [M][inner_p], bc fp32
+// [M][2 * nc_scan_bc_cols]
+size_t nc_scan_workspace_bytes(const NcScanGeom& g);
+int nc_launch_scan(int dtype, const NcScanGeom& g, const void* u, const float* dt, const float* bc, const float* a_log2, const float* skip,
+                   const void* z, int ldz, const int32_t* seqlens, const float* state_in, float* state_out, void* out, int ldo, void* workspace,
+                   hipStream_t s);

@@ -1,12 +1,16 @@
 // Host-side sequencing of one forward of the layer stack on a stream (include/nanochat_amd_stack.h): one call enqueues every kernel of
 // the step; no host synchronisation, no allocation.
 //
-// Per layer run, h = the normed rows:
+// Per run of a parallel layer, h = the normed rows:
 //   linear   [projections | router logits | first feed-forward matrix] . h    the activation of the feed-forward in the epilogue
-//   mixer    latent attention or retention  -> its part of `cat`; the feed-forward's part is there already
+//   mixer    -> its part of `cat`; the feed-forward's part is there already
 //   experts  route (softmax, choice, expert order), gate and up with their activation, down: one row per (token, choice)
 //   linear   w_out . cat, added to the residual stream: in its epilogue, or (few rows) as partial sums by the row kernel
-//   row add  x += partial sums + weighted expert rows (+ embedding output + step vector at the start of a pass), layer norm -> h
+//   row add  x += partial sums + weighted expert rows (+ embedding output + step vector at the start of a pass), norm -> h
+// Per run of a post-norm layer, h = x in the storage type:
+//   linear   projections . h;  mixers, side by side if there are two  -> `cat`
+//   linear   w_out . cat -> sums in fp32 (few rows: partial ones);  row add  x += norm1(sums) -> h
+//   linear   gate and up . h, activation in the epilogue;  linear  down -> sums;  row add  x += norm2(sums) -> h
 // Few rows (decode): weights are streamed by linear_few_kernel; more rows: the tiled kernel.
 #include "../../include/nanochat_amd_stack.h"
 #include "nc_stack.h"
@@ -31,22 +35,28 @@ struct Carver {
 };
 
 struct Workspace {
-    float *x, *x0, *router, *parts;
-    void *h, *proj, *cat, *h_last, *q_lat, *o_lat, *kv, *att_parts, *ret, *act, *e_out;
+    float *x, *x0, *router, *parts, *raw, *bc, *dt;
+    void *h, *proj, *cat, *h_last, *q_lat, *o_lat, *kv, *att_parts, *ret, *act, *e_out, *u, *dtr;
     float* slot_w;
     int32_t *chosen, *slot_of, *perm, *tiles, *n_tiles;
     size_t att_part_bytes, part_bytes, total;
 };
 
-NcLatentGeom latent_geom(const nc_stack_layer& l, int B, int T, int Tmax, int pos_max) {
+NcLatentGeom latent_geom(const nc_stack_mixer& l, int B, int T, int Tmax, int pos_max) {
     return NcLatentGeom{l.heads, l.dim_p, l.rot_p, l.rot_dims, l.rank, l.rank_p, l.vdim_p, l.score_scale, B, T, Tmax, pos_max};
 }
-NcRetentionGeom retention_geom(const nc_stack_layer& l, int B, int T) {
-    return NcRetentionGeom{l.heads, l.dim, l.dim_p, l.vdim, l.vdim_p, l.rot_dims, l.score_scale, B, T};
+NcRetentionGeom retention_geom(const nc_stack_mixer& l, int B, int T, float* raw) {
+    return NcRetentionGeom{l.heads, l.dim, l.dim_p, l.vdim, l.vdim_p, l.rot_dims, l.score_scale, B, T, raw};
+}
+NcWindowGeom window_geom(const nc_stack_mixer& l, int B, int T, int Tmax, int pos_max) {
+    return NcWindowGeom{l.heads, l.kv_heads, l.dim, l.dim_p, l.vdim_p, l.rot_dims, l.window, l.keep_first, l.score_scale, l.out_scale, B, T, Tmax, pos_max};
+}
+NcScanGeom scan_geom(const nc_stack_mixer& l, int B, int T) {
+    return NcScanGeom{l.inner, l.inner_p, l.state, l.state_p, l.taps, l.dt_rank_p, l.out_scale, B, T};
 }
 // Expanding keys and values costs rank (dim + vdim) per key and head; after that a (query, key) pair costs dim + rot + vdim and only the
 // visible half of the new pairs is visited, against 2 rank + rot in latent space.
-bool expand(int dtype, const nc_stack_layer& l, const NcLatentGeom& g) {
+bool expand(int dtype, const nc_stack_mixer& l, const NcLatentGeom& g) {
     if (!nc_latent_expanded_ok(dtype, g) || g.T < 32) return false;
     return (double)g.T * (2.0 * l.rank_p + l.rot_p - 0.5 * (l.dim_p + l.rot_p + l.vdim_p)) > (double)l.rank_p * (l.dim_p + l.vdim_p);
 }
@@ -62,7 +72,8 @@ size_t max_of(size_t a, size_t b) { return a > b ? a : b; }
 
 Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_keys, void* base) {
     const size_t M = (size_t)B * T, Wp = m->width_p, es = m->dtype ? 4 : 2;
-    size_t proj = 0, router = 0, parts = 0, qlat = 0, olat = 0, kv = 0, att = 0, ret = 0, act = 0, eout = 0, pairs = 0, tiles = 0;
+    size_t proj = 0, router = 0, parts = 0, qlat = 0, olat = 0, kv = 0, att = 0, ret = 0, act = 0, eout = 0, pairs = 0, tiles = 0, raw = 0, bc = 0, dt = 0, u = 0,
+           dtr = 0;
     bool again = false;
     for (int i = 0; i < m->n_runs; i++) again |= m->runs[i].add_embedding != 0;
     for (int i = 0; i < m->n_layers; i++) {
@@ -70,17 +81,37 @@ Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_key
         proj = max_of(proj, M * l.mix_cols * es);
         router = max_of(router, M * l.router_cols * 4);
         if (M <= NC_FEW_ROWS) parts = max_of(parts, (size_t)nc_linear_few_splits((int)M, (int)Wp, l.k_out) * M * Wp * 4);
-        if (l.mixer == NC_MIXER_LATENT_ATTENTION) {
-            const NcLatentGeom g = latent_geom(l, B, T, max_keys, max_keys - T);
-            if (expand(m->dtype, l, g)) {
-                kv = max_of(kv, (size_t)B * max_keys * l.heads * (l.dim_p + l.vdim_p) * es);
-            } else {
-                qlat = max_of(qlat, M * l.heads * (l.rank_p + l.rot_p) * es);
-                olat = max_of(olat, M * l.heads * l.rank_p * es);
-                att = max_of(att, nc_latent_partial_bytes(m->dtype, g));
+        else if (l.block == NC_BLOCK_POST_NORM) parts = max_of(parts, M * Wp * 4);
+        if (l.block == NC_BLOCK_POST_NORM && l.ff) {
+            if (M <= NC_FEW_ROWS) parts = max_of(parts, (size_t)nc_linear_few_splits((int)M, (int)Wp, l.ff_p) * M * Wp * 4);
+            act = max_of(act, M * l.ff_p * es);
+        }
+        for (int j = 0; j < l.n_mixers; j++) {
+            const nc_stack_mixer& x = l.mix[j];
+            switch (x.kind) {
+                case NC_MIXER_LATENT_ATTENTION: {
+                    const NcLatentGeom g = latent_geom(x, B, T, max_keys, max_keys - T);
+                    if (expand(m->dtype, x, g)) {
+                        kv = max_of(kv, (size_t)B * max_keys * x.heads * (x.dim_p + x.vdim_p) * es);
+                    } else {
+                        qlat = max_of(qlat, M * x.heads * (x.rank_p + x.rot_p) * es);
+                        olat = max_of(olat, M * x.heads * x.rank_p * es);
+                        att = max_of(att, nc_latent_partial_bytes(m->dtype, g));
+                    }
+                    break;
+                }
+                case NC_MIXER_RETENTION:
+                    ret = max_of(ret, nc_retention_workspace_bytes(m->dtype, retention_geom(x, B, T, nullptr)));
+                    if (x.gate == NC_GATE_JOINT_NORM_SIGMOID) raw = max_of(raw, M * x.heads * x.vdim_p * 4);
+                    break;
+                case NC_MIXER_WINDOW_ATTENTION:
+                    att = max_of(att, nc_window_partial_bytes(m->dtype, window_geom(x, B, T, max_keys, max_keys - T)));
+                    break;
+                default:
+                    ret = max_of(ret, nc_scan_workspace_bytes(scan_geom(x, B, T)));
+                    u = max_of(u, M * x.inner_p * es), dt = max_of(dt, M * x.inner_p * 4);
+                    dtr = max_of(dtr, M * x.dt_rank_p * es), bc = max_of(bc, M * 2 * nc_scan_bc_cols(x.state_p) * 4);
             }
-        } else {
-            ret = max_of(ret, nc_retention_workspace_bytes(m->dtype, retention_geom(l, B, T)));
         }
         if (l.ff == NC_FF_EXPERTS) {
             const size_t p = M * l.top;
@@ -115,6 +146,11 @@ Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_key
     w.perm = (int32_t*)c.take(pairs * 4);
     w.tiles = (int32_t*)c.take(tiles * NC_TILE_WORDS * 4);
     w.n_tiles = (int32_t*)c.take(4);
+    w.raw = (float*)c.take(raw);
+    w.u = c.take(u);
+    w.dtr = c.take(dtr);
+    w.bc = (float*)c.take(bc);
+    w.dt = (float*)c.take(dt);
     w.total = (c.off + 255) & ~(size_t)255;
     return w;
 }
@@ -126,21 +162,23 @@ int run_linear(int dtype, const NcLinear& l, hipStream_t s) {
     return l.M <= NC_FEW_ROWS || l.K % 64 != 0 ? nc_launch_linear_few(dtype, l, s) : nc_launch_linear_tiled(dtype, l, s);
 }
 
-int run_latent_attention(int dt, const nc_stack_layer& l, const NcLatentGeom& g, const Workspace& w, const float* kv_norm_w, float eps, const float* rope,
-                         int rope_len, const int32_t* seqlens, void* cache, int ld_cat, hipStream_t s) {
+// A mixer reads its columns of the projected rows (`proj`, leading dimension ldp) and writes its columns of what the output matrix multiplies
+// (`cat`, leading dimension ld_cat).
+int run_latent_attention(int dt, const nc_stack_mixer& l, const NcLatentGeom& g, const Workspace& w, void* proj, int ldp, float eps, int rope_len,
+                         const int32_t* seqlens, void* cache, void* cat, int ld_cat, hipStream_t s) {
     const int M = g.B * g.T, qd = l.dim_p + l.rot_p, rw = l.rank_p + l.rot_p, head_w = l.dim_p + l.vdim_p;
     const bool ex = expand(dt, l, g);
-    TRY(nc_launch_latent_append(dt, g, w.proj, l.mix_cols, kv_norm_w, eps, rope, rope_len, seqlens, cache, ex ? nullptr : w.q_lat, s));
+    TRY(nc_launch_latent_append(dt, g, proj, ldp, l.kv_norm_w, eps, l.rope, rope_len, seqlens, cache, ex ? nullptr : w.q_lat, s));
     if (ex) {
         const int keys = g.pos_max + g.T;
         NcLinear e = nc_linear(cache, rw, l.w_ukv, keys, l.heads * head_w, l.rank_p);
         e.batch = g.B, e.a_stride = (int64_t)g.Tmax * rw, e.w_stride = 0, e.out_stride = (int64_t)keys * l.heads * head_w;
         nc_linear_seg(e, e.N, NC_SEG_PLAIN, w.kv, l.heads * head_w);
         TRY(nc_launch_linear_tiled(dt, e, s));
-        return nc_launch_latent_expanded(g, (const bf16_t*)w.proj, l.mix_cols, (const bf16_t*)w.kv, keys, (const bf16_t*)cache, seqlens, (bf16_t*)w.cat, ld_cat, s);
+        return nc_launch_latent_expanded(g, (const bf16_t*)proj, ldp, (const bf16_t*)w.kv, keys, (const bf16_t*)cache, seqlens, (bf16_t*)cat, ld_cat, s);
     }
     // unrotated queries into latent space, one product per head
-    NcLinear q = nc_linear(w.proj, l.mix_cols, l.w_uk_t, M, l.rank_p, l.dim_p);
+    NcLinear q = nc_linear(proj, ldp, l.w_uk_t, M, l.rank_p, l.dim_p);
     q.batch = l.heads, q.a_stride = qd, q.w_stride = (int64_t)l.rank_p * l.dim_p, q.out_stride = rw;
     nc_linear_seg(q, q.N, NC_SEG_PLAIN, w.q_lat, l.heads * rw);
     TRY(run_linear(dt, q, s));
@@ -148,8 +186,81 @@ int run_latent_attention(int dt, const nc_stack_layer& l, const NcLatentGeom& g,
     // ... and the weighted latents out of it: the value rows of w_ukv sit behind the head's dim_p key rows
     NcLinear v = nc_linear(w.o_lat, l.heads * l.rank_p, at(l.w_ukv, (int64_t)l.dim_p * l.rank_p, dt), M, l.vdim_p, l.rank_p);
     v.batch = l.heads, v.a_stride = l.rank_p, v.w_stride = (int64_t)head_w * l.rank_p, v.out_stride = l.vdim_p;
-    nc_linear_seg(v, v.N, NC_SEG_PLAIN, w.cat, ld_cat);
+    nc_linear_seg(v, v.N, NC_SEG_PLAIN, cat, ld_cat);
     return run_linear(dt, v, s);
+}
+
+int run_window_attention(int dt, const nc_stack_mixer& l, const NcWindowGeom& g, const Workspace& w, void* proj, int ldp, float eps, int rope_len,
+                         const int32_t* seqlens, void* cache, void* cat, int ld_cat, hipStream_t s) {
+    TRY(nc_launch_window_append(dt, g, proj, ldp, l.qkv_bias, l.q_norm_w, l.k_norm_w, eps, l.rope, rope_len, seqlens, cache, s));
+    return nc_launch_window_attention(dt, g, proj, ldp, cache, l.sink, seqlens, cat, ld_cat, w.att_parts, w.att_part_bytes, s);
+}
+
+int run_retention(int dt, const nc_stack_mixer& l, const NcRetentionGeom& g, const Workspace& w, const void* proj, int ldp, float eps, int rope_len,
+                  const int32_t* seqlens, const float* state_in, float* state_out, void* cat, int ld_cat, hipStream_t s) {
+    TRY(nc_launch_retention(dt, g, proj, ldp, l.decay, l.rope, rope_len, seqlens, state_in, state_out, eps, cat, ld_cat, w.ret, s));
+    if (!g.raw) return 0;
+    const void* gate = at(proj, (int64_t)l.heads * (2 * l.dim_p + l.vdim_p), dt);
+    return nc_launch_joint_gate(dt, g.raw, l.heads * l.vdim_p, l.heads * l.vdim, gate, ldp, l.out_norm_w, eps, l.out_scale, cat, ld_cat, g.B * g.T, s);
+}
+
+int run_selective_scan(int dt, const nc_stack_mixer& l, const NcScanGeom& g, const Workspace& w, const void* proj, int ldp, const int32_t* seqlens,
+                       const float* state_in, float* state_out, void* cat, int ld_cat, hipStream_t s) {
+    const int M = g.B * g.T, bc = nc_scan_bc_cols(l.state_p);
+    TRY(nc_launch_scan_conv(dt, g, proj, ldp, l.conv_w, l.conv_b, seqlens, state_in, state_out, w.u, s));
+    NcLinear x = nc_linear(w.u, l.inner_p, l.w_x, M, l.dt_rank_p + 2 * bc, l.inner_p);
+    nc_linear_seg(x, l.dt_rank_p, NC_SEG_PLAIN, w.dtr, l.dt_rank_p);
+    nc_linear_seg(x, x.N, NC_SEG_F32, w.bc, 2 * bc);
+    TRY(run_linear(dt, x, s));
+    NcLinear d = nc_linear(w.dtr, l.dt_rank_p, l.w_dt, M, l.inner_p, l.dt_rank_p);
+    nc_linear_seg(d, d.N, NC_SEG_SOFTPLUS, w.dt, l.inner_p, 0.f, 0.f, l.dt_b);
+    TRY(run_linear(dt, d, s));
+    return nc_launch_scan(dt, g, w.u, w.dt, w.bc, l.a_log2, l.skip, at(proj, l.inner_p, dt), ldp, seqlens, state_in, state_out, cat, ld_cat, w.ret, s);
+}
+
+// The mixers of one layer run, on the projected rows w.proj, into w.cat.
+int run_mixers(const nc_stack_model* m, const nc_stack_cache* kv, const nc_stack_run& run, const Workspace& w, int B, int T, hipStream_t s) {
+    const nc_stack_layer& l = m->layers[run.layer];
+    const int dt = m->dtype;
+    int col = 0, to = 0;
+    for (int j = 0; j < l.n_mixers; j++) {
+        const nc_stack_mixer& x = l.mix[j];
+        const int slot = run.slot[j];
+        void *proj = at(w.proj, col, dt), *cat = at(w.cat, to, dt);
+        switch (x.kind) {
+            case NC_MIXER_LATENT_ATTENTION:
+                TRY(run_latent_attention(dt, x, latent_geom(x, B, T, kv->max_seq_len, kv->pos_max), w, proj, l.mix_cols, m->eps, m->rope_len, kv->cache_seqlens,
+                                         kv->rows[slot], cat, l.k_out, s));
+                break;
+            case NC_MIXER_RETENTION:
+                TRY(run_retention(dt, x, retention_geom(x, B, T, x.gate == NC_GATE_JOINT_NORM_SIGMOID ? w.raw : nullptr), w, proj, l.mix_cols, m->eps, m->rope_len,
+                                  kv->cache_seqlens, kv->state_in[slot], kv->state_out[slot], cat, l.k_out, s));
+                break;
+            case NC_MIXER_WINDOW_ATTENTION:
+                TRY(run_window_attention(dt, x, window_geom(x, B, T, kv->max_seq_len, kv->pos_max), w, proj, l.mix_cols, m->eps, m->rope_len, kv->cache_seqlens,
+                                         kv->rows[slot], cat, l.k_out, s));
+                break;
+            default:
+                TRY(run_selective_scan(dt, x, scan_geom(x, B, T), w, proj, l.mix_cols, kv->cache_seqlens, kv->state_in[slot], kv->state_out[slot], cat, l.k_out, s));
+        }
+        col += x.cols, to += x.out;
+    }
+    return 0;
+}
+// The columns of the input matrix that are the mixers' own.
+void mixer_segs(const nc_stack_layer& l, NcLinear& in, const Workspace& w, int dt) {
+    int col = 0;
+    for (int j = 0; j < l.n_mixers; j++) {
+        const nc_stack_mixer& x = l.mix[j];
+        int from = col;
+        if (x.silu_qkv) {
+            const int qkv = x.heads * (2 * x.dim_p + x.vdim_p);
+            nc_linear_seg(in, col + qkv, NC_SEG_SILU, at(w.proj, col, dt), l.mix_cols);
+            from += qkv;
+        }
+        nc_linear_seg(in, col + x.cols, NC_SEG_PLAIN, at(w.proj, from, dt), l.mix_cols);
+        col += x.cols;
+    }
 }
 
 int run_experts(int dt, const nc_stack_layer& l, int M, int width_p, const Workspace& w, hipStream_t s) {
@@ -172,31 +283,79 @@ int run_experts(int dt, const nc_stack_layer& l, int M, int width_p, const Works
     return grouped(down);
 }
 
-int check_layer(const nc_stack_layer& l, int width_p, int i) {
-    NC_CHECK_ARG(l.w_in && l.w_out && l.norm_w && l.rope, "stack: layer %d has no weights", i);
-    NC_CHECK_ARG(l.mix_cols % 16 == 0 && l.router_cols % 16 == 0 && l.ff_cols % 16 == 0 && l.n_in == l.mix_cols + l.router_cols + l.ff_cols,
-                 "stack: layer %d input columns", i);
-    NC_CHECK_ARG(l.mix_out == l.heads * l.vdim_p && l.k_out == l.mix_out + l.ff_p && l.k_out % NC_STACK_PAD == 0 && l.ff_p % NC_STACK_PAD == 0,
-                 "stack: layer %d output columns", i);
-    if (l.mixer == NC_MIXER_LATENT_ATTENTION) {
-        NC_CHECK_ARG(l.kv_norm_w && l.w_uk_t && l.w_ukv, "stack: layer %d has no latent weights", i);
-        NC_CHECK_ARG(l.dim_p % 32 == 0 && l.rot_p % 32 == 0 && l.vdim_p % 16 == 0 && l.rank_p % NC_STACK_PAD == 0 &&
-                         l.mix_cols == l.heads * (l.dim_p + l.rot_p) + l.rank_p + l.rot_p, "stack: layer %d latent sizes", i);
-    } else {
-        NC_CHECK_ARG(l.mixer == NC_MIXER_RETENTION && l.decay, "stack: layer %d mixer", i);
-        NC_CHECK_ARG(l.dim_p % 16 == 0 && l.vdim_p % 16 == 0 && l.mix_cols == 2 * l.heads * (l.dim_p + l.vdim_p), "stack: layer %d retention sizes", i);
+int check_mixer(const nc_stack_mixer& x, int i) {
+    NC_CHECK_ARG(x.cols % 16 == 0 && x.out % 16 == 0 && (x.rope || x.rot_dims == 0), "stack: layer %d mixer columns", i);
+    const bool scales = x.kind == NC_MIXER_WINDOW_ATTENTION || x.kind == NC_MIXER_SELECTIVE_SCAN || (x.kind == NC_MIXER_RETENTION && x.gate);
+    NC_CHECK_ARG(scales || x.out_scale == 1.f, "stack: layer %d: a mixer of this kind does not scale its result", i);
+    if (x.kind != NC_MIXER_SELECTIVE_SCAN) NC_CHECK_ARG(x.out == x.heads * x.vdim_p, "stack: layer %d output columns", i);
+    switch (x.kind) {
+        case NC_MIXER_LATENT_ATTENTION:
+            NC_CHECK_ARG(x.kv_norm_w && x.w_uk_t && x.w_ukv, "stack: layer %d has no latent weights", i);
+            NC_CHECK_ARG(x.dim_p % 32 == 0 && x.rot_p % 32 == 0 && x.vdim_p % 16 == 0 && x.rank_p % NC_STACK_PAD == 0 &&
+                             x.cols == x.heads * (x.dim_p + x.rot_p) + x.rank_p + x.rot_p, "stack: layer %d latent sizes", i);
+            return 0;
+        case NC_MIXER_RETENTION:
+            NC_CHECK_ARG(x.decay && (!x.gate || x.out_norm_w), "stack: layer %d has no retention weights", i);
+            NC_CHECK_ARG(x.dim_p % 16 == 0 && x.vdim_p % 16 == 0 && x.cols == 2 * x.heads * (x.dim_p + x.vdim_p), "stack: layer %d retention sizes", i);
+            return 0;
+        case NC_MIXER_WINDOW_ATTENTION:
+            NC_CHECK_ARG(x.qkv_bias && x.q_norm_w && x.k_norm_w && x.sink, "stack: layer %d has no window attention weights", i);
+            NC_CHECK_ARG(x.kv_heads >= 1 && x.heads % x.kv_heads == 0 && x.dim_p % 32 == 0 && x.vdim_p % 16 == 0 &&
+                             x.cols == (x.heads + x.kv_heads) * x.dim_p + x.kv_heads * x.vdim_p, "stack: layer %d window attention sizes", i);
+            return 0;
+        case NC_MIXER_SELECTIVE_SCAN:
+            NC_CHECK_ARG(x.conv_w && x.conv_b && x.w_x && x.w_dt && x.w_dt_t && x.dt_b && x.a_log2 && x.skip, "stack: layer %d has no scan weights", i);
+            NC_CHECK_ARG(x.inner_p % NC_STACK_PAD == 0 && x.dt_rank_p % NC_STACK_PAD == 0 && x.state_p % 4 == 0 && x.taps >= 1 && x.cols == 2 * x.inner_p &&
+                             x.out == x.inner_p, "stack: layer %d scan sizes", i);
+            return 0;
     }
+    NC_FAIL(-1, "stack: layer %d mixer", i);
+}
+
+int check_layer(const nc_stack_layer& l, int i) {
+    NC_CHECK_ARG(l.w_in && l.w_out && l.norm_w, "stack: layer %d has no weights", i);
+    NC_CHECK_ARG(l.n_mixers >= 1 && l.n_mixers <= NC_STACK_MAX_MIXERS, "stack: layer %d has %d mixers", i, l.n_mixers);
+    int cols = 0, out = 0, segs = 0;
+    for (int j = 0; j < l.n_mixers; j++) {
+        TRY(check_mixer(l.mix[j], i));
+        cols += l.mix[j].cols, out += l.mix[j].out, segs += l.mix[j].silu_qkv ? 2 : 1;
+    }
+    const bool post = l.block == NC_BLOCK_POST_NORM;
+    NC_CHECK_ARG(l.block == NC_BLOCK_PARALLEL || post, "stack: layer %d block", i);
+    NC_CHECK_ARG(cols == l.mix_cols && l.router_cols % 16 == 0 && l.ff_cols % 16 == 0 && l.n_in == l.mix_cols + (post ? 0 : l.router_cols + l.ff_cols),
+                 "stack: layer %d input columns", i);
+    NC_CHECK_ARG(out == l.mix_out && l.k_out == l.mix_out + (post ? 0 : l.ff_p) && l.k_out % NC_STACK_PAD == 0 && l.ff_p % NC_STACK_PAD == 0,
+                 "stack: layer %d output columns", i);
+    NC_CHECK_ARG(segs + (l.router_cols > 0) + (!post && l.ff_cols > 0) <= 4, "stack: layer %d has too many parts", i);
+    const bool dense = l.ff == NC_FF_DENSE_GELU || l.ff == NC_FF_DENSE_SWIGLU;
+    if (post) NC_CHECK_ARG(l.ff == NC_FF_NONE || (dense && l.w_ff_in && l.w_ff_out && l.norm2_w && l.ff_p > 0), "stack: layer %d feed-forward", i);
     if (l.ff == NC_FF_EXPERTS)
         NC_CHECK_ARG(l.w_e1 && l.w_e2 && l.router_cols >= l.experts && l.top >= 1 && l.top <= l.experts && l.expert_ff_p % NC_STACK_PAD == 0 &&
                          l.ff_cols == 2 * l.ff_p, "stack: layer %d expert sizes", i);
     else
-        NC_CHECK_ARG(l.router_cols == 0 && l.ff_cols == l.ff_p && (l.ff == NC_FF_DENSE_GELU || (l.ff == NC_FF_NONE && l.ff_p == 0)), "stack: layer %d feed-forward sizes", i);
-    (void)width_p;
+        NC_CHECK_ARG(l.router_cols == 0 && l.ff_cols == (l.ff == NC_FF_DENSE_SWIGLU ? 2 : 1) * l.ff_p && (dense || (l.ff == NC_FF_NONE && l.ff_p == 0)),
+                     "stack: layer %d feed-forward sizes", i);
     return 0;
+}
+int ff_seg_kind(int ff) { return ff == NC_FF_EXPERTS ? NC_SEG_GLU : ff == NC_FF_DENSE_SWIGLU ? NC_SEG_SWIGLU : NC_SEG_GELU; }
+// how the rows that enter a run's first linear come out of x
+void entry_norm(const nc_stack_model* m, const nc_stack_run& run, int& norm, const float*& w) {
+    const nc_stack_layer& l = m->layers[run.layer];
+    norm = l.block == NC_BLOCK_POST_NORM ? NC_ROW_COPY : m->norm == NC_NORM_RMS ? NC_ROW_RMS_NORM : NC_ROW_LAYER_NORM;
+    w = l.norm_w;
+}
+// sums = W rows, in fp32 for the row kernel: whole, or (few rows) in as many shares as fill the chip
+int run_sums(int dt, const void* a, const void* w, int M, int N, int K, float* parts, NcRowAdd& add, hipStream_t s) {
+    NcLinear l = nc_linear(a, K, w, M, N, K);
+    const int splits = M <= NC_FEW_ROWS ? nc_linear_few_splits(M, N, K) : 1;
+    if (splits > 1) l.partials = parts, l.splits = splits;
+    else nc_linear_seg(l, N, NC_SEG_F32, parts, N);
+    add.partials = parts, add.splits = splits;
+    return run_linear(dt, l, s);
 }
 }  // namespace
 
-extern "C" int nc_stack_abi_version(void) { return 1; }
+extern "C" int nc_stack_abi_version(void) { return 2; }
 
 extern "C" size_t nc_stack_workspace_bytes(const nc_stack_model* m, int B, int T, int n_logits, int max_keys) {
     if (!m || B <= 0 || T <= 0 || max_keys < T) return 0;
@@ -214,7 +373,7 @@ extern "C" int nc_stack_forward(const nc_stack_model* m, const nc_stack_cache* k
     NC_CHECK_ARG(logit_rows || n_logits == 0 || n_logits == B * T, "stack_forward: without a selection all rows have logits");
     NC_CHECK_ARG(!kv->advance || (!logit_rows && n_logits > 0), "stack_forward: the positions are advanced by the pass over all rows");
     NC_CHECK_ARG(((uintptr_t)workspace & 255) == 0, "stack_forward: workspace must be 256-byte aligned");
-    for (int i = 0; i < m->n_layers; i++) TRY(check_layer(m->layers[i], m->width_p, i));
+    for (int i = 0; i < m->n_layers; i++) TRY(check_layer(m->layers[i], i));
     const int M = B * T, Wp = m->width_p, dt = m->dtype;
     const int keys = kv->pos_max + T;
     // the caller sized the workspace for its own bound on the keys; what this call needs is never more than that
@@ -226,42 +385,53 @@ extern "C" int nc_stack_forward(const nc_stack_model* m, const nc_stack_cache* k
         NC_CHECK_ARG(r.layer >= 0 && r.layer < m->n_layers && (r.step < 0 || m->steps), "stack_forward: run %d", i);
         again |= r.add_embedding != 0;
     }
-    const int32_t* pos = kv->cache_seqlens;
-
+    const int final_norm = m->norm == NC_NORM_RMS ? NC_ROW_RMS_NORM : NC_ROW_LAYER_NORM;
+    int norm;
+    const float* norm_w;
+    entry_norm(m, m->runs[0], norm, norm_w);
     TRY(nc_launch_stack_embed(dt, idx, m->embed, m->embed_scale, m->runs[0].step >= 0 ? m->steps + (int64_t)m->runs[0].step * Wp : nullptr, m->vocab, w.x,
-                              again ? w.x0 : nullptr, m->layers[m->runs[0].layer].norm_w, m->eps, w.h, M, m->width, Wp, s));
+                              again ? w.x0 : nullptr, norm, norm_w, m->eps, w.h, M, m->width, Wp, s));
     for (int i = 0; i < m->n_runs; i++) {
         const nc_stack_run& run = m->runs[i];
         const nc_stack_layer& l = m->layers[run.layer];
+        const bool post = l.block == NC_BLOCK_POST_NORM;
         NcLinear in = nc_linear(w.h, Wp, l.w_in, M, l.n_in, Wp);
-        nc_linear_seg(in, l.mix_cols, NC_SEG_PLAIN, w.proj, l.mix_cols);
+        mixer_segs(l, in, w, dt);
         if (l.router_cols) nc_linear_seg(in, l.mix_cols + l.router_cols, NC_SEG_F32, w.router, l.router_cols);
-        if (l.ff_cols)
-            nc_linear_seg(in, l.n_in, l.ff == NC_FF_EXPERTS ? NC_SEG_GLU : NC_SEG_GELU, at(w.cat, l.mix_out, dt), l.k_out, l.ff_limit);
+        if (!post && l.ff_cols) nc_linear_seg(in, l.n_in, ff_seg_kind(l.ff), at(w.cat, l.mix_out, dt), l.k_out, l.ff_limit);
         TRY(run_linear(dt, in, s));
-
-        if (l.mixer == NC_MIXER_LATENT_ATTENTION)
-            TRY(run_latent_attention(dt, l, latent_geom(l, B, T, kv->max_seq_len, kv->pos_max), w, l.kv_norm_w, m->eps, l.rope, m->rope_len, pos,
-                                     kv->latents[run.slot], l.k_out, s));
-        else
-            TRY(nc_launch_retention(dt, retention_geom(l, B, T), w.proj, l.mix_cols, l.decay, l.rope, m->rope_len, pos, kv->state_in[run.slot],
-                                    kv->state_out[run.slot], m->eps, w.cat, l.k_out, w.ret, s));
-        if (l.ff == NC_FF_EXPERTS) TRY(run_experts(dt, l, M, Wp, w, s));
+        TRY(run_mixers(m, kv, run, w, B, T, s));
 
         NcRowAdd add{};
         add.x = w.x, add.tokens_per_row = T;
-        NcLinear out = nc_linear(w.cat, l.k_out, l.w_out, M, Wp, l.k_out);
-        const int splits = M <= NC_FEW_ROWS ? nc_linear_few_splits(M, Wp, l.k_out) : 1;
-        if (splits > 1) out.partials = w.parts, out.splits = splits, add.partials = w.parts, add.splits = splits;
-        else nc_linear_seg(out, Wp, NC_SEG_RESIDUAL, w.x, Wp);
-        TRY(run_linear(dt, out, s));
-        if (l.ff == NC_FF_EXPERTS) add.expert_out = w.e_out, add.slot_of = w.slot_of, add.slot_w = w.slot_w, add.top = l.top;
+        if (post) {
+            TRY(run_sums(dt, w.cat, l.w_out, M, Wp, l.k_out, w.parts, add, s));
+            add.post_norm_w = l.norm_w;
+            if (l.ff) {
+                add.norm = NC_ROW_COPY, add.h = w.h;
+                TRY(nc_launch_stack_row_add(dt, add, m->eps, M, M, m->width, Wp, s));
+                NcLinear up = nc_linear(w.h, Wp, l.w_ff_in, M, l.ff_cols, Wp);
+                nc_linear_seg(up, l.ff_cols, ff_seg_kind(l.ff), w.act, l.ff_p);
+                TRY(run_linear(dt, up, s));
+                TRY(run_sums(dt, w.act, l.w_ff_out, M, Wp, l.ff_p, w.parts, add, s));
+                add.post_norm_w = l.norm2_w, add.h = nullptr;
+            }
+        } else {
+            if (l.ff == NC_FF_EXPERTS) TRY(run_experts(dt, l, M, Wp, w, s));
+            NcLinear out = nc_linear(w.cat, l.k_out, l.w_out, M, Wp, l.k_out);
+            const int splits = M <= NC_FEW_ROWS ? nc_linear_few_splits(M, Wp, l.k_out) : 1;
+            if (splits > 1) out.partials = w.parts, out.splits = splits, add.partials = w.parts, add.splits = splits;
+            else nc_linear_seg(out, Wp, NC_SEG_RESIDUAL, w.x, Wp);
+            TRY(run_linear(dt, out, s));
+            if (l.ff == NC_FF_EXPERTS) add.expert_out = w.e_out, add.slot_of = w.slot_of, add.slot_w = w.slot_w, add.top = l.top;
+        }
         if (taps) add.tap = taps + (int64_t)i * M * Wp;
         if (i + 1 < m->n_runs) {
             const nc_stack_run& next = m->runs[i + 1];
             add.x0 = next.add_embedding ? w.x0 : nullptr;
             add.step = next.step >= 0 ? m->steps + (int64_t)next.step * Wp : nullptr;
-            add.norm_w = m->layers[next.layer].norm_w, add.h = w.h;
+            entry_norm(m, next, add.norm, add.norm_w);
+            add.h = w.h;
             TRY(nc_launch_stack_row_add(dt, add, m->eps, M, M, m->width, Wp, s));
             continue;
         }
@@ -271,7 +441,7 @@ extern "C" int nc_stack_forward(const nc_stack_model* m, const nc_stack_cache* k
             add.x = w.x, add.tokens_per_row = T;
         }
         if (n_logits == 0) return 0;
-        add.norm_w = m->final_norm_w, add.h = w.h_last, add.rows = logit_rows;
+        add.norm = final_norm, add.norm_w = m->final_norm_w, add.h = w.h_last, add.rows = logit_rows;
         if (kv->advance) add.bump = kv->cache_seqlens, add.bump_by = kv->advance;
         TRY(nc_launch_stack_row_add(dt, add, m->eps, M, n_logits, m->width, Wp, s));
         NcLinear head = nc_linear(w.h_last, Wp, m->head, n_logits, m->vocab, Wp);
@@ -283,7 +453,7 @@ extern "C" int nc_stack_forward(const nc_stack_model* m, const nc_stack_cache* k
 
 extern "C" int nc_stack_linear(int dtype, const void* a, int64_t lda, const void* w, void* out, int ldc, int M, int N, int K, int kind, float limit,
                                int kernel, nc_stream_t stream) {
-    NC_CHECK_ARG(out && kind >= 0 && kind <= 3 && N % 16 == 0 && kernel >= 0 && kernel <= 4, "stack_linear: kind %d, N %d", kind, N);
+    NC_CHECK_ARG(out && ((kind >= NC_SEG_PLAIN && kind <= NC_SEG_F32) || kind == NC_SEG_SILU || kind == NC_SEG_SWIGLU) && N % 16 == 0 && kernel >= 0 && kernel <= 4, "stack_linear: kind %d, N %d", kind, N);
     NcLinear l = nc_linear(a, lda, w, M, N, K);
     nc_linear_seg(l, N, kind, out, ldc, limit);
     if (kernel == 0) return run_linear(dtype, l, (hipStream_t)stream);

@@ -9,7 +9,7 @@
 //   linear_tiled_kernel  more rows: 64 x 128 or 128 x 256 tiles, operands straight into a ring of three LDS stages.
 //
 // A stacked weight is several matrices that read the same input; the epilogue sends each run of output columns its own way (store,
-// gelu, clamped GLU, router logits, residual add, soft-capped logits).  Rows can be grouped by weight (experts).
+// gelu, silu, GLUs, softplus, router logits, residual add, soft-capped logits).  Rows can be grouped by weight (experts).
 #include <atomic>
 #include "nc_stack.h"
 
@@ -63,6 +63,19 @@ __device__ __forceinline__ void store_cols(const NcLinear& g, int64_t out_off, i
             const float y0 = clamped_glu_f32(v[0], v[1], sg.p0), y1 = clamped_glu_f32(v[2], v[3], sg.p0);
             if constexpr (sizeof(T) == 2) *(uint32_t*)o = pack_bf16(y0, y1);
             else o[0] = y0, o[1] = y1;
+            break;
+        }
+        case NC_SEG_SILU: st4_f32((T*)sg.out + out_off + (int64_t)row * sg.ld + c, v4f{silu_f32(v[0]), silu_f32(v[1]), silu_f32(v[2]), silu_f32(v[3])}); break;
+        case NC_SEG_SWIGLU: {
+            T* o = (T*)sg.out + out_off + (int64_t)row * sg.ld + (c >> 1);
+            const float y0 = silu_f32(v[0]) * v[1], y1 = silu_f32(v[2]) * v[3];
+            if constexpr (sizeof(T) == 2) *(uint32_t*)o = pack_bf16(y0, y1);
+            else o[0] = y0, o[1] = y1;
+            break;
+        }
+        case NC_SEG_SOFTPLUS: {
+            const v4f z = v + *(const v4f*)(sg.bias + c);
+            *(v4f*)((float*)sg.out + out_off + (int64_t)row * sg.ld + c) = v4f{softplus_f32(z[0]), softplus_f32(z[1]), softplus_f32(z[2]), softplus_f32(z[3])};
             break;
         }
         case NC_SEG_F32: *(v4f*)((float*)sg.out + out_off + (int64_t)row * sg.ld + c) = v; break;

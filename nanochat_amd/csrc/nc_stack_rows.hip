@@ -1,32 +1,51 @@
-// Row kernels of the layer stack: embedding, residual add + layer norm, expert choice, cache copy.  The residual stream is fp32
+// Row kernels of the layer stack: embedding, residual add + norm, expert choice, cache copy.  The residual stream is fp32
 // [M][width_p] (columns past `width` stay zero), norms are fp32, the normed rows leave in the storage type of the linears.
 #include "nc_stack.h"
 
 namespace {
 constexpr int ROW_THREADS = 256;
 
-// h[i] = (x[i] - mean) / sqrt(var + eps) * w[i] of one row held in registers, four columns per thread and step; columns past width hold 0
-template <typename T, int STEPS>
-__device__ __forceinline__ void layer_norm_row(const v4f (&x)[STEPS], const float* __restrict__ w, float eps, int width, int width_p, T* __restrict__ h,
-                                               float* red) {
-    float sum = 0.f;
-#pragma unroll
-    for (int i = 0; i < STEPS; i++) sum += (x[i][0] + x[i][1]) + (x[i][2] + x[i][3]);
-    const float mean = block_sum<ROW_THREADS / 64>(sum, red) / (float)width;
+// 1 / rms of one row held in registers, four columns per thread and step; columns past width hold 0
+template <int STEPS>
+__device__ __forceinline__ float inverse_rms(const v4f (&x)[STEPS], float eps, int width, float* red) {
     float sq = 0.f;
 #pragma unroll
     for (int i = 0; i < STEPS; i++)
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS) + r;
-            const float d = x[i][r] - mean;
-            sq += c < width ? d * d : 0.f;
-        }
-    const float inv = 1.0f / sqrtf(block_sum<ROW_THREADS / 64>(sq, red) / (float)width + eps);
+        for (int r = 0; r < 4; r++) sq = fmaf(x[i][r], x[i][r], sq);
+    return 1.0f / sqrtf(block_sum<ROW_THREADS / 64>(sq, red) / (float)width + eps);
+}
+
+// h[i] = norm(x)[i] of such a row: (x[i] - mean) / sqrt(var + eps) * w[i], or x[i] / rms(x) * w[i], or x[i]
+template <typename T, int STEPS>
+__device__ __forceinline__ void norm_row(int norm, const v4f (&x)[STEPS], const float* __restrict__ w, float eps, int width, int width_p, T* __restrict__ h,
+                                         float* red) {
+    float mean = 0.f, inv = 1.f;
+    if (norm == NC_ROW_LAYER_NORM) {           // (uniform)
+        float sum = 0.f, sq = 0.f;
+#pragma unroll
+        for (int i = 0; i < STEPS; i++) sum += (x[i][0] + x[i][1]) + (x[i][2] + x[i][3]);
+        mean = block_sum<ROW_THREADS / 64>(sum, red) / (float)width;
+#pragma unroll
+        for (int i = 0; i < STEPS; i++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS) + r;
+                const float d = x[i][r] - mean;
+                sq += c < width ? d * d : 0.f;
+            }
+        inv = 1.0f / sqrtf(block_sum<ROW_THREADS / 64>(sq, red) / (float)width + eps);
+    } else if (norm == NC_ROW_RMS_NORM) {
+        inv = inverse_rms<STEPS>(x, eps, width, red);
+    }
 #pragma unroll
     for (int i = 0; i < STEPS; i++) {
         const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS);
         if (c >= width_p) break;
+        if (norm == NC_ROW_COPY) {
+            st4_f32(h + c, x[i]);
+            continue;
+        }
         const v4f wv = *(const v4f*)(w + c);
         st4_f32(h + c, v4f{(x[i][0] - mean) * inv * wv[0], (x[i][1] - mean) * inv * wv[1], (x[i][2] - mean) * inv * wv[2], (x[i][3] - mean) * inv * wv[3]});
     }
@@ -35,7 +54,7 @@ __device__ __forceinline__ void layer_norm_row(const v4f (&x)[STEPS], const floa
 template <typename T, int STEPS>
 __global__ __launch_bounds__(ROW_THREADS) void stack_embed_kernel(const int64_t* __restrict__ idx, const T* __restrict__ embed, float scale,
                                                                   const float* __restrict__ step, int vocab, float* __restrict__ x,
-                                                                  float* __restrict__ x0, const float* __restrict__ norm_w, float eps,
+                                                                  float* __restrict__ x0, int norm, const float* __restrict__ norm_w, float eps,
                                                                   T* __restrict__ h, int width, int width_p) {
     __shared__ float red[ROW_THREADS / 64];
     const int64_t m = blockIdx.x;
@@ -53,7 +72,7 @@ __global__ __launch_bounds__(ROW_THREADS) void stack_embed_kernel(const int64_t*
             *(v4f*)(x + m * width_p + c) = v[i];
         }
     }
-    layer_norm_row<T, STEPS>(v, norm_w, eps, width, width_p, h + m * width_p, red);
+    norm_row<T, STEPS>(norm, v, norm_w, eps, width, width_p, h + m * width_p, red);
 }
 
 // (every loop over splits and choices asks for its loads in batches, all of a batch before the first sum: a few rows' worth of these
@@ -63,16 +82,17 @@ __global__ __launch_bounds__(ROW_THREADS) void stack_row_add_kernel(NcRowAdd a, 
     constexpr int BATCH = 8;
     __shared__ float red[ROW_THREADS / 64];
     const int64_t m = a.rows ? a.rows[blockIdx.x] : (int)blockIdx.x;
-    v4f v[STEPS];
+    v4f v[STEPS], y[STEPS];
 #pragma unroll
     for (int i = 0; i < STEPS; i++) {
         const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS);
         v[i] = c < width_p ? *(const v4f*)(a.x + m * width_p + c) : v4f{0.f, 0.f, 0.f, 0.f};
+        y[i] = v4f{0.f, 0.f, 0.f, 0.f};
     }
     if (a.partials) {
 #pragma unroll
         for (int i = 0; i < STEPS; i++) {
-            const int c = min(4 * ((int)threadIdx.x + i * ROW_THREADS), width_p - 4);
+            const int at = 4 * ((int)threadIdx.x + i * ROW_THREADS), c = min(at, width_p - 4);
             v4f p[BATCH], sum = v4f{0.f, 0.f, 0.f, 0.f};
             for (int s0 = 0; s0 < a.splits; s0 += BATCH) {
 #pragma unroll
@@ -81,13 +101,10 @@ __global__ __launch_bounds__(ROW_THREADS) void stack_row_add_kernel(NcRowAdd a, 
                 for (int s = 0; s < BATCH; s++)
                     if (s0 + s < a.splits) sum += p[s];
             }
-            v[i] += sum;
+            if (at < width_p) y[i] = sum;
         }
     }
     if (a.expert_out) {
-        v4f sum[STEPS];
-#pragma unroll
-        for (int i = 0; i < STEPS; i++) sum[i] = v4f{0.f, 0.f, 0.f, 0.f};
         for (int k0 = 0; k0 < a.top; k0 += BATCH) {
             int64_t slot[BATCH];
             float w[BATCH];
@@ -100,17 +117,22 @@ __global__ __launch_bounds__(ROW_THREADS) void stack_row_add_kernel(NcRowAdd a, 
 #pragma unroll
             for (int i = 0; i < STEPS; i++) {
                 const int c = min(4 * ((int)threadIdx.x + i * ROW_THREADS), width_p - 4);
-                v4f y[BATCH];
+                v4f e[BATCH];
 #pragma unroll
-                for (int k = 0; k < BATCH; k++) y[k] = ld4_f32((const T*)a.expert_out + slot[k] * width_p + c);
+                for (int k = 0; k < BATCH; k++) e[k] = ld4_f32((const T*)a.expert_out + slot[k] * width_p + c);
 #pragma unroll
                 for (int k = 0; k < BATCH; k++)
-                    if (k0 + k < a.top) sum[i] += y[k] * w[k];
+                    if (k0 + k < a.top) y[i] += e[k] * w[k];
             }
         }
-#pragma unroll
-        for (int i = 0; i < STEPS; i++) v[i] += sum[i];
     }
+    if (a.post_norm_w) {                       // (uniform; no expert rows here: y is zero past the padded width)
+        const float inv = inverse_rms<STEPS>(y, eps, width, red);
+#pragma unroll
+        for (int i = 0; i < STEPS; i++) y[i] *= *(const v4f*)(a.post_norm_w + min(4 * ((int)threadIdx.x + i * ROW_THREADS), width_p - 4)) * inv;
+    }
+#pragma unroll
+    for (int i = 0; i < STEPS; i++) v[i] += y[i];
 #pragma unroll
     for (int i = 0; i < STEPS; i++) {
         const int c = 4 * ((int)threadIdx.x + i * ROW_THREADS);
@@ -123,7 +145,7 @@ __global__ __launch_bounds__(ROW_THREADS) void stack_row_add_kernel(NcRowAdd a, 
         if (a.step) v[i] += *(const v4f*)(a.step + c);
         if (!a.rows) *(v4f*)(a.x + m * width_p + c) = v[i];
     }
-    if (a.h) layer_norm_row<T, STEPS>(v, a.norm_w, eps, width, width_p, (T*)a.h + (int64_t)blockIdx.x * width_p, red);
+    if (a.h) norm_row<T, STEPS>(a.norm, v, a.norm_w, eps, width, width_p, (T*)a.h + (int64_t)blockIdx.x * width_p, red);
     if (a.bump && threadIdx.x == 0 && (int)blockIdx.x % a.tokens_per_row == a.tokens_per_row - 1) a.bump[(int)blockIdx.x / a.tokens_per_row] += a.bump_by;
 }
 
@@ -236,6 +258,27 @@ __global__ __launch_bounds__(1024) void route_sort_kernel(NcRoute r, int M) {
     }
 }
 
+// ------------------------------------------------------------------------------------------------ joint norm and gate
+// One workgroup per row; the row passes twice, the second time out of the cache.
+template <typename T>
+__global__ __launch_bounds__(256) void joint_gate_kernel(const float* __restrict__ raw, int cols, int count, const T* __restrict__ gate, int ldg,
+                                                         const float* __restrict__ w, float eps, float scale, T* __restrict__ out, int ldo) {
+    __shared__ float red[4];
+    const int64_t m = blockIdx.x;
+    const float* o = raw + m * cols;
+    float sq = 0.f;
+    for (int c = 4 * threadIdx.x; c < cols; c += 1024) {
+        const v4f v = *(const v4f*)(o + c);
+        sq += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+    }
+    const float inv = scale / sqrtf(block_sum<4>(sq, red) / (float)count + eps);
+    for (int c = 4 * threadIdx.x; c < cols; c += 1024) {
+        const v4f v = *(const v4f*)(o + c), g = ld4_f32(gate + m * ldg + c), wv = *(const v4f*)(w + c);
+        st4_f32(out + m * ldo + c, v4f{v[0] * inv * wv[0] * sigmoid_f32(g[0]), v[1] * inv * wv[1] * sigmoid_f32(g[1]), v[2] * inv * wv[2] * sigmoid_f32(g[2]),
+                                       v[3] * inv * wv[3] * sigmoid_f32(g[3])});
+    }
+}
+
 __global__ __launch_bounds__(256) void stack_cache_copy_kernel(const uint8_t* __restrict__ src, uint8_t* __restrict__ dst, int src_rows,
                                                                int64_t src_stride, int64_t dst_stride, int64_t pieces) {
     const int row = blockIdx.y;
@@ -256,14 +299,14 @@ __global__ __launch_bounds__(256) void stack_cache_copy_kernel(const uint8_t* __
 }  // namespace
 
 int nc_launch_stack_embed(int dtype, const int64_t* idx, const void* embed, float scale, const float* step, int vocab, float* x, float* x0,
-                          const float* norm_w, float eps, void* h, int M, int width, int width_p, hipStream_t s) {
+                          int norm, const float* norm_w, float eps, void* h, int M, int width, int width_p, hipStream_t s) {
     NC_CHECK_ARG(width_p % 4 == 0 && width <= width_p && width_p <= 8192, "stack_embed: width %d", width_p);
     NcProfScope prof(NC_CLS_ROWS, (double)M * width_p * 8, s);
 #define CALL(S)                                                                                                                                \
     if (dtype) hipLaunchKernelGGL((stack_embed_kernel<float, S>), dim3(M), dim3(ROW_THREADS), 0, s, idx, (const float*)embed, scale, step, vocab, \
-                                  x, x0, norm_w, eps, (float*)h, width, width_p);                                                              \
+                                  x, x0, norm, norm_w, eps, (float*)h, width, width_p);                                                              \
     else hipLaunchKernelGGL((stack_embed_kernel<bf16_t, S>), dim3(M), dim3(ROW_THREADS), 0, s, idx, (const bf16_t*)embed, scale, step, vocab, x, \
-                            x0, norm_w, eps, (bf16_t*)h, width, width_p)
+                            x0, norm, norm_w, eps, (bf16_t*)h, width, width_p)
     STEPS_SWITCH(width_p, CALL);
 #undef CALL
     NC_CHECK_LAUNCH("stack_embed");
@@ -308,5 +351,17 @@ int nc_launch_stack_cache_copy(const void* src, void* dst, int src_rows, int dst
     hipLaunchKernelGGL(stack_cache_copy_kernel, dim3(gx, dst_rows), dim3(256), 0, s, (const uint8_t*)src, (uint8_t*)dst, src_rows, src_stride, dst_stride,
                        pieces);
     NC_CHECK_LAUNCH("stack_cache_copy");
+    return 0;
+}
+
+int nc_launch_joint_gate(int dtype, const float* raw, int cols, int count, const void* gate, int ldg, const float* w, float eps, float scale, void* out,
+                         int ldo, int M, hipStream_t s) {
+    NC_CHECK_ARG(raw && gate && w && out && cols % 4 == 0 && count > 0 && count <= cols && ldg % 4 == 0 && ldo % 4 == 0, "joint_gate: %d of %d columns", count, cols);
+    NcProfScope prof(NC_CLS_ROWS, (double)M * cols * (dtype ? 12 : 8), s);
+    if (dtype)
+        hipLaunchKernelGGL((joint_gate_kernel<float>), dim3(M), dim3(256), 0, s, raw, cols, count, (const float*)gate, ldg, w, eps, scale, (float*)out, ldo);
+    else
+        hipLaunchKernelGGL((joint_gate_kernel<bf16_t>), dim3(M), dim3(256), 0, s, raw, cols, count, (const bf16_t*)gate, ldg, w, eps, scale, (bf16_t*)out, ldo);
+    NC_CHECK_LAUNCH("joint_gate");
     return 0;
 }

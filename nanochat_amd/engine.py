@@ -69,7 +69,7 @@ def use_calculator(expr):
 class SequenceCache:
     """Positions of the rows of a cache: per-row lengths in an int32 device tensor, with a host-side copy so that get_pos() does not
     have to read the device tensor back every decode step.  What the rows hold is the subclass's: keys and values (KVCache), or
-    latents and recurrent states (StackCache).  The Engine uses: get_pos, advance / note_advanced (by the model), mark and rewind."""
+    token rows and recurrent states (StackCache).  The Engine uses: get_pos, advance / note_advanced (by the model), mark and rewind."""
 
     def __init__(self, batch_size, seq_len, device):
         self.batch_size = batch_size
@@ -190,18 +190,18 @@ class KVCache(SequenceCache):
 
 
 class StackCache(SequenceCache):
-    """Cache of a layer stack (nanochat_amd/stack.py): for every run of a latent-attention layer the latents of all tokens, for every
-    run of a recurrent layer one fp32 state per row.  A layer that runs several times has a slot for each of its runs.
+    """Cache of a layer stack (nanochat_amd/stack.py): for every run of an attention mixer a row per token (latents, or
+    keys and values), for every run of a recurrent mixer one fp32 state per sequence.  A layer that runs several times has slots for each
+    of its runs.
 
-    `latents[slot]` [B, seq_len, latent width]; `states[i][slot]` [B, heads, dim, vdim], two buffers: a forward reads one and writes the
-    other, so a forward can be taken back.  A row at position 0 does not read its state: a slot of the batch is given back by
+    `rows[slot]` [B, seq_len, row width]; `states[i][slot]` [B, ...], two buffers: a forward reads one and writes the other, so a forward can be taken back.  A row at position 0 does not read its state: a slot of the batch is given back by
     setting its position to zero."""
 
-    def __init__(self, latent_widths, state_shapes, dtype, batch_size, seq_len, device, prefill_from=None):
+    def __init__(self, row_widths, state_shapes, dtype, batch_size, seq_len, device, prefill_from=None):
         super().__init__(batch_size, seq_len, device)
         self.dtype = dtype
         # (zeros: the positions past a row's end enter products with weight zero, and must be finite there)
-        self.latents = [torch.zeros(batch_size, seq_len, w, device=device, dtype=dtype) for w in latent_widths]
+        self.rows = [torch.zeros(batch_size, seq_len, w, device=device, dtype=dtype) for w in row_widths]
         self.states = [[torch.zeros(batch_size, *s, device=device, dtype=torch.float32) for s in state_shapes] for _ in range(2)]
         self._pointers = None
         self._current = 0                          # which of the two state buffers holds the states
@@ -229,9 +229,9 @@ class StackCache(SequenceCache):
         return self.states[self._current], self.states[self._current ^ 1]
 
     def pointers(self):
-        """Arrays of device pointers: latents, states to read, states to write (the tensors of a cache never move)."""
+        """Arrays of device pointers: token rows, states to read, states to write (the tensors of a cache never move)."""
         if self._pointers is None:
-            lat, a, b = ((ctypes.c_void_p * max(1, len(ts)))(*(t.data_ptr() for t in ts)) for ts in (self.latents, *self.states))
+            lat, a, b = ((ctypes.c_void_p * max(1, len(ts)))(*(t.data_ptr() for t in ts)) for ts in (self.rows, *self.states))
             self._pointers = ((lat, a, b), (lat, b, a))
         return self._pointers[self._current]
 
@@ -242,7 +242,7 @@ class StackCache(SequenceCache):
         self._last_tokens = num_tokens
 
     def rewind(self, num_tokens, mark=None):
-        """Take back the last forward, which brought `num_tokens` tokens (their latents are overwritten by the next ones)."""
+        """Take back the last forward, which brought `num_tokens` tokens (their rows are overwritten by the next ones)."""
         assert 0 < num_tokens == self._last_tokens, "only the last forward can be taken back"
         self.cache_seqlens -= num_tokens
         self._host_pos = [p - num_tokens for p in self._host_pos]
@@ -268,8 +268,8 @@ class StackCache(SequenceCache):
     def _copy(self, other, src_row, src_rows, dst_row, dst_rows):
         n = other._pos_max
         assert n <= self.max_seq_len and self.dtype == other.dtype
-        assert [t.shape[2] for t in self.latents] == [t.shape[2] for t in other.latents]
-        for src, dst in zip(other.latents, self.latents):
+        assert [t.shape[2] for t in self.rows] == [t.shape[2] for t in other.rows]
+        for src, dst in zip(other.rows, self.rows):
             ops.stack_cache_copy(src[src_row:src_row + src_rows], dst[dst_row:dst_row + dst_rows], n)
         for src, dst in zip(other.state_buffers()[0], self.state_buffers()[0]):
             ops.stack_cache_copy(src[src_row:src_row + src_rows], dst[dst_row:dst_row + dst_rows], src.shape[1])

@@ -2,9 +2,6 @@
 feed-forward (both sublayers read one layer norm), with a run of layers that repeats with the same weights.
 
 The design's config.json keys and tensor names are read here; the mechanisms are those of stack.py."""
-import torch
-
-from .checkpoint import read_config, read_safetensors
 from .stack import DenseGelu, Experts, LatentAttention, LayerSpec, LayerStack, Retention, StackConfig
 
 ARCHITECTURE = "Palilix"
@@ -46,13 +43,4 @@ def stack_config(cfg):
 
 
 class Palilix(LayerStack):
-    @classmethod
-    def from_config(cls, cfg, dtype=torch.bfloat16):
-        return cls(stack_config(cfg), dtype)
-
-    @classmethod
-    def load(cls, model_dir, dtype=torch.bfloat16, device="cuda"):
-        """The model in a folder with config.json and model.safetensors."""
-        with torch.device("meta"):
-            model = cls.from_config(read_config(model_dir), dtype)
-        return model.load_tensors(read_safetensors(model_dir), torch.device(device)).eval()
+    stack_config = staticmethod(stack_config)

@@ -9,7 +9,7 @@ import torch
 from .checkpoint import read_config
 
 # architecture -> (module, class); a class has load(model_dir, dtype, device)
-ARCHITECTURES = {"Palilix": ("palilix", "Palilix")}
+ARCHITECTURES = {"Palilix": ("palilix", "Palilix"), "Zodirax": ("zodirax", "Zodirax")}
 
 
 def model_class(architecture):

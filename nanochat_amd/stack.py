@@ -1,14 +1,16 @@
 """Decoders made of configured layers: any order of mixers and feed-forwards, a run of layers that may repeat with the same weights.
 
-A layer is `x += mixer(h) + ff(h)` with `h = layer_norm(x)`.  The mechanisms are classes of their own with their sizes and constants as
-fields; each knows the tensors it needs, how they are packed for the kernels and what it keeps per sequence:
+A layer is `x += mixer(h) + ff(h)` with `h = norm(x)` (block "parallel"), or `x += norm1(mixer(x)); x += norm2(ff(x))` (block
+"post_norm").  The mechanisms are classes of their own with their sizes and constants as fields; each knows the tensors it needs, how they
+are packed for the kernels and what it keeps per sequence:
 
-    mixers         LatentAttention, Retention
-    feed-forwards  DenseGelu, Experts (clamped GLU experts, softmax router, optional shared expert)
+    mixers         LatentAttention, Retention, WindowAttention, SelectiveScan, SideBySide (two of them on the same input)
+    feed-forwards  DenseGelu, DenseSwiglu, Experts (clamped GLU experts, softmax router, optional shared expert)
 
 `LayerStack` is the model: weights by name, a packed plan that is rebuilt whenever a weight changes, and a forward that is one native
 call (nc_stack_forward).  It has the surface the Engine and the harness use on every model of this package (forward, forward_last,
-new_cache, get_device, the cost accounting).  A design is a class that turns its configuration into a StackConfig (palilix.py).
+new_cache, get_device, the cost accounting).  A design is a class that turns its configuration into a StackConfig (palilix.py,
+zodirax.py).
 
 Two storage types: bfloat16 (matrix products in bf16 with 32-bit sums; residual stream, norms, angles, scores, router and recurrent
 state in 32-bit), and float32 (everything in true 32-bit).
@@ -21,8 +23,10 @@ import torch
 import torch.nn as nn
 
 from . import _lib, ops
+from .checkpoint import read_config, read_safetensors
 
 PAD = ops.STACK_PAD
+WEIGHT_FIELDS = ("w_uk_t", "w_ukv", "w_x", "w_dt", "w_dt_t")       # of a mixer's descriptor: in the storage type; the others are fp32
 
 
 def round_up(n, m):
@@ -36,9 +40,58 @@ def padded(t, *shape):
     return out
 
 
+@dataclass(frozen=True)
+class Rotation:
+    """Rotary positions: pair i of `dims` leading dimensions turns by position * base^(-2i/dims).  With `factor`, wavelengths longer than
+    original / low are stretched by it, those shorter than original / high are kept, and a ramp in 1 / wavelength joins the two."""
+    base: float
+    dims: int
+    factor: float = 1.0
+    low: float = 1.0
+    high: float = 1.0
+    original: float = 0.0           # 0: no stretching
+
+    def frequencies(self):
+        i = torch.arange(self.dims // 2, dtype=torch.float64)
+        f = self.base ** (-2.0 * i / max(self.dims, 1))
+        if not self.original:
+            return f
+        turns = self.original * f / (2 * math.pi)             # original / wavelength
+        if self.high == self.low:
+            keep = (turns > self.high).double()
+        else:
+            keep = ((turns - self.low) / (self.high - self.low)).clamp(0.0, 1.0)
+        return (1 - keep) * f / self.factor + keep * f
+
+
+NO_ROTATION = Rotation(1.0, 0)
+ROW_CACHE, STATE_CACHE = 0, 1       # what a mixer keeps: a row per token, or a state per sequence
+
+
+class Mixer:
+    """What the layers ask of a mixer.  `cols` rows of the input matrix are its projections, `out` columns of the output matrix take its
+    result; `row_width` values per token or a state of `state_shape` are kept per sequence.  Tensors named in `fp32` stay 32-bit."""
+    cache = ROW_CACHE
+    row_width = 0
+    state_shape = ()
+    rotation = NO_ROTATION
+    out_scale = 1.0
+    fp32 = ()
+    per_key = ()                    # tensors applied per key or query, counted in flops() rather than as weights a token passes
+    scales_output = False
+
+    def prefill_flops(self, tokens):
+        return sum(self.flops(n) for n in range(1, tokens + 1))
+
+    @property
+    def parts(self):
+        """[(prefix of its tensors' names, mixer)]: itself, or what it is made of."""
+        return [("", self)]
+
+
 # ------------------------------------------------------------------------------------------------ mixers
 @dataclass
-class LatentAttention:
+class LatentAttention(Mixer):
     """Causal softmax attention whose keys and values are linear in one cached latent per token, plus one rotated key part that the heads
     share.  Per head: `dim` unrotated and `rot_dim` rotated query / key dimensions, `vdim` values; the latent has `rank` values."""
     heads: int
@@ -50,16 +103,17 @@ class LatentAttention:
     rot_base: float
 
     kind = 0
+    per_key = ("uk", "uv")
 
     def __post_init__(self):
         assert self.rot_dim % 2 == 0, f"rotated part of odd size {self.rot_dim}"
-        self.rot_dims = self.rot_dim
+        self.rotation = Rotation(self.rot_base, self.rot_dim)
         self.dim_p, self.rot_p, self.rank_p = round_up(self.dim, 32), round_up(self.rot_dim, 32), round_up(self.rank, PAD)
         # the heads' values side by side fill whole K-steps of the output matrix
         self.vdim_p = round_up(self.vdim, 16 * (4 // math.gcd(self.heads, 4)))
-        self.mix_cols = self.heads * (self.dim_p + self.rot_p) + self.rank_p + self.rot_p
-        self.mix_out = self.heads * self.vdim_p
-        self.latent_width = self.rank_p + self.rot_p
+        self.cols = self.heads * (self.dim_p + self.rot_p) + self.rank_p + self.rot_p
+        self.out = self.heads * self.vdim_p
+        self.row_width = self.rank_p + self.rot_p
 
     def tensors(self, width):
         H = self.heads
@@ -82,8 +136,7 @@ class LatentAttention:
                 {"kv_norm_w": padded(w["dkv.norm"].float(), self.rank_p), "w_uk_t": padded(uk.transpose(1, 2), H, self.rank_p, self.dim_p), "w_ukv": ukv})
 
     def describe(self, d):
-        d.dim, d.dim_p, d.vdim, d.vdim_p, d.rot_dim, d.rot_p, d.rot_dims = (self.dim, self.dim_p, self.vdim, self.vdim_p, self.rot_dim, self.rot_p,
-                                                                              self.rot_dims)
+        d.heads, d.dim, d.dim_p, d.vdim, d.vdim_p, d.rot_dim, d.rot_p = self.heads, self.dim, self.dim_p, self.vdim, self.vdim_p, self.rot_dim, self.rot_p
         d.rank, d.rank_p, d.score_scale = self.rank, self.rank_p, self.scale
 
     def flops(self, keys):
@@ -100,36 +153,42 @@ class LatentAttention:
 
 
 @dataclass
-class Retention:
-    """Linear attention with one fixed decay per head, rotary positions on the first `rot_dims` dimensions of q and k, outputs normed per
-    head and gated.  `decay` holds one factor per head."""
+class Retention(Mixer):
+    """Linear attention with one fixed decay per head, rotary positions on the first `rot_dims` dimensions of q and k.  `decay` holds one
+    factor per head.  q, k and v pass silu if `silu_qkv`.  The outputs are normed per head and multiplied by silu(gate), or (`joint_norm`)
+    normed over all heads at once with a weight and multiplied by sigmoid(gate)."""
     heads: int
     dim: int
     vdim: int
     decay: list
-    rot_dims: int
-    rot_base: float
+    rot_dims: int = 0
+    rot_base: float = 1.0
     k_scale: float = field(default=None)
+    silu_qkv: bool = False
+    joint_norm: bool = False
 
     kind = 1
+    cache = STATE_CACHE
 
     def __post_init__(self):
         assert len(self.decay) == self.heads, f"{len(self.decay)} decays for {self.heads} heads"
         assert self.rot_dims % 2 == 0 and self.rot_dims <= self.dim
+        self.rotation = Rotation(self.rot_base, self.rot_dims)
+        self.scales_output = self.joint_norm
         if self.k_scale is None:
             self.k_scale = self.dim ** -0.5
         # sizes the kernels hold a state in registers for; larger ones go through memory
         sizes = [n for n in (64, 128, 256)]
         self.dim_p = next((n for n in sizes if n >= self.dim), round_up(self.dim, PAD))
         self.vdim_p = next((n for n in sizes if n >= max(self.vdim, 128 if self.dim_p == 256 else 0)), round_up(self.vdim, PAD))
-        self.mix_cols = 2 * self.heads * (self.dim_p + self.vdim_p)
-        self.mix_out = self.heads * self.vdim_p
+        self.cols = 2 * self.heads * (self.dim_p + self.vdim_p)
+        self.out = self.heads * self.vdim_p
         self.state_shape = (self.heads, self.dim_p, self.vdim_p)
 
     def tensors(self, width):
         H = self.heads
         return {"q": (H * self.dim, width), "k": (H * self.dim, width), "v": (H * self.vdim, width), "g": (H * self.vdim, width),
-                "o": (width, H * self.vdim)}
+                "o": (width, H * self.vdim)} | ({"norm": (H * self.vdim,)} if self.joint_norm else {})
 
     def pack(self, w):
         H, width = self.heads, w["q"].shape[1]
@@ -141,10 +200,14 @@ class Retention:
         o = padded(w["o"].view(width, H, self.vdim), width, H, self.vdim_p).view(width, H * self.vdim_p)
         decay = torch.tensor(self.decay, dtype=torch.float32)
         log2 = torch.log2(decay.double()).clamp(min=-1000.0).float()          # a decay of 0 forgets everything: 2^-1000 is 0 as well
-        return torch.cat(rows), o, {"decay": torch.stack([decay, log2], dim=1).to(o.device)}
+        extra = {"decay": torch.stack([decay, log2], dim=1).to(o.device)}
+        if self.joint_norm:
+            extra["out_norm_w"] = padded(w["norm"].float().view(H, self.vdim), H, self.vdim_p)
+        return torch.cat(rows), o, extra
 
     def describe(self, d):
-        d.dim, d.dim_p, d.vdim, d.vdim_p, d.rot_dims, d.score_scale = self.dim, self.dim_p, self.vdim, self.vdim_p, self.rot_dims, self.k_scale
+        d.heads, d.dim, d.dim_p, d.vdim, d.vdim_p, d.score_scale = self.heads, self.dim, self.dim_p, self.vdim, self.vdim_p, self.k_scale
+        d.silu_qkv, d.gate = int(self.silu_qkv), int(self.joint_norm)
 
     def flops(self, keys):
         return 4 * self.heads * self.dim * self.vdim
@@ -154,6 +217,137 @@ class Retention:
 
     def read_elements(self, keys):
         return 0, 2 * self.heads * self.dim * self.vdim
+
+
+@dataclass
+class WindowAttention(Mixer):
+    """Grouped-query softmax attention over the last `window` keys and, however far away, the first `keep_first`.  q, k and v have biases;
+    q and k are RMS-normed over all heads at once, then turned; a number per head (the sink) counts in the softmax's denominator."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int
+    keep_first: int
+    rotation: Rotation = NO_ROTATION
+    out_scale: float = 1.0
+
+    kind = 2
+    scales_output = True
+
+    def __post_init__(self):
+        assert self.kv_heads >= 1 and self.heads % self.kv_heads == 0, f"{self.heads} query heads on {self.kv_heads} key heads"
+        assert self.rotation.dims % 2 == 0 and self.rotation.dims <= self.dim, f"{self.rotation.dims} of {self.dim} dimensions turn"
+        assert self.window >= 1 and self.keep_first >= 0
+        self.dim_p = round_up(self.dim, 32)
+        self.vdim_p = round_up(self.vdim, 16 * (4 // math.gcd(self.heads, 4)))
+        self.cols = (self.heads + self.kv_heads) * self.dim_p + self.kv_heads * self.vdim_p
+        self.out = self.heads * self.vdim_p
+        self.row_width = self.kv_heads * (self.dim_p + self.vdim_p)
+
+    def tensors(self, width):
+        out = {"o": (width, self.heads * self.vdim), "sink": (self.heads,), "q.norm": (self.heads * self.dim,), "k.norm": (self.kv_heads * self.dim,)}
+        for name, n in (("q", self.heads * self.dim), ("k", self.kv_heads * self.dim), ("v", self.kv_heads * self.vdim)):
+            out |= {name: (n, width), f"{name}.b": (n,)}
+        return out
+
+    def pack(self, w):
+        H, G, width = self.heads, self.kv_heads, w["q"].shape[1]
+        sizes = {"q": (H, self.dim, self.dim_p), "k": (G, self.dim, self.dim_p), "v": (G, self.vdim, self.vdim_p)}
+        rows = [padded(w[name].view(n, d, width), n, d_p, width).view(n * d_p, width) for name, (n, d, d_p) in sizes.items()]
+        bias = [padded(w[f"{name}.b"].float().view(n, d), n, d_p).view(-1) for name, (n, d, d_p) in sizes.items()]
+        norms = {f"{name}_norm_w": padded(w[f"{name}.norm"].float().view(n, d), n, d_p) for name, (n, d, d_p) in sizes.items() if name != "v"}
+        o = padded(w["o"].view(width, H, self.vdim), width, H, self.vdim_p).view(width, H * self.vdim_p)
+        return torch.cat(rows), o, {"qkv_bias": torch.cat(bias), "sink": w["sink"].float(), **norms}
+
+    def describe(self, d):
+        d.heads, d.kv_heads, d.dim, d.dim_p, d.vdim, d.vdim_p = self.heads, self.kv_heads, self.dim, self.dim_p, self.vdim, self.vdim_p
+        d.score_scale, d.window, d.keep_first = self.scale, min(self.window, 1 << 30), min(self.keep_first, 1 << 30)
+
+    def seen(self, keys):
+        return min(keys, self.window + self.keep_first)
+
+    def flops(self, keys):
+        return 2 * self.heads * self.seen(keys) * (self.dim + self.vdim)
+
+    def read_elements(self, keys):
+        return self.seen(keys) * self.kv_heads * (self.dim + self.vdim), 0
+
+
+@dataclass
+class SelectiveScan(Mixer):
+    """A causal convolution of `conv` taps per channel, then `state` linear recurrences per channel whose step sizes, inputs and read-outs
+    come from the token; gated by silu of a second projection."""
+    inner: int
+    state: int
+    conv: int
+    dt_rank: int
+
+    kind = 3
+    cache = STATE_CACHE
+    fp32 = ("conv", "A_log")
+    scales_output = True
+
+    def __post_init__(self):
+        assert min(self.inner, self.state, self.conv, self.dt_rank) >= 1
+        assert self.state <= 256, f"{self.state} states per channel"
+        self.inner_p, self.dt_rank_p = round_up(self.inner, PAD), round_up(self.dt_rank, PAD)
+        # 4, 8, 12 or 16 states in each of 1, 2, 4, 8 or 16 lanes
+        self.state_p = min(n << k for n in (4, 8, 12, 16) for k in range(5) if n << k >= self.state)
+        self.bc_p = round_up(self.state_p, 16)
+        self.cols, self.out = 2 * self.inner_p, self.inner_p
+        self.state_shape = (self.state_p + self.conv - 1, self.inner_p)
+
+    def tensors(self, width):
+        n = self.inner
+        return {"in": (2 * n, width), "conv": (n, self.conv), "conv.b": (n,), "x": (self.dt_rank + 2 * self.state, n), "dt": (n, self.dt_rank), "dt.b": (n,),
+                "A_log": (n, self.state), "D": (n,), "o": (width, n)}
+
+    def pack(self, w):
+        n, n_p, width = self.inner, self.inner_p, w["in"].shape[1]
+        rows = padded(w["in"].view(2, n, width), 2, n_p, width).view(2 * n_p, width)
+        step, B, C = w["x"].split([self.dt_rank, self.state, self.state])
+        w_x = torch.cat([padded(step, self.dt_rank_p, n_p), padded(B, self.bc_p, n_p), padded(C, self.bc_p, n_p)])
+        w_dt = padded(w["dt"], n_p, self.dt_rank_p)
+        a = -torch.exp(w["A_log"].double()) * math.log2(math.e)
+        return rows, padded(w["o"], width, n_p), {
+            "conv_w": padded(w["conv"].float().T, self.conv, n_p), "conv_b": padded(w["conv.b"].float(), n_p), "w_x": w_x, "w_dt": w_dt, "w_dt_t": w_dt.T,
+            "dt_b": padded(w["dt.b"].float(), n_p), "a_log2": padded(a.T, self.state_p, n_p).float(), "skip": padded(w["D"].float(), n_p)}
+
+    def describe(self, d):
+        d.inner, d.inner_p, d.state, d.state_p, d.taps = self.inner, self.inner_p, self.state, self.state_p, self.conv
+        d.dt_rank, d.dt_rank_p = self.dt_rank, self.dt_rank_p
+
+    def flops(self, keys):
+        return 6 * self.inner * self.state
+
+    def prefill_flops(self, tokens):
+        return tokens * self.flops(0)
+
+    def read_elements(self, keys):
+        return 0, 2 * self.inner * (self.state + self.conv - 1)
+
+
+@dataclass
+class SideBySide:
+    """Two mixers on the same input; the layer's mixer result is the sum of theirs, each times its scale."""
+    left: Mixer
+    right: Mixer
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+    def __post_init__(self):
+        for mixer, scale in ((self.left, self.left_scale), (self.right, self.right_scale)):
+            assert scale == 1.0 or mixer.scales_output, f"{type(mixer).__name__} does not scale its result"
+            mixer.out_scale = scale
+
+    @property
+    def parts(self):
+        return [("left.", self.left), ("right.", self.right)]
+
+    def tensors(self, width):
+        return {prefix + k: s for prefix, m in self.parts for k, s in m.tensors(width).items()}
 
 
 # ------------------------------------------------------------------------------------------------ feed-forwards
@@ -185,6 +379,30 @@ class DenseGelu:
 
     def active_params(self, width):
         return 2 * self.ff * width
+
+
+@dataclass
+class DenseSwiglu:
+    """down (silu(gate h) * (up h))."""
+    ff: int
+
+    kind = 3
+
+    def __post_init__(self):
+        self.ff_p = round_up(self.ff, PAD)
+        self.router_cols, self.ff_cols = 0, 2 * self.ff_p
+
+    def tensors(self, width):
+        return {"gate": (self.ff, width), "up": (self.ff, width), "down": (width, self.ff)}
+
+    def pack(self, w, width_p):
+        return None, interleaved(w["gate"], w["up"], self.ff_p, width_p), padded(w["down"], width_p, self.ff_p), {}
+
+    def describe(self, d):
+        d.ff_limit = 0.0
+
+    def active_params(self, width):
+        return 3 * self.ff * width
 
 
 @dataclass
@@ -237,8 +455,16 @@ class Experts:
 # ------------------------------------------------------------------------------------------------ configuration
 @dataclass
 class LayerSpec:
-    mixer: object
+    mixer: object                   # a Mixer, or two SideBySide
     ff: object = None               # None: no feed-forward
+
+    @property
+    def mixers(self):
+        return [m for _, m in self.mixer.parts]
+
+
+BLOCKS = {"parallel": 0, "post_norm": 1}
+NORMS = {"layer": 0, "rms": 1}
 
 
 @dataclass
@@ -254,7 +480,17 @@ class StackConfig:
     loop_stop: int = 0
     loop_times: int = 1
     loop_steps: bool = False        # a learned vector is added at the start of every pass
+    block: str = "parallel"         # "parallel": one norm, both sublayers read it; "post_norm": one after the other, a norm on each output
+    norm: str = "layer"             # "layer" or "rms"
+    norm_offset: float = 0.0        # added to the stored weights of the model's norms (1: stored around zero)
+    tied_head: bool = False         # the output matrix is the embedding table
     sequence_len: int = 2048        # how far a generation without a token limit goes; the model itself has no limit
+
+    def __post_init__(self):
+        if self.block not in BLOCKS or self.norm not in NORMS:
+            raise ValueError(f"block {self.block!r}, norm {self.norm!r}")
+        if self.block == "post_norm" and (self.norm != "rms" or any(isinstance(layer.ff, Experts) for layer in self.layers)):
+            raise ValueError("a post-norm block has RMS norms and dense feed-forwards")
 
     @property
     def n_layer(self):
@@ -298,6 +534,18 @@ class LayerStack(nn.Module):
         self._rope_len = 0
         self._workspaces = {}
 
+    @classmethod
+    def from_config(cls, cfg, dtype=torch.bfloat16):
+        """A design's model (its class has a stack_config) from a config.json dictionary."""
+        return cls(cls.stack_config(cfg), dtype)
+
+    @classmethod
+    def load(cls, model_dir, dtype=torch.bfloat16, device="cuda"):
+        """The model in a folder with config.json and model.safetensors."""
+        with torch.device("meta"):
+            model = cls.from_config(read_config(model_dir), dtype)
+        return model.load_tensors(read_safetensors(model_dir), torch.device(device)).eval()
+
     @staticmethod
     def tensor_shapes(config):
         """{tensor name: shape} of the whole model."""
@@ -309,8 +557,9 @@ class LayerStack(nn.Module):
             out[f"l{i}.norm1"] = (W,)
             out |= {f"l{i}.mix.{k}": s for k, s in layer.mixer.tensors(W).items()}
             if layer.ff is not None:
+                out |= {f"l{i}.norm2": (W,)} if config.block == "post_norm" else {}
                 out |= {f"l{i}.mlp.{k}": s for k, s in layer.ff.tensors(W).items()}
-        return out | {"final.norm": (W,), "head": (config.vocab_size, W)}
+        return out | {"final.norm": (W,)} | ({} if config.tied_head else {"head": (config.vocab_size, W)})
 
     def held_tensors(self):
         """{name: parameter} as the model holds them (experts of a layer together)."""
@@ -324,9 +573,11 @@ class LayerStack(nn.Module):
         return out
 
     def load_tensors(self, tensors, device):
-        """Take the weights by name, in the dtype they come in; names and shapes must be exactly the model's."""
+        """Take the weights by name, in the dtype they come in; names and shapes must be exactly the model's (the norm of a feed-forward
+        that a layer does not have may be there)."""
         want = self.tensor_shapes(self.config)
-        missing, extra = sorted(set(want) - set(tensors)), sorted(set(tensors) - set(want))
+        idle = {f"l{i}.norm2" for i, layer in enumerate(self.config.layers) if layer.ff is None and self.config.block == "post_norm"}
+        missing, extra = sorted(set(want) - set(tensors)), sorted(set(tensors) - set(want) - idle)
         if missing or extra:
             raise RuntimeError(f"weights do not match the model: missing {missing[:4]}, unexpected {extra[:4]}")
         for name, shape in want.items():
@@ -350,12 +601,15 @@ class LayerStack(nn.Module):
 
     # ---- cache
     def new_cache(self, batch_size, seq_len, prefill_from=None, share_prompt_reads=False):
-        """(share_prompt_reads: every model's new_cache takes it; latents are read per row here)"""
+        """(share_prompt_reads: every model's new_cache takes it; cached rows are read per sequence here)"""
         from .engine import StackCache
-        mixers = [self.config.layers[i].mixer for i, _, _ in self.run_list]
-        cache = StackCache([m.latent_width for m in mixers if isinstance(m, LatentAttention)], [m.state_shape for m in mixers if isinstance(m, Retention)],
-                           self.dtype, batch_size, seq_len, self.get_device(), prefill_from=prefill_from)
-        return cache
+        mixers = self.run_mixers()
+        return StackCache([m.row_width for m in mixers if m.cache == ROW_CACHE], [m.state_shape for m in mixers if m.cache == STATE_CACHE],
+                          self.dtype, batch_size, seq_len, self.get_device(), prefill_from=prefill_from)
+
+    def run_mixers(self):
+        """The mixers in the order they run, a repeated layer's once per run."""
+        return [m for i, _, _ in self.run_list for m in self.config.layers[i].mixers]
 
     # ---- cost accounting
     def num_active_matmul_params(self):
@@ -363,48 +617,46 @@ class LayerStack(nn.Module):
         W, total = self.config.n_embd, self.config.vocab_size * self.config.n_embd
         for i, _, _ in self.run_list:
             layer = self.config.layers[i]
-            skip = ("uk", "uv", "dkv.norm")      # applied per key or query: in the mixer's own count
-            total += sum(math.prod(s) for k, s in layer.mixer.tensors(W).items() if k not in skip)
+            for m in layer.mixers:
+                total += sum(math.prod(s) for k, s in m.tensors(W).items() if len(s) == 2 and k not in m.per_key + m.fp32)
             total += layer.ff.active_params(W) if layer.ff is not None else 0
         return total
 
     def estimate_decode_flops(self, context_len):
-        return 2 * self.num_active_matmul_params() + sum(self.config.layers[i].mixer.flops(context_len) for i, _, _ in self.run_list)
+        return 2 * self.num_active_matmul_params() + sum(m.flops(context_len) for m in self.run_mixers())
 
     def estimate_prefill_flops(self, num_tokens):
-        return 2 * self.num_active_matmul_params() * num_tokens + sum(self.config.layers[i].mixer.prefill_flops(num_tokens) for i, _, _ in self.run_list)
+        return 2 * self.num_active_matmul_params() * num_tokens + sum(m.prefill_flops(num_tokens) for m in self.run_mixers())
 
     def kv_bytes_per_token(self):
         """Cache bytes that grow with the sequence (a recurrent state does not)."""
         es = self.dtype.itemsize
-        return sum(self.config.layers[i].mixer.read_elements(1)[0] for i, _, _ in self.run_list) * es
+        return sum(m.read_elements(1)[0] for m in self.run_mixers()) * es
 
     def kv_read_bytes(self, context_len):
         """Cache bytes one decode step reads or writes per row."""
-        parts = [self.config.layers[i].mixer.read_elements(context_len) for i, _, _ in self.run_list]
+        parts = [m.read_elements(context_len) for m in self.run_mixers()]
         return sum(p[0] for p in parts) * self.dtype.itemsize + sum(p[1] for p in parts) * 4
 
     def streamed_weight_bytes(self):
         """Weight bytes one single-row decode step reads."""
-        per_head = sum(math.prod(s) for i, _, _ in self.run_list for k, s in self.config.layers[i].mixer.tensors(self.config.n_embd).items() if k in ("uk", "uv"))
+        per_head = sum(math.prod(s) for m in self.run_mixers() for k, s in m.tensors(self.config.n_embd).items() if k in m.per_key)
         return (self.num_active_matmul_params() + per_head) * self.dtype.itemsize
 
     def describe(self):
-        kinds = [type(layer.mixer).__name__ for layer in self.config.layers]
+        kinds = [" + ".join(type(m).__name__ for m in layer.mixers) for layer in self.config.layers]
         mix = ", ".join(f"{kinds.count(k)} {k}" for k in dict.fromkeys(kinds))
         return f"layers {len(kinds)} ({mix}), {len(self.run_list)} layer runs, dim {self.config.n_embd}"
 
     # ---- plan
-    def _rope_table(self, base, dims):
-        """cos, sin of position * base^(-2i/dims), fp32 [len, dims/2, 2] (worked out in fp64: an angle of thousands of radians keeps its
+    def _rope_table(self, rotation):
+        """cos, sin of position * frequency, fp32 [len, dims/2, 2] (worked out in fp64: an angle of thousands of radians keeps its
         fraction)."""
-        key = (base, dims)
-        t = self._rope.get(key)
+        t = self._rope.get(rotation)
         if t is None:
             dev = self.get_device()
-            i = torch.arange(dims // 2, dtype=torch.float64, device=dev)
-            ang = torch.outer(torch.arange(self._rope_len, dtype=torch.float64, device=dev), base ** (-2.0 * i / max(dims, 1)))
-            t = self._rope[key] = torch.stack([ang.cos(), ang.sin()], dim=-1).float().contiguous()
+            ang = torch.outer(torch.arange(self._rope_len, dtype=torch.float64, device=dev), rotation.frequencies().to(dev))
+            t = self._rope[rotation] = torch.stack([ang.cos(), ang.sin()], dim=-1).float().contiguous()
         return t
 
     def _build_plan(self):
@@ -420,39 +672,59 @@ class LayerStack(nn.Module):
             keep.append(t)
             return t.data_ptr()
 
+        def norm_weight(name):
+            return own(padded(w[name].float() + cfg.norm_offset, Wp), torch.float32)
+
+        def pick(prefix, fp32=()):
+            mine = {k[len(prefix):]: v for k, v in w.items() if k.startswith(prefix)}
+            return {k: v.to(self.dtype) if v.dim() > 1 and k not in fp32 else v for k, v in mine.items()}
+
         layers = (_lib.StackLayer * cfg.n_layer)()
         for i, spec in enumerate(cfg.layers):
-            d, mixer, ff = layers[i], spec.mixer, spec.ff
-            pick = lambda prefix: {k[len(prefix):]: v.to(self.dtype) if v.dim() > 1 else v for k, v in w.items() if k.startswith(prefix)}  # noqa: E731
-            rows, cols, extra = mixer.pack(pick(f"l{i}.mix."))
-            rows, cols = [padded(rows, rows.shape[0], Wp)], [padded(cols, Wp, mixer.mix_out)]
-            d.mixer, d.heads, d.mix_cols, d.mix_out = mixer.kind, mixer.heads, mixer.mix_cols, mixer.mix_out
-            mixer.describe(d)
+            d, ff = layers[i], spec.ff
+            rows, cols, extra = [], [], {}
+            d.block, d.n_mixers = BLOCKS[cfg.block], len(spec.mixers)
+            assert d.n_mixers <= _lib.STACK_MAX_MIXERS
+            for j, (prefix, mixer) in enumerate(spec.mixer.parts):
+                md = d.mix[j]
+                r, c, more = mixer.pack(pick(f"l{i}.mix.{prefix}", mixer.fp32))
+                rows.append(padded(r, r.shape[0], Wp))
+                cols.append(padded(c, Wp, mixer.out))
+                md.kind, md.cols, md.out, md.out_scale, md.rot_dims = mixer.kind, mixer.cols, mixer.out, mixer.out_scale, mixer.rotation.dims
+                mixer.describe(md)
+                for name, t in more.items():
+                    setattr(md, name, own(t, self.dtype if name in WEIGHT_FIELDS else torch.float32))
+                d.mix_cols += mixer.cols
+                d.mix_out += mixer.out
             if ff is not None:
-                router, first, last, more = ff.pack(pick(f"l{i}.mlp."), Wp)
-                rows += [t for t in (router, first) if t is not None]
-                cols += [t for t in (last,) if t is not None]
-                extra |= more
+                router, first, last, extra = ff.pack(pick(f"l{i}.mlp."), Wp)
                 d.ff, d.router_cols, d.ff_cols, d.ff_p = ff.kind, ff.router_cols, ff.ff_cols, ff.ff_p
                 ff.describe(d)
-            d.n_in, d.k_out = d.mix_cols + d.router_cols + d.ff_cols, d.mix_out + d.ff_p
+                if cfg.block == "post_norm":
+                    d.w_ff_in, d.w_ff_out, d.norm2_w = own(first, self.dtype), own(last, self.dtype), norm_weight(f"l{i}.norm2")
+                else:
+                    rows += [t for t in (router, first) if t is not None]
+                    cols += [t for t in (last,) if t is not None]
+            d.n_in, d.k_out = sum(t.shape[0] for t in rows), sum(t.shape[1] for t in cols)
             d.w_in, d.w_out = own(torch.cat(rows), self.dtype), own(torch.cat(cols, dim=1), self.dtype)
-            d.norm_w = own(padded(w[f"l{i}.norm1"].float(), Wp), torch.float32)
+            d.norm_w = norm_weight(f"l{i}.norm1")
             for name, t in extra.items():
-                setattr(d, name, own(t, torch.float32 if name in ("kv_norm_w", "decay") else self.dtype))
+                setattr(d, name, own(t, self.dtype))
         runs = (_lib.StackRun * len(self.run_list))()
-        used = {0: 0, 1: 0}
+        used = {ROW_CACHE: 0, STATE_CACHE: 0}
         for r, (i, again, step) in zip(runs, self.run_list):
-            kind = cfg.layers[i].mixer.kind
-            r.layer, r.slot, r.add_embedding, r.step = i, used[kind], int(again), step
-            used[kind] += 1
+            r.layer, r.add_embedding, r.step = i, int(again), step
+            for j, mixer in enumerate(cfg.layers[i].mixers):
+                r.slot[j] = used[mixer.cache]
+                used[mixer.cache] += 1
         md = _lib.StackModel()
         md.dtype, md.width, md.width_p, md.vocab = ops.STACK_DTYPES[self.dtype], cfg.n_embd, Wp, cfg.vocab_size
         md.n_layers, md.n_runs, md.max_k_out = cfg.n_layer, len(self.run_list), max(d.k_out for d in layers)
+        md.norm = NORMS[cfg.norm]
         md.eps, md.embed_scale, md.logit_scale, md.logit_softcap = cfg.eps, cfg.embed_scale, cfg.logit_scale, cfg.logit_softcap
         md.embed = own(padded(w["embed"], cfg.vocab_size, Wp), self.dtype)
-        md.head = own(padded(w["head"], cfg.vocab_size, Wp), self.dtype)
-        md.final_norm_w = own(padded(w["final.norm"].float(), Wp), torch.float32)
+        md.head = md.embed if cfg.tied_head else own(padded(w["head"], cfg.vocab_size, Wp), self.dtype)
+        md.final_norm_w = norm_weight("final.norm")
         if cfg.loop_steps:
             md.steps = own(padded(w["loop.step"].float(), cfg.loop_times, Wp), torch.float32)
         md.layers, md.runs = C.cast(layers, C.POINTER(_lib.StackLayer)), C.cast(runs, C.POINTER(_lib.StackRun))
@@ -470,7 +742,8 @@ class LayerStack(nn.Module):
             self._rope_len = round_up(positions, 1024)
             self._rope = {}
             for d, spec in zip(layers, self.config.layers):
-                d.rope = self._rope_table(spec.mixer.rot_base, spec.mixer.rot_dims).data_ptr()
+                for md_mix, mixer in zip(d.mix, spec.mixers):
+                    md_mix.rope = self._rope_table(mixer.rotation).data_ptr() if mixer.rotation.dims else None
             md.rope_len = self._rope_len
         return md
 
@@ -512,7 +785,7 @@ class LayerStack(nn.Module):
         logits = torch.empty(n_logits, self.config.vocab_size, dtype=torch.float32, device=idx.device)
         tap = torch.empty(len(self.run_list), B, T, self.width_p, dtype=torch.float32, device=idx.device) if taps else None
         cd = _lib.StackCacheDesc()
-        cd.latents, cd.state_in, cd.state_out = kv_cache.pointers()
+        cd.rows, cd.state_in, cd.state_out = kv_cache.pointers()
         cd.cache_seqlens = kv_cache.cache_seqlens.data_ptr()
         cd.batch, cd.max_seq_len, cd.pos_max = B, kv_cache.max_seq_len, pos_max
         cd.advance = T if rows is None else 0

@@ -87,7 +87,7 @@ def bench_palilix(width, device, groups):
         shapes = {}
         for layer in sc.layers:
             m, f = layer.mixer, layer.ff
-            n_in, k_out = m.mix_cols + f.router_cols + f.ff_cols, m.mix_out + f.ff_p
+            n_in, k_out = m.cols + f.router_cols + f.ff_cols, m.out + f.ff_p
             kind = f"{type(m).__name__}+{type(f).__name__}"
             shapes[f"{kind} in"], shapes[f"{kind} out"] = (n_in, Wp, rows), (Wp, k_out, rows)
         if decode:
@@ -120,7 +120,7 @@ def bench_palilix(width, device, groups):
         res["prefill"][T] = {"ms": round(s * 1e3, 3), "tokens_per_s": round(T / s, 1), "kernels": kernels(T, False)}
     for B in DECODE:
         cache = model.new_cache(B, CONTEXT + 64)
-        for t in cache.latents:
+        for t in cache.rows:
             t.normal_(generator=g)
         cache.cache_seqlens.fill_(CONTEXT - 32)
         cache._host_pos = [CONTEXT - 32] * B

@@ -28,7 +28,7 @@ def test_stack_library_exports_what_the_header_declares():
     names = sorted(set(re.findall(r"\b(nc_[a-z0-9_]+)\s*\(", re.sub(r"/\*.*?\*/", "", text, flags=re.S))))
     lib = ctypes.CDLL(_lib._load("stack")._name)
     assert sorted(_lib.STACK_EXPORTS) == names and all(hasattr(lib, n) for n in names)
-    assert _lib.stack_lib().nc_stack_abi_version() == 1
+    assert _lib.stack_lib().nc_stack_abi_version() == 2
 
 
 def _header():
@@ -67,7 +67,7 @@ def test_tensor_table_and_sizes(name):
     assert [(i, t if t >= 0 else None) for i, _, t in sc.runs()] == ref.layer_runs(cfg)
     assert [again for _, again, _ in sc.runs()] == [bool(t) for _, t in ref.layer_runs(cfg)]
     for layer in sc.layers:
-        assert layer.mixer.mix_out % 64 == 0 and layer.mixer.mix_cols % 16 == 0
+        assert layer.mixer.out % 64 == 0 and layer.mixer.cols % 16 == 0
         if isinstance(layer.mixer, LatentAttention):
             assert layer.mixer.vdim_p >= layer.mixer.vdim and layer.mixer.rank_p % 64 == 0
         else:
@@ -188,7 +188,7 @@ def new_cache(rows=3, seq_len=16):
 
 def test_cache_positions_and_state_buffers():
     c = new_cache()
-    assert [t.shape for t in c.latents] == [(3, 16, 8), (3, 16, 24)] and [s.shape for s in c.states[0]] == [(3, 2, 4, 4)]
+    assert [t.shape for t in c.rows] == [(3, 16, 8), (3, 16, 24)] and [s.shape for s in c.states[0]] == [(3, 2, 4, 4)]
     first_in, first_out = c.state_buffers()
     c.advance(5)
     assert c.get_pos() == 5 and c.cache_seqlens.tolist() == [5, 5, 5]

@@ -2,6 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W]
     python bench.py --palilix                 (another workload: the Palilix design beside the GPT, see nanochat_amd/stack_bench.py)
+    python bench.py --zodirax                 (likewise: the Zodirax design beside a dense Palilix and the GPT)
 
 Workload (the headline decode configuration, whatever K and W are): nanochat d26 (n_embd 1664, 13 heads, head_dim 128,
 26 layers, vocab 32768, window pattern SSSL), bf16 weights with FP8 linears, random init seed 2; one prompt of 1792 random
@@ -482,6 +483,8 @@ def main():
     ap.add_argument("--palilix", action="store_true",
                     help="instead of the headline workload: prefill and decode throughput of the Palilix design at widths 2048 and 4096, "
                          "beside the FP8 GPT of equal width and layers, every kind of kernel against its roofline")
+    ap.add_argument("--zodirax", action="store_true",
+                    help="the same for the Zodirax design, beside a Palilix of dense layers and the FP8 GPT of equal width and layers")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (decode would shard by batch row, one independent copy per GPU). "
@@ -493,12 +496,14 @@ def main():
     device = torch.device("cuda:0")
     torch.cuda.set_device(device)
 
-    if args.palilix:
+    if args.palilix or args.zodirax:
         from nanochat_amd import stack_bench
-        r = stack_bench.run(device)
-        print(json.dumps({"metric": "palilix decode tokens/sec @ width 2048, 8 layers, bs64 ctx2048", "unit": "tokens/s", "n_gpus": 1,
-                          "value": r["width 2048"]["palilix"]["decode"][64]["tokens_per_s"], "higher_is_better": True, "vs_baseline": None,
-                          "dtype": "bf16 (linears, latents), fp32 (residual, scores, states)", "data": "synthetic: random token ids, random weights",
+        name = "palilix" if args.palilix else "zodirax"
+        r = (stack_bench.run_palilix if args.palilix else stack_bench.run_zodirax)(device)
+        kept = "latents" if args.palilix else "keys and values"
+        print(json.dumps({"metric": f"{name} decode tokens/sec @ width 2048, 8 layers, bs64 ctx2048", "unit": "tokens/s", "n_gpus": 1,
+                          "value": r["width 2048"][name]["decode"][64]["tokens_per_s"], "higher_is_better": True, "vs_baseline": None,
+                          "dtype": f"bf16 (linears, {kept}), fp32 (residual, scores, states)", "data": "synthetic: random token ids, random weights",
                           "config": {"context": stack_bench.CONTEXT, "prefill_tokens": list(stack_bench.PREFILL)}, "results": r}))
         return
     K, W = args.steps, max(1, args.warmup)

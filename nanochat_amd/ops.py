@@ -494,11 +494,11 @@ def stack_cache_copy(src, dst, n):
 
 def stack_linear(a, w, kind=0, limit=0.0, kernel=0):
     """a [M, K] w [N, K]^T in the storage type of both, 32-bit sums (nc_stack_linear).  kind: 0 plain, 1 tanh-form gelu, 2 clamped GLU of
-    interleaved (gate, up) rows of w, 3 float output; kernel: 0 choose, 1 the few-rows kernel, 2 the tiled one (3, 4: its 64 x 128, 128 x 256 tiles)."""
+    interleaved (gate, up) rows of w, 3 float output, 6 silu, 7 silu(gate) * up of interleaved rows; kernel: 0 choose, 1 the few-rows kernel, 2 the tiled one (3, 4: its 64 x 128, 128 x 256 tiles)."""
     _need_cuda(a, w)
     (M, K), N = a.shape, w.shape[0]
     assert w.shape[1] == K and a.dtype == w.dtype and a.is_contiguous() and w.is_contiguous()
-    out = torch.empty(M, N // 2 if kind == 2 else N, dtype=torch.float32 if kind == 3 else a.dtype, device=a.device)
+    out = torch.empty(M, N // 2 if kind in (2, 7) else N, dtype=torch.float32 if kind == 3 else a.dtype, device=a.device)
     rc = _lib.stack_lib().nc_stack_linear(STACK_DTYPES[a.dtype], _ptr(a), K, _ptr(w), _ptr(out), out.shape[1], M, N, K, kind, limit, kernel, _stream())
     _lib.check(rc, _lib.stack_lib())
     return out

@@ -1,8 +1,9 @@
-"""Prefill and decode throughput of Palilix at sizes like a real model's layers (random weights), beside the FP8 GPT of equal width and
-number of layers, with each kind of kernel against its roofline.  Run through `bench.py --palilix`.
+"""Prefill and decode throughput of the layer-stack designs at sizes like a real model's layers (random weights), with each kind of kernel
+against its roofline: Palilix beside the FP8 GPT of equal width and number of layers (`bench.py --palilix`), Zodirax beside a Palilix of
+dense layers and the GPT (`bench.py --zodirax`).
 
 Rooflines: HBM 8 TB/s for kernels that stream weights, cached rows or states; the dense matrix peak of the operands' format (bf16 2.5,
-fp8 5.0 PFLOP/s) for products of many rows.  Algorithmic bytes and flops: every weight, cached row and state once, causal pairs only, and
+fp8 5.0 PFLOP/s) for products of many rows.  Algorithmic bytes and flops: every weight, cached row and state once, visible pairs only, and
 no credit for what a kernel repeats for exactness.  Kernel times are HIP event pairs around each launch.
 """
 import ctypes as C
@@ -15,8 +16,9 @@ from .common import PEAK_BF16_FLOPS, PEAK_FP8_FLOPS, PEAK_HBM_BYTES_PER_S
 from .engine import KVCache
 from .gpt import GPTConfig
 from .palilix import Palilix
-from .stack import Experts, LatentAttention
-from .synthetic import palilix_config, random_init_model, random_stack_model
+from .stack import Experts, SelectiveScan
+from .synthetic import palilix_config, random_init_model, random_stack_model, zodirax_config
+from .zodirax import Zodirax
 
 PREFILL = (1792,)
 DECODE = (1, 16, 64)
@@ -76,38 +78,62 @@ def _linears(lib, shapes, decode, peak, weight_bytes):
     return out
 
 
-def bench_palilix(width, device, groups):
-    cfg = palilix_config(width, width // 128, vocab=VOCAB, groups=groups)
-    model = random_stack_model(Palilix, cfg, device)
+def _stack_shapes(sc, Wp):
+    """{names: (N, K)} of the weights of a stack's layers; weights of one shape are one entry."""
+    shapes = {}
+
+    def add(name, N, K):
+        names = shapes.setdefault((N, K), [])
+        if name not in names:
+            names.append(name)
+    for layer in sc.layers:
+        f, kind = layer.ff, "+".join(type(m).__name__ for m in layer.mixers)
+        n_in, k_out = sum(m.cols for m in layer.mixers), sum(m.out for m in layer.mixers)
+        if f is not None and sc.block == "post_norm":
+            add(f"{type(f).__name__} in", f.ff_cols, Wp)
+            add(f"{type(f).__name__} out", Wp, f.ff_p)
+        elif f is not None:
+            kind += f"+{type(f).__name__}"
+            n_in, k_out = n_in + f.router_cols + f.ff_cols, k_out + f.ff_p
+        add(f"{kind} in", n_in, Wp)
+        add(f"{kind} out", Wp, k_out)
+        for m in layer.mixers:
+            if isinstance(m, SelectiveScan):
+                add("scan x", m.dt_rank_p + 2 * m.bc_p, m.inner_p)
+                add("scan dt", m.inner_p, m.dt_rank_p)
+    return {" / ".join(names): shape for shape, names in shapes.items()}
+
+
+# timing class of the library -> (name, bound of a prompt, bound of decoding)
+STACK_CLASSES = {0: ("latent attention", "mfma", "hbm"), 2: ("retention", "hbm", "hbm"), 5: ("window attention", "mfma", "hbm"), 6: ("selective scan", "hbm", "hbm")}
+
+
+def bench_stack(cls, cfg, device):
+    model = random_stack_model(cls, cfg, device)
     lib = _lib.stack_lib()
     sc, Wp = model.config, model.width_p
     g = torch.Generator(device=device).manual_seed(1)
 
     def kernels(rows, decode):
-        shapes = {}
-        for layer in sc.layers:
-            m, f = layer.mixer, layer.ff
-            n_in, k_out = m.cols + f.router_cols + f.ff_cols, m.out + f.ff_p
-            kind = f"{type(m).__name__}+{type(f).__name__}"
-            shapes[f"{kind} in"], shapes[f"{kind} out"] = (n_in, Wp, rows), (Wp, k_out, rows)
+        shapes = {name: (N, K, rows) for name, (N, K) in _stack_shapes(sc, Wp).items()}
         if decode:
             shapes["head"] = (VOCAB, Wp, rows)          # (a prompt has one row of logits)
         out = _linears(lib, shapes, decode, PEAK_BF16_FLOPS, 2)
-        ms, units, n = _read(lib, 0)
-        out["latent attention"] = _entry(ms, units, n, PEAK_HBM_BYTES_PER_S if decode else PEAK_BF16_FLOPS, "hbm" if decode else "mfma")
-        ms, units, n = _read(lib, 2)
-        out["retention"] = _entry(ms, units, n, PEAK_HBM_BYTES_PER_S, "hbm")       # at prefill: projections, outputs, four passes over chunk states
-        ms, units, n = _read(lib, 4)
-        ff = next(l.ff for l in sc.layers if isinstance(l.ff, Experts))
-        # how many experts a step touches, on average, if every choice is as likely
-        touched = ff.experts * (1 - (1 - ff.top / ff.experts) ** rows)
-        out["experts"] = _entry(ms, n / 2 * touched * 3 * ff.expert_ff_p * Wp * 2 if decode else units, n, PEAK_HBM_BYTES_PER_S if decode else PEAK_BF16_FLOPS,
-                                "hbm" if decode else "mfma")
+        for c, (name, prompt, single) in STACK_CLASSES.items():
+            bound = single if decode else prompt
+            out[name] = _entry(*_read(lib, c), PEAK_HBM_BYTES_PER_S if bound == "hbm" else PEAK_BF16_FLOPS, bound)
+        ff = next((l.ff for l in sc.layers if isinstance(l.ff, Experts)), None)
+        if ff is not None:
+            ms, units, n = _read(lib, 4)
+            # how many experts a step touches, on average, if every choice is as likely
+            touched = ff.experts * (1 - (1 - ff.top / ff.experts) ** rows)
+            out["experts"] = _entry(ms, n / 2 * touched * 3 * ff.expert_ff_p * Wp * 2 if decode else units, n, PEAK_HBM_BYTES_PER_S if decode else PEAK_BF16_FLOPS,
+                                    "hbm" if decode else "mfma")
         out["row kernels ms per step"] = round(_read(lib, 3)[0] / 4, 4)
         lib.nc_profile_enable(0)
         return {k: v for k, v in out.items() if v is not None}
 
-    res = {"layers": len(sc.layers), "width": width, "parameters": sum(p.numel() for p in model.parameters()), "prefill": {}, "decode": {}}
+    res = {"layers": len(sc.layers), "width": cfg["width"], "parameters": sum(p.numel() for p in model.parameters()), "prefill": {}, "decode": {}}
     for T in PREFILL:
         ids = torch.randint(0, VOCAB, (1, T), device=device, generator=g)
         cache = model.new_cache(1, T)
@@ -130,7 +156,6 @@ def bench_palilix(width, device, groups):
         _profiled(lib, lambda: model.forward_last(tok, kv_cache=cache))
         res["decode"][B] = {"ms": round(s * 1e3, 4), "tokens_per_s": round(B / s, 1), "kernels": kernels(B, True)}
         del cache
-    assert any(isinstance(l.mixer, LatentAttention) for l in sc.layers)
     return res
 
 
@@ -179,12 +204,27 @@ def bench_gpt(width, device, layers):
     return res
 
 
-def run(device, widths=(2048, 4096)):
+def _groups(width):
+    return 2 if width <= 2048 else 1
+
+
+def run_palilix(device, widths=(2048, 4096)):
     out = {}
     for width in widths:
-        groups = 2 if width <= 2048 else 1
-        p = bench_palilix(width, device, groups)
+        p = bench_stack(Palilix, palilix_config(width, width // 128, vocab=VOCAB, groups=_groups(width)), device)
         torch.cuda.empty_cache()
         out[f"width {width}"] = {"palilix": p, "gpt": bench_gpt(width, device, p["layers"])}
+        torch.cuda.empty_cache()
+    return out
+
+
+def run_zodirax(device, widths=(2048, 4096)):
+    out = {}
+    for width in widths:
+        z = bench_stack(Zodirax, zodirax_config(width, width // 128, vocab=VOCAB, groups=_groups(width)), device)
+        torch.cuda.empty_cache()
+        p = bench_stack(Palilix, palilix_config(width, width // 128, vocab=VOCAB, groups=_groups(width), dense=True), device)
+        torch.cuda.empty_cache()
+        out[f"width {width}"] = {"zodirax": z, "palilix, dense": p, "gpt": bench_gpt(width, device, z["layers"])}
         torch.cuda.empty_cache()
     return out

@@ -53,11 +53,13 @@ def random_init_model(cfg, device, seed=0):
     return model
 
 
-def palilix_config(width, heads, rank=512, experts=64, top=6, expert_ff=1024, vocab=32768, groups=1):
+def palilix_config(width, heads, rank=512, experts=64, top=6, expert_ff=1024, vocab=32768, groups=1, dense=False):
     """A Palilix configuration with the proportions of an ordinary model of this width: `groups` times (latent attention + dense,
-    retention + experts twice, latent attention + experts), heads of 128, no repeated layers."""
+    retention + experts twice, latent attention + experts), heads of 128, no repeated layers; `dense`: no experts."""
     head = width // heads
     moe = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "router": {"experts": experts, "top": top}, "shared": {"ff": 2 * expert_ff, "limit": 7.0}}
+    if dense:
+        moe = {"kind": "dense", "ff": 4 * width}
     lat = {"heads": heads, "dim": head, "rot_dim": head // 2, "vdim": head, "kv_rank": rank, "scale": (1.5 * head) ** -0.5,
            "rot": {"base": 10000.0, "dims": head // 2}}
     ret = {"heads": heads, "dim": head, "vdim": head, "decay": [1 - 2.0 ** -(5 + 6 * i / max(1, heads - 1)) for i in range(heads)],
@@ -66,6 +68,20 @@ def palilix_config(width, heads, rank=512, experts=64, top=6, expert_ff=1024, vo
              {"type": "retention", "mixer": ret, "mlp": moe}, {"type": "latent_attention", "mixer": lat, "mlp": moe}]
     return {"architecture": "Palilix", "embedding": {"scale": 1.0}, "layers": group * groups, "logit_scale": 1.0, "logit_softcap": 30.0,
             "norm": {"eps": 1e-6}, "vocab": vocab, "width": width}
+
+
+def zodirax_config(width, heads, window=1024, vocab=32768, groups=1):
+    """A Zodirax configuration with the proportions of an ordinary model of this width: `groups` times (window attention beside lightning
+    attention, selective scan twice, the first again), heads of 128, four query heads per key head, SwiGLU of 8/3 of the width."""
+    head = width // heads
+    left = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head, "vdim": head, "scale": head ** -0.5, "mask": {"size": window, "keep_first": 4},
+            "rot": {"base": 500000.0, "dims": head, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    right = {"heads": heads, "dim": head, "vdim": head, "decay": [1 - 2.0 ** -(5 + 6 * i / max(1, heads - 1)) for i in range(heads)]}
+    ff = {"kind": "dense", "ff": round(8 * width / 3 / 128) * 128}
+    pair = {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.5, "right_scale": 0.5}, "mlp": ff}
+    scan = {"type": "mamba1", "mixer": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4}, "mlp": ff}
+    return {"architecture": "Zodirax", "embedding": {"scale": 1.0}, "layers": [pair, scan, scan, pair] * groups, "norm": {"eps": 1e-6}, "vocab": vocab,
+            "width": width}
 
 
 def random_stack_model(cls, cfg, device, dtype=torch.bfloat16, seed=0):
@@ -78,8 +94,12 @@ def random_stack_model(cls, cfg, device, dtype=torch.bfloat16, seed=0):
         t = torch.empty(shape, dtype=torch.bfloat16, device=device)
         if name == "embed" or name == "loop.step":
             t.normal_(0.0, 1.0, generator=g)
+        elif name.endswith("A_log"):
+            t.copy_(torch.arange(1, shape[1] + 1, device=device).log().expand(shape))
+        elif name.endswith(".dt.b"):
+            t.fill_(-4.0)
         elif len(shape) == 1:
-            t.fill_(1.0)
+            t.fill_(0.0 if model.config.norm_offset and "norm" in name and ".mix." not in name else 1.0)
         else:
             t.normal_(0.0, shape[-1] ** -0.5, generator=g)
         tensors[name] = t

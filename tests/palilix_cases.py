@@ -109,14 +109,3 @@ def weights(cfg, seed=0):
             t = t * (1.4 / math.sqrt(shape[-1]))
         out[name] = t.bfloat16()
     return out
-
-
-def tokens(cfg, n, seed=1):
-    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(seed)).tolist()
-
-
-def rel_rms(got, want):
-    """Per position: root mean square of the difference over that of the (centred) logits."""
-    got, want = got.double().cpu(), want.double()
-    scale = (want - want.mean(-1, keepdim=True)).pow(2).mean().sqrt()
-    return ((got - want).pow(2).mean(-1).sqrt() / scale)

@@ -2,7 +2,6 @@
 unequal sequences, slots that are used again, generation through the Engine; both storage types."""
 import functools
 import json
-import struct
 
 import pytest
 import torch
@@ -13,17 +12,10 @@ from nanochat_amd.palilix import Palilix
 from nanochat_amd.registry import load_model
 from nanochat_amd.synthetic import SyntheticTokenizer
 from oracle import palilix_ref as ref
-from palilix_cases import CASES, config, dense, latent, moe, rel_rms, retention, tokens, variant, weights
+from palilix_cases import CASES, config, dense, latent, moe, retention, variant, weights
+from stack_helpers import BAR, DEV, DTYPES, build_model, check, ids, judge, rel_rms, run, say, tokens, trace_runner, write_model
 
 pytestmark = pytest.mark.gpu
-DEV = "cuda"
-DTYPES = [torch.float32, torch.bfloat16]
-# difference from the oracle per position (root mean square over the vocabulary, relative): 32-bit rounding, bf16 rounding
-BAR = {torch.float32: 2e-5, torch.bfloat16: 4e-2}
-
-
-def say(msg):
-    print(f"[gpu-case] {msg}", flush=True)
 
 
 @functools.lru_cache(maxsize=None)
@@ -43,43 +35,12 @@ def case_model(name, dtype):
 
 
 def build(cfg, w, dtype):
-    with torch.device("meta"):
-        model = Palilix.from_config(cfg, dtype)
-    return model.load_tensors(w, DEV)
-
-
-def ids(toks):
-    return torch.tensor([toks], dtype=torch.long, device=DEV)
-
-
-def run(model, toks, cuts, seq_len=None):
-    """Logits [T, vocab] of one sequence brought in portions of the given sizes."""
-    cache = model.new_cache(1, seq_len or len(toks))
-    out, at = [], 0
-    for n in cuts:
-        out.append(model.forward(ids(toks[at:at + n]), kv_cache=cache)[0].clone())
-        at += n
-    assert at == len(toks) == cache.get_pos() == int(cache.cache_seqlens[0])
-    return torch.cat(out)
-
-
-def judge(err, dtype, what, bar=None):
-    """Every position below the bar in 32-bit.  In bf16 one position in thirty (or one) may lie over it, up to ten times: where two experts
-    score almost alike, or a head's output is almost zero before its norm, a rounded input turns into another answer."""
-    bar = bar or BAR[dtype]
-    worst, over = err.max().item(), int((err > bar).sum())
-    print(f"{what} {str(dtype)[6:]}: worst position {worst:.2e}, {over} of {err.numel()} over {bar:.0e}", flush=True)
-    allowed = 0 if dtype == torch.float32 else max(1, err.numel() // 30)
-    assert worst == worst and over <= allowed and worst <= (bar if allowed == 0 else 10 * bar), f"{what}: worst at {err.argmax().item()}"
-
-
-def check(got, want, dtype, what, bar=None):
-    judge(rel_rms(got, want), dtype, what, bar)
+    return build_model(Palilix, cfg, w, dtype)
 
 
 # ------------------------------------------------------------------------------------------------ linears
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("kind", [0, 1, 2, 3])
+@pytest.mark.parametrize("kind", [0, 1, 2, 3, 6, 7])
 def test_linear_kernels(dtype, kind):
     say(f"linears, kind {kind}, {dtype}")
     g = torch.Generator().manual_seed(kind)
@@ -90,6 +51,10 @@ def test_linear_kernels(dtype, kind):
             want = ref.gelu_tanh(want)
         elif kind == 2:
             want = ref.clamped_glu(want[:, 0::2], want[:, 1::2], 0.6)
+        elif kind == 6:
+            want = ref.silu(want)
+        elif kind == 7:
+            want = ref.silu(want[:, 0::2]) * want[:, 1::2]
         for kernel in (1, 2, 3, 4):
             got = ops.stack_linear(a.to(DEV), w.to(DEV), kind=kind, limit=0.6, kernel=kernel).cpu()
             tol = 1e-2 if got.dtype == torch.bfloat16 else 2e-5
@@ -370,17 +335,6 @@ def test_chosen_places_and_errors():
 
 
 # ------------------------------------------------------------------------------------------------ generation
-def write_model(path, cfg, w):
-    blob, header = b"", {}
-    for k, t in w.items():
-        data = t.contiguous().view(torch.int16).numpy().tobytes()
-        header[k] = {"dtype": "BF16", "shape": list(t.shape), "data_offsets": [len(blob), len(blob) + len(data)]}
-        blob += data
-    head = json.dumps(header).encode()
-    (path / "model.safetensors").write_bytes(struct.pack("<Q", len(head)) + head + blob)
-    (path / "config.json").write_text(json.dumps(cfg))
-
-
 def test_greedy_generation_through_the_engine(tmp_path):
     """A folder on disk, the registry, the Engine's scheduler, the sampler: the ids are the oracle's greedy ids (32-bit)."""
     say("greedy generation")
@@ -457,14 +411,7 @@ def test_forced_tokens_take_the_step_back():
 def test_trace_replay(tmp_path):
     """bin/trace_run's own replay loop on two requests, one after the other, with a cache that is handed on."""
     say("trace replay")
-    import importlib.machinery
-    import importlib.util
-    import os
-    path = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "bin", "trace_run")
-    loader = importlib.machinery.SourceFileLoader("trace_run", path)
-    spec = importlib.util.spec_from_loader("trace_run", loader)
-    mod = importlib.util.module_from_spec(spec)
-    loader.exec_module(mod)
+    mod = trace_runner()
     cfg, model = CASES["odd"], case_model("odd", torch.float32)
     toks = tokens(cfg, 45)
     want = oracle_logits("odd", 45)

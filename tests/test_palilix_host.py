@@ -14,7 +14,8 @@ from nanochat_amd.engine import Engine, StackCache
 from nanochat_amd.palilix import Palilix, stack_config
 from nanochat_amd.stack import Experts, LatentAttention, LayerStack, Retention
 from oracle import palilix_ref as ref
-from palilix_cases import CASES, config, latent, moe, rel_rms, retention, tensor_shapes, tokens, variant, weights
+from palilix_cases import CASES, config, latent, moe, retention, tensor_shapes, variant, weights
+from stack_helpers import rel_rms, tokens
 
 
 def meta_model(cfg, dtype=torch.float32):
@@ -44,12 +45,14 @@ def test_struct_layouts_match_the_header(tmp_path):
     """Sizes and a few offsets as the C compiler lays them out."""
     import subprocess
     src = tmp_path / "s.c"
-    src.write_text('#include <stdio.h>\n#include "%s"\nint main(){printf("%%zu %%zu %%zu %%zu %%zu %%zu", sizeof(nc_stack_layer), sizeof(nc_stack_run),'
-                   'sizeof(nc_stack_model), sizeof(nc_stack_cache), offsetof(nc_stack_layer, norm_w), offsetof(nc_stack_model, embed));}' % _header())
+    src.write_text('#include <stdio.h>\n#include "%s"\nint main(){printf("%%zu %%zu %%zu %%zu %%zu %%zu %%zu %%zu %%zu", sizeof(nc_stack_layer), sizeof(nc_stack_run),'
+                   'sizeof(nc_stack_model), sizeof(nc_stack_cache), offsetof(nc_stack_layer, mix), offsetof(nc_stack_model, embed),'
+                   'sizeof(nc_stack_mixer), offsetof(nc_stack_mixer, kv_norm_w), offsetof(nc_stack_mixer, skip));}' % _header())
     subprocess.run(["gcc", str(src), "-o", str(tmp_path / "s")], check=True)
     got = [int(x) for x in subprocess.run([str(tmp_path / "s")], capture_output=True, text=True, check=True).stdout.split()]
     assert got == [ctypes.sizeof(_lib.StackLayer), ctypes.sizeof(_lib.StackRun), ctypes.sizeof(_lib.StackModel), ctypes.sizeof(_lib.StackCacheDesc),
-                   _lib.StackLayer.norm_w.offset, _lib.StackModel.embed.offset]
+                   _lib.StackLayer.mix.offset, _lib.StackModel.embed.offset, ctypes.sizeof(_lib.StackMixer), _lib.StackMixer.kv_norm_w.offset,
+                   _lib.StackMixer.skip.offset]
 
 
 def test_errors_come_before_any_gpu_call():

@@ -8,7 +8,8 @@
 // A channel's states are dealt to LG lanes, SP to each, in registers: lane = part * (64 / LG) + channel, so that neighbours read
 // neighbouring channels.  Tokens go TB at a time: their B and C through LDS (every channel reads the same ones), a lane's own dt, u and z
 // into registers ahead of their use.
-//   one pass    decode and short portions: the tokens one after the other
+//   step        one token per row (decode): from the shares of the product that gives dt, B and C to the result in one launch
+//   one pass    short portions: the tokens one after the other
 //   chunked     long portions: every chunk's own sums from a zero state side by side, a scan over the chunks
 //               S <- exp(A sum dt) S + own sums, then every chunk again from its true start, with outputs
 // A is kept times log2(e), so that a decay is one exp2.
@@ -18,27 +19,154 @@ namespace {
 constexpr int TB = 8;
 enum { SCAN_WHOLE = 0, SCAN_SUMS = 1, SCAN_OUT = 2 };
 
+// Four channels and CONV_TOKENS tokens per thread, the inputs sliding through registers (up to MAX_TAPS of them; more are read again).
+constexpr int CONV_TOKENS = 8, MAX_TAPS = 4;
 template <typename T>
 __global__ __launch_bounds__(256) void scan_conv_kernel(NcScanGeom g, const T* __restrict__ x, int ldx, const float* __restrict__ w, const float* __restrict__ bias,
                                                         const int32_t* __restrict__ seqlens, const float* __restrict__ state_in, float* __restrict__ state_out,
                                                         T* __restrict__ u) {
-    const int c = 4 * ((int)blockIdx.x * 256 + (int)threadIdx.x), t = blockIdx.y, b = blockIdx.z;
+    const int c = 4 * ((int)blockIdx.x * 256 + (int)threadIdx.x), t0 = (int)blockIdx.y * CONV_TOKENS, b = blockIdx.z;
     if (c >= g.inner_p) return;
     const int old = g.taps - 1;
     const bool fresh = seqlens[b] == 0;
     const int64_t so = ((int64_t)b * (g.state_p + old) + g.state_p) * g.inner_p + c;
     // input of token tt of this portion; earlier ones come out of the state, oldest first
     auto input = [&](int tt) -> v4f {
-        if (tt >= 0) return ld4_f32(x + ((int64_t)b * g.T + tt) * ldx + c);
+        if (tt >= 0) return ld4_f32(x + ((int64_t)b * g.T + min(tt, g.T - 1)) * ldx + c);
         if (fresh) return v4f{0.f, 0.f, 0.f, 0.f};
         return *(const v4f*)(state_in + so + (int64_t)(old + tt) * g.inner_p);
     };
-    v4f y = v4f{0.f, 0.f, 0.f, 0.f};
-    for (int i = 0; i < g.taps; i++) y += *(const v4f*)(w + (int64_t)i * g.inner_p + c) * input(t - old + i);
-    y += *(const v4f*)(bias + c);
-    st4_f32(u + ((int64_t)b * g.T + t) * g.inner_p + c, v4f{silu_f32(y[0]), silu_f32(y[1]), silu_f32(y[2]), silu_f32(y[3])});
-    if (t == g.T - 1)
+    const v4f bv = *(const v4f*)(bias + c);
+    auto store = [&](int t, v4f y) {
+        st4_f32(u + ((int64_t)b * g.T + t) * g.inner_p + c, v4f{silu_f32(y[0]), silu_f32(y[1]), silu_f32(y[2]), silu_f32(y[3])});
+    };
+    if (g.taps == MAX_TAPS) {                               // (uniform)
+        v4f wv[MAX_TAPS], in[CONV_TOKENS + MAX_TAPS - 1];
+#pragma unroll
+        for (int i = 0; i < MAX_TAPS; i++) wv[i] = *(const v4f*)(w + (int64_t)i * g.inner_p + c);
+#pragma unroll
+        for (int i = 0; i < CONV_TOKENS + MAX_TAPS - 1; i++)
+            if (i < MAX_TAPS || t0 + i - old < g.T) in[i] = input(t0 + i - old);
+            else in[i] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < CONV_TOKENS; j++) {
+            if (t0 + j >= g.T) break;
+            v4f y = bv;
+#pragma unroll
+            for (int i = 0; i < MAX_TAPS; i++) y += wv[i] * in[j + i];
+            store(t0 + j, y);
+        }
+    } else {
+        for (int t = t0; t < min(t0 + CONV_TOKENS, g.T); t++) {
+            v4f y = bv;
+            for (int i = 0; i < g.taps; i++) y += *(const v4f*)(w + (int64_t)i * g.inner_p + c) * input(t - old + i);
+            store(t, y);
+        }
+    }
+    if (t0 + CONV_TOKENS >= g.T)
         for (int j = 0; j < old; j++) *(v4f*)(state_out + so + (int64_t)j * g.inner_p) = input(g.T - old + j);
+}
+
+// One thread per four columns of one row.
+template <typename T>
+__global__ __launch_bounds__(256) void scan_join_kernel(const float* __restrict__ parts, int splits, int64_t M, int rank_p, int bc_cols, T* __restrict__ dtr,
+                                                        float* __restrict__ bc) {
+    const int N = rank_p + 2 * bc_cols;
+    const int64_t e = 4 * ((int64_t)blockIdx.x * 256 + threadIdx.x);
+    if (e >= M * N) return;
+    v4f p[8], sum = v4f{0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < splits; s0 += 8) {
+#pragma unroll
+        for (int s = 0; s < 8; s++) p[s] = *(const v4f*)(parts + min(s0 + s, splits - 1) * M * N + e);
+#pragma unroll
+        for (int s = 0; s < 8; s++)
+            if (s0 + s < splits) sum += p[s];
+    }
+    const int64_t m = e / N;
+    const int n = (int)(e % N);
+    if (n < rank_p) st4_f32(dtr + m * rank_p + n, sum);
+    else *(v4f*)(bc + m * 2 * bc_cols + n - rank_p) = sum;
+}
+
+// One token per row.  A workgroup of four waves takes 64 channels (one per lane) and RB rows: the waves share the sum over the step's rank,
+// then the states (SPW at most each); partial sums meet in LDS.
+template <typename T, int RB, int SPW>
+__global__ __launch_bounds__(256) void scan_step_kernel(NcScanGeom g, NcScanStep p) {
+    extern __shared__ __align__(16) float lds[];             // the rows' [step before W_dt | B | C]
+    __shared__ float red[4][RB][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = (int)blockIdx.x * 64 + lane, b0 = (int)blockIdx.y * RB, rows = min(RB, g.B - b0);
+    const int bc_cols = nc_scan_bc_cols(g.state_p), N = g.dt_rank_p + 2 * bc_cols, per = g.state_p / 4, n0 = wave * per;
+    const int64_t plane = (int64_t)(g.state_p + g.taps - 1) * g.inner_p;
+    float S[RB][SPW], a[SPW], uv[RB], zv[RB];
+#pragma unroll
+    for (int r = 0; r < RB; r++) {
+        const int b = b0 + min(r, rows - 1);
+        const bool fresh = p.seqlens[b] == 0;
+        uv[r] = ld_f32((const T*)p.u + (int64_t)b * g.inner_p + c);
+        zv[r] = ld_f32((const T*)p.z + (int64_t)b * p.ldz + c);
+#pragma unroll
+        for (int i = 0; i < SPW; i++) S[r][i] = fresh || i >= per ? 0.f : p.state_in[b * plane + (int64_t)(n0 + i) * g.inner_p + c];
+    }
+#pragma unroll
+    for (int i = 0; i < SPW; i++) a[i] = i < per ? p.a_log2[(int64_t)(n0 + i) * g.inner_p + c] : 0.f;
+    const float bias = p.dt_b[c], d = p.skip[c];
+    for (int i = 4 * tid; i < rows * N; i += 1024) {
+        v4f sum = v4f{0.f, 0.f, 0.f, 0.f};
+        const float* src = p.parts + (int64_t)b0 * N + i;
+#pragma unroll 8
+        for (int s = 0; s < p.splits; s++) sum += *(const v4f*)(src + (int64_t)s * g.B * N);
+        *(v4f*)(lds + i) = sum;
+    }
+    __syncthreads();
+    float dt[RB];
+#pragma unroll
+    for (int r = 0; r < RB; r++) dt[r] = 0.f;
+    const int share = g.dt_rank_p / 4, k0 = wave * share;    // a multiple of 16
+    const T* wp = (const T*)p.w_dt_t + (int64_t)k0 * g.inner_p + c;
+#pragma unroll 1
+    for (int k = 0; k < share; k += 16) {
+        float wv[16];
+#pragma unroll
+        for (int j = 0; j < 16; j++) wv[j] = ld_f32(wp + (int64_t)(k + j) * g.inner_p);
+#pragma unroll
+        for (int j = 0; j < 16; j++)
+#pragma unroll
+            for (int r = 0; r < RB; r++) dt[r] = fmaf(wv[j], lds[min(r, rows - 1) * N + k0 + k + j], dt[r]);
+    }
+#pragma unroll
+    for (int r = 0; r < RB; r++) red[wave][r][lane] = dt[r];
+    __syncthreads();
+    float y[RB];
+#pragma unroll
+    for (int r = 0; r < RB; r++) {
+        dt[r] = softplus_f32((red[0][r][lane] + red[1][r][lane]) + (red[2][r][lane] + red[3][r][lane]) + bias);
+        const float* bj = lds + min(r, rows - 1) * N + g.dt_rank_p + n0;
+        const float du = dt[r] * uv[r];
+        y[r] = 0.f;
+#pragma unroll
+        for (int i = 0; i < SPW; i++)
+            if (i < per) {                                   // uniform
+                S[r][i] = fmaf(__builtin_amdgcn_exp2f(dt[r] * a[i]), S[r][i], du * bj[i]);
+                y[r] = fmaf(S[r][i], bj[bc_cols + i], y[r]);
+            }
+    }
+    __syncthreads();                                         // everyone has read the sums of dt
+#pragma unroll
+    for (int r = 0; r < RB; r++) red[wave][r][lane] = y[r];
+#pragma unroll
+    for (int r = 0; r < RB; r++)
+        if (r < rows)
+#pragma unroll
+            for (int i = 0; i < SPW; i++)
+                if (i < per) p.state_out[(b0 + r) * plane + (int64_t)(n0 + i) * g.inner_p + c] = S[r][i];
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < RB; r++)
+        if (r < rows && wave == (r & 3)) {
+            const float t = (red[0][r][lane] + red[1][r][lane]) + (red[2][r][lane] + red[3][r][lane]);
+            st_f32((T*)p.out + (int64_t)(b0 + r) * p.ldo + c, fmaf(d, uv[r], t) * silu_f32(zv[r]) * g.out_scale);
+        }
 }
 
 // MODE WHOLE: all tokens from the stored state, outputs, state out.  SUMS: one chunk from zero, its end and its sum of dt into `ends` /
@@ -189,14 +317,58 @@ int launch_scan(const NcScanGeom& g, int lg, const T* u, const float* dt, const 
 int nc_launch_scan_conv(int dtype, const NcScanGeom& g, const void* x, int ldx, const float* w, const float* b, const int32_t* seqlens, const float* state_in,
                         float* state_out, void* u, hipStream_t s) {
     NC_CHECK_ARG(x && w && b && u && state_in != state_out && g.taps >= 1 && g.inner_p % 4 == 0 && ldx % 4 == 0, "scan_conv: %d taps, %d channels", g.taps, g.inner_p);
-    NC_CHECK_ARG(g.T <= 65535 && g.B <= 65535, "scan_conv: %d tokens in one portion", g.T);
+    NC_CHECK_ARG(g.T <= 65535 * CONV_TOKENS && g.B <= 65535, "scan_conv: %d tokens in one portion", g.T);
     NcProfScope prof(NC_CLS_ROWS, (double)g.B * g.T * g.inner_p * (dtype ? 8 : 4), s);
-    const dim3 grid((g.inner_p + 1023) / 1024, g.T, g.B);
+    const dim3 grid((g.inner_p + 1023) / 1024, (g.T + CONV_TOKENS - 1) / CONV_TOKENS, g.B);
     if (dtype)
         hipLaunchKernelGGL((scan_conv_kernel<float>), grid, dim3(256), 0, s, g, (const float*)x, ldx, w, b, seqlens, state_in, state_out, (float*)u);
     else
         hipLaunchKernelGGL((scan_conv_kernel<bf16_t>), grid, dim3(256), 0, s, g, (const bf16_t*)x, ldx, w, b, seqlens, state_in, state_out, (bf16_t*)u);
     NC_CHECK_LAUNCH("scan_conv");
+    return 0;
+}
+
+int nc_launch_scan_join(int dtype, const NcScanGeom& g, const float* parts, int splits, void* dtr, float* bc, hipStream_t s) {
+    const int bc_cols = nc_scan_bc_cols(g.state_p);
+    const int64_t M = (int64_t)g.B * g.T, work = M * (g.dt_rank_p + 2 * bc_cols) / 4;
+    NC_CHECK_ARG(parts && dtr && bc && splits >= 1 && g.dt_rank_p % 4 == 0, "scan_join: null operand");
+    NcProfScope prof(NC_CLS_ROWS, (double)work * 16 * (splits + 1), s);
+    if (dtype)
+        hipLaunchKernelGGL((scan_join_kernel<float>), dim3((unsigned)((work + 255) / 256)), dim3(256), 0, s, parts, splits, M, g.dt_rank_p, bc_cols, (float*)dtr, bc);
+    else
+        hipLaunchKernelGGL((scan_join_kernel<bf16_t>), dim3((unsigned)((work + 255) / 256)), dim3(256), 0, s, parts, splits, M, g.dt_rank_p, bc_cols, (bf16_t*)dtr, bc);
+    NC_CHECK_LAUNCH("scan_join");
+    return 0;
+}
+
+int nc_launch_scan_step(int dtype, const NcScanGeom& g, const NcScanStep& p, hipStream_t s) {
+    NC_CHECK_ARG(g.T == 1 && g.state_p % 4 == 0 && g.state_p <= 256 && g.inner_p % 64 == 0 && g.dt_rank_p % 64 == 0, "scan_step: %d tokens, %d states", g.T, g.state_p);
+    NC_CHECK_ARG(p.parts && p.splits >= 1 && p.w_dt_t && p.dt_b && p.a_log2 && p.skip && p.u && p.z && p.out && p.state_in != p.state_out, "scan_step: null operand");
+    const int N = g.dt_rank_p + 2 * nc_scan_bc_cols(g.state_p), per = g.state_p / 4;
+    // state in and out, the step's weight once, the rows in and out (bytes)
+    const double es = dtype ? 4 : 2;
+    NcProfScope prof(NC_CLS_SCAN, (double)g.B * (8.0 * g.state * g.inner + g.inner * 3 * es) + (double)g.dt_rank_p * g.inner * es, s, g.T);
+    // (few rows: one each, so that the launch covers the chip)
+    const int rb = per <= 16 && (int64_t)g.B * (g.inner_p / 64) >= 4 * nc_cu_count() ? 4 : 1;
+    const int bytes = rb * N * 4;
+    NC_CHECK_ARG(bytes <= 56 * 1024 && (g.B + rb - 1) / rb <= 65535, "scan_step: a step of rank %d", g.dt_rank_p);
+    const dim3 grid(g.inner_p / 64, (g.B + rb - 1) / rb);
+#define GO(RB, SPW)                                                                                          \
+    do {                                                                                                     \
+        if (dtype) hipLaunchKernelGGL((scan_step_kernel<float, RB, SPW>), grid, dim3(256), bytes, s, g, p);  \
+        else hipLaunchKernelGGL((scan_step_kernel<bf16_t, RB, SPW>), grid, dim3(256), bytes, s, g, p);       \
+    } while (0)
+    if (rb == 4) {
+        if (per <= 4) GO(4, 4);
+        else if (per <= 8) GO(4, 8);
+        else GO(4, 16);
+    } else {
+        if (per <= 4) GO(1, 4);
+        else if (per <= 16) GO(1, 16);
+        else GO(1, 64);
+    }
+#undef GO
+    NC_CHECK_LAUNCH("scan_step");
     return 0;
 }
 

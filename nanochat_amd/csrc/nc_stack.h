@@ -63,7 +63,8 @@ struct NcSeg {
 struct NcLinear {
     const void* a;
     int64_t lda;
-    const void* w;         // [N, K], rows of K elements
+    const void* w;         // [N, K], rows ldw elements apart
+    int64_t ldw;
     int M, N, K;
     int nseg;
     NcSeg seg[4];
@@ -82,7 +83,7 @@ struct NcLinear {
 };
 inline NcLinear nc_linear(const void* a, int64_t lda, const void* w, int M, int N, int K) {
     NcLinear l{};
-    l.a = a, l.lda = lda, l.w = w, l.M = M, l.N = N, l.K = K, l.batch = 1, l.a_div = 1, l.splits = 1;
+    l.a = a, l.lda = lda, l.w = w, l.ldw = K, l.M = M, l.N = N, l.K = K, l.batch = 1, l.a_div = 1, l.splits = 1;
     return l;
 }
 inline void nc_linear_seg(NcLinear& l, int end, int kind, void* out, int ld, float p0 = 0.f, float p1 = 0.f, const float* bias = nullptr) {
@@ -202,8 +203,26 @@ __host__ __device__ inline int nc_scan_bc_cols(int state_p) { return (state_p + 
 // u = silu(causal convolution of x); the convolution's part of the state moves on
 int nc_launch_scan_conv(int dtype, const NcScanGeom& g, const void* x, int ldx, const float* w, const float* b, const int32_t* seqlens, const float* state_in,
                         float* state_out, void* u, hipStream_t s);
-// the recurrence and what follows it: out = (sum_n S C + skip u) * silu(z) * scale.  dt fp32 [M][inner_p], bc fp32
-// [M][2 * nc_scan_bc_cols]
+// The product that gives a token its step (before W_dt), B and C has few columns and a long sum: it is left in `splits` shares,
+// parts fp32 [splits][M][dt_rank_p + 2 * nc_scan_bc_cols].  nc_launch_scan_join adds them up into dtr T [M][dt_rank_p] and bc fp32
+// [M][2 * nc_scan_bc_cols].
+int nc_launch_scan_join(int dtype, const NcScanGeom& g, const float* parts, int splits, void* dtr, float* bc, hipStream_t s);
+// One token per row (T = 1): everything from those shares on in one launch.
+struct NcScanStep {
+    const float* parts;
+    int splits;
+    const void* w_dt_t;            // T [dt_rank_p][inner_p]
+    const float *dt_b, *a_log2, *skip;
+    const void *u, *z;
+    int ldz;
+    const int32_t* seqlens;
+    const float* state_in;
+    float* state_out;
+    void* out;
+    int ldo;
+};
+int nc_launch_scan_step(int dtype, const NcScanGeom& g, const NcScanStep& p, hipStream_t s);
+// the recurrence and what follows it: out = (sum_n S C + skip u) * silu(z) * scale.  dt fp32 [M][inner_p], bc as above
 size_t nc_scan_workspace_bytes(const NcScanGeom& g);
 int nc_launch_scan(int dtype, const NcScanGeom& g, const void* u, const float* dt, const float* bc, const float* a_log2, const float* skip,
                    const void* z, int ldz, const int32_t* seqlens, const float* state_in, float* state_out, void* out, int ldo, void* workspace,

@@ -35,7 +35,7 @@ struct Carver {
 };
 
 struct Workspace {
-    float *x, *x0, *router, *parts, *raw, *bc, *dt;
+    float *x, *x0, *router, *parts, *raw, *bc, *dt, *x_parts;
     void *h, *proj, *cat, *h_last, *q_lat, *o_lat, *kv, *att_parts, *ret, *act, *e_out, *u, *dtr;
     float* slot_w;
     int32_t *chosen, *slot_of, *perm, *tiles, *n_tiles;
@@ -50,6 +50,15 @@ NcRetentionGeom retention_geom(const nc_stack_mixer& l, int B, int T, float* raw
 }
 NcWindowGeom window_geom(const nc_stack_mixer& l, int B, int T, int Tmax, int pos_max) {
     return NcWindowGeom{l.heads, l.kv_heads, l.dim, l.dim_p, l.vdim_p, l.rot_dims, l.window, l.keep_first, l.score_scale, l.out_scale, B, T, Tmax, pos_max};
+}
+// shares of the sum over channels that the few columns of w_x are cut into, to fill the chip
+int scan_x_cols(const nc_stack_mixer& l) { return l.dt_rank_p + 2 * nc_scan_bc_cols(l.state_p); }
+int scan_x_splits(const nc_stack_mixer& l, int M) {
+    if (M <= NC_FEW_ROWS) return nc_linear_few_splits(M, scan_x_cols(l), l.inner_p);
+    const int64_t tiles = (int64_t)((M + 63) / 64) * ((scan_x_cols(l) + 127) / 128);
+    int splits = 1;
+    while (splits < 16 && tiles * splits < 512 && l.inner_p % (2 * splits * NC_STACK_PAD) == 0 && l.inner_p / (2 * splits) >= 256) splits *= 2;
+    return splits;
 }
 NcScanGeom scan_geom(const nc_stack_mixer& l, int B, int T) {
     return NcScanGeom{l.inner, l.inner_p, l.state, l.state_p, l.taps, l.dt_rank_p, l.out_scale, B, T};
@@ -73,7 +82,7 @@ size_t max_of(size_t a, size_t b) { return a > b ? a : b; }
 Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_keys, void* base) {
     const size_t M = (size_t)B * T, Wp = m->width_p, es = m->dtype ? 4 : 2;
     size_t proj = 0, router = 0, parts = 0, qlat = 0, olat = 0, kv = 0, att = 0, ret = 0, act = 0, eout = 0, pairs = 0, tiles = 0, raw = 0, bc = 0, dt = 0, u = 0,
-           dtr = 0;
+           dtr = 0, x_parts = 0;
     bool again = false;
     for (int i = 0; i < m->n_runs; i++) again |= m->runs[i].add_embedding != 0;
     for (int i = 0; i < m->n_layers; i++) {
@@ -109,7 +118,10 @@ Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_key
                     break;
                 default:
                     ret = max_of(ret, nc_scan_workspace_bytes(scan_geom(x, B, T)));
-                    u = max_of(u, M * x.inner_p * es), dt = max_of(dt, M * x.inner_p * 4);
+                    u = max_of(u, M * x.inner_p * es);
+                    x_parts = max_of(x_parts, (size_t)scan_x_splits(x, (int)M) * M * scan_x_cols(x) * 4);
+                    if (T == 1) break;
+                    dt = max_of(dt, M * x.inner_p * 4);
                     dtr = max_of(dtr, M * x.dt_rank_p * es), bc = max_of(bc, M * 2 * nc_scan_bc_cols(x.state_p) * 4);
             }
         }
@@ -151,6 +163,7 @@ Workspace carve(const nc_stack_model* m, int B, int T, int n_logits, int max_key
     w.dtr = c.take(dtr);
     w.bc = (float*)c.take(bc);
     w.dt = (float*)c.take(dt);
+    w.x_parts = (float*)c.take(x_parts);
     w.total = (c.off + 255) & ~(size_t)255;
     return w;
 }
@@ -206,16 +219,27 @@ int run_retention(int dt, const nc_stack_mixer& l, const NcRetentionGeom& g, con
 
 int run_selective_scan(int dt, const nc_stack_mixer& l, const NcScanGeom& g, const Workspace& w, const void* proj, int ldp, const int32_t* seqlens,
                        const float* state_in, float* state_out, void* cat, int ld_cat, hipStream_t s) {
-    const int M = g.B * g.T, bc = nc_scan_bc_cols(l.state_p);
+    const int M = g.B * g.T, N = scan_x_cols(l), splits = scan_x_splits(l, M);
     TRY(nc_launch_scan_conv(dt, g, proj, ldp, l.conv_w, l.conv_b, seqlens, state_in, state_out, w.u, s));
-    NcLinear x = nc_linear(w.u, l.inner_p, l.w_x, M, l.dt_rank_p + 2 * bc, l.inner_p);
-    nc_linear_seg(x, l.dt_rank_p, NC_SEG_PLAIN, w.dtr, l.dt_rank_p);
-    nc_linear_seg(x, x.N, NC_SEG_F32, w.bc, 2 * bc);
+    NcLinear x = nc_linear(w.u, l.inner_p, l.w_x, M, N, l.inner_p);
+    if (M <= NC_FEW_ROWS) {
+        if (splits > 1) x.partials = w.x_parts, x.splits = splits;
+        else nc_linear_seg(x, N, NC_SEG_F32, w.x_parts, N);
+    } else {                                       // every share is a product of its own
+        x.K = l.inner_p / splits, x.batch = splits, x.a_stride = x.w_stride = x.K, x.out_stride = (int64_t)M * N;
+        nc_linear_seg(x, N, NC_SEG_F32, w.x_parts, N);
+    }
     TRY(run_linear(dt, x, s));
+    const void* z = at(proj, l.inner_p, dt);
+    if (g.T == 1) {
+        const NcScanStep p{w.x_parts, splits, l.w_dt_t, l.dt_b, l.a_log2, l.skip, w.u, z, ldp, seqlens, state_in, state_out, cat, ld_cat};
+        return nc_launch_scan_step(dt, g, p, s);
+    }
+    TRY(nc_launch_scan_join(dt, g, w.x_parts, splits, w.dtr, w.bc, s));
     NcLinear d = nc_linear(w.dtr, l.dt_rank_p, l.w_dt, M, l.inner_p, l.dt_rank_p);
     nc_linear_seg(d, d.N, NC_SEG_SOFTPLUS, w.dt, l.inner_p, 0.f, 0.f, l.dt_b);
     TRY(run_linear(dt, d, s));
-    return nc_launch_scan(dt, g, w.u, w.dt, w.bc, l.a_log2, l.skip, at(proj, l.inner_p, dt), ldp, seqlens, state_in, state_out, cat, ld_cat, w.ret, s);
+    return nc_launch_scan(dt, g, w.u, w.dt, w.bc, l.a_log2, l.skip, z, ldp, seqlens, state_in, state_out, cat, ld_cat, w.ret, s);
 }
 
 // The mixers of one layer run, on the projected rows w.proj, into w.cat.

@@ -128,7 +128,7 @@ __global__ __launch_bounds__(256) void linear_few_kernel(NcLinear g) {
 #pragma unroll
     for (int j = 0; j < NB; j++) {
         const int n = min(n0 + 16 * j + frow, g.N - 1);
-        wp[j] = (const uint8_t*)((const T*)g.w + sp.w_off + (int64_t)n * g.K) + piece * 16;
+        wp[j] = (const uint8_t*)((const T*)g.w + sp.w_off + (int64_t)n * g.ldw) + piece * 16;
     }
 #pragma unroll
     for (int i = 0; i < MT; i++) {
@@ -244,7 +244,7 @@ __global__ __launch_bounds__(64 * WM * WN) void linear_tiled_kernel(NcLinear g, 
     // block, and the global chunk that belongs in its LDS slot
     const int sub = lane >> 3, gch = (lane & 7) ^ sub ^ (wave & 1);
     const int rd_lo = frow * 128 + (((2 * piece) ^ TILE_SWZ(frow)) << 4), rd_hi = frow * 128 + (((2 * piece + 1) ^ TILE_SWZ(frow)) << 4);
-    const uint32_t row_a = (uint32_t)(g.lda * sizeof(T)), row_w = (uint32_t)(g.K * sizeof(T));
+    const uint32_t row_a = (uint32_t)(g.lda * sizeof(T)), row_w = (uint32_t)(g.ldw * sizeof(T)), k_bytes = (uint32_t)(g.K * sizeof(T));
     const T* const A = (const T*)g.a + sp.a_off;
     const T* const W = (const T*)g.w + sp.w_off;
     uint32_t vo_a[A_P], vo_w[W_P];
@@ -258,14 +258,14 @@ __global__ __launch_bounds__(64 * WM * WN) void linear_tiled_kernel(NcLinear g, 
         const int r = n0 + 8 * (wave + NW * i) + sub;
         vo_w[i] = r < g.N ? (uint32_t)r * row_w + gch * 16 : TILE_OOB;
     }
-    const int ksteps = row_w / 128;
+    const int ksteps = k_bytes / 128;
     v4f acc[WTM][WTN];
 #pragma unroll
     for (int i = 0; i < WTM; i++)
 #pragma unroll
         for (int j = 0; j < WTN; j++) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
     auto fetch = [&](int t, int stage) {
-        tile_fetch<A_P, W_P, NW * 1024>(A, a_bytes, W, (uint32_t)g.N * row_w, lds + stage * STAGE + wave * 1024, BM * 128, vo_a, vo_w,
+        tile_fetch<A_P, W_P, NW * 1024>(A, a_bytes, W, (uint32_t)(g.N - 1) * row_w + k_bytes, lds + stage * STAGE + wave * 1024, BM * 128, vo_a, vo_w,
                                         t < ksteps ? t * 128 : 0);
     };
     auto meet = [&]() {
@@ -343,7 +343,7 @@ int check_linear(const NcLinear& l, int dtype) {
     NC_CHECK_ARG(l.a && l.w && l.nseg <= 4, "linear: null operand");
     NC_CHECK_ARG(l.M > 0 && l.N > 0 && l.K > 0 && l.K % 32 == 0 && l.batch >= 1, "linear: bad shape M=%d N=%d K=%d batch=%d", l.M, l.N, l.K, l.batch);
     NC_CHECK_ARG(dtype == 0 || dtype == 1, "linear: dtype must be 0 (bfloat16) or 1 (float)");
-    NC_CHECK_ARG(l.lda % (dtype ? 4 : 8) == 0 && ((uintptr_t)l.a & 15) == 0 && ((uintptr_t)l.w & 15) == 0, "linear: operands must be 16-byte aligned");
+    NC_CHECK_ARG(l.lda % (dtype ? 4 : 8) == 0 && l.ldw % (dtype ? 4 : 8) == 0 && l.ldw >= l.K && ((uintptr_t)l.a & 15) == 0 && ((uintptr_t)l.w & 15) == 0, "linear: operands must be 16-byte aligned");
     for (int i = 0; i < l.nseg; i++)
         NC_CHECK_ARG(l.seg[i].kind == NC_SEG_LOGITS || (l.seg[i].end % 16 == 0 && l.seg[i].ld % 4 == 0), "linear: segments must end at multiples of 16 columns");
     return 0;
@@ -373,7 +373,7 @@ int launch_tiled(const NcLinear& l, hipStream_t s) {
     // rows of A this launch may reach: all of them (a gathered row index is below M / a_div)
     const int64_t a_rows = l.a_rows ? (l.M + l.a_div - 1) / l.a_div : l.M;
     const int64_t a_bytes = ((a_rows - 1) * l.lda + l.K) * (int64_t)sizeof(T);
-    NC_CHECK_ARG(a_bytes < (1ll << 31) && (int64_t)l.N * l.K * (int64_t)sizeof(T) < (1ll << 31), "linear: operand past 2 GiB");
+    NC_CHECK_ARG(a_bytes < (1ll << 31) && (int64_t)l.N * l.ldw * (int64_t)sizeof(T) < (1ll << 31), "linear: operand past 2 GiB");
     hipLaunchKernelGGL((linear_tiled_kernel<T, BM, BN, WM, WN, STAGES>), dim3(tm * tn, l.batch), dim3(64 * WM * WN), LDS, s, l, tm, tn, (uint32_t)a_bytes);
     NC_CHECK_LAUNCH("linear_tiled");
     return 0;
@@ -416,7 +416,9 @@ int nc_launch_linear_tiled(int dtype, const NcLinear& l, hipStream_t s, int cls,
         // the widest tile unless it leaves compute units without one (measured at 1792 rows: 858 against 679 TFLOP/s at N = 12352, 551
         // against 717 at N = 2048, where the launch has 112 or 448 tiles)
         const int64_t wide = (int64_t)((l.M + 127) / 128) * ((l.N + 255) / 256) * l.batch;
-        shape = l.tiles ? (l.tile_rows == 64 ? 1 : 2) : wide < 200 ? 1 : 2;
+        // (a sum of a few K-steps is mostly its epilogue: two workgroups per compute unit, one of which works while the other stores)
+        const bool brief = l.K * (dtype ? 4 : 2) <= 512;
+        shape = l.tiles ? (l.tile_rows == 64 ? 1 : 2) : wide < 200 || brief ? 1 : 2;
     }
     if (l.tiles) NC_CHECK_ARG(l.tile_rows == (shape == 1 ? 64 : 128), "linear: group tiles of %d rows", l.tile_rows);
     return dtype ? launch_tiled_shape<float>(l, shape, s) : launch_tiled_shape<bf16_t>(l, shape, s);

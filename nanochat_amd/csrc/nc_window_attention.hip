@@ -12,7 +12,7 @@
 // Scores, softmax and sums are fp32; where the weights meet bf16 values on the matrix cores they go in as two bf16 terms.
 //
 //   window_few_kernel      decode and short portions: 16 query rows of one kv head, keys dealt to waves and workgroups
-//   window_prefill_kernel  long portions: waves of 32 queries of one head, keys through LDS
+//   window_prefill_kernel  long portions: waves of 32 queries of one head, keys through LDS; two waves may share the keys of their queries
 //   window_simple_kernel   any sizes, either storage type
 #include "nc_stack.h"
 
@@ -333,14 +333,17 @@ __global__ __launch_bounds__(64) void window_combine_kernel(const float* __restr
 
 // ------------------------------------------------------------------------------------------------ many query rows
 // Flash attention written transposed (S^T = K Q^T, O^T = V^T P^T with v_mfma_f32_32x32x16_bf16; a lane owns one query's column of both):
-// NW waves of 32 queries, one head per workgroup, 16 NW entries of the workgroup's key list at a time through LDS.
-template <int DQ, int DV, int NW>
-__global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(2, 2))) void window_prefill_kernel(
+// NQ groups of 32 queries, one head per workgroup, KB entries of the workgroup's key list at a time through LDS; the blocks of 32 keys are
+// dealt to KS waves per group, whose sums meet in LDS at the end.
+template <int DQ, int DV, int NQ, int KS>
+__global__ __launch_bounds__(64 * NQ * KS) __attribute__((amdgpu_waves_per_eu(2, 2))) void window_prefill_kernel(
     NcWindowGeom g, const bf16_t* __restrict__ q, int ldq, const bf16_t* __restrict__ cache, const float* __restrict__ sink,
     const int32_t* __restrict__ seqlens, bf16_t* __restrict__ out, int ldo) {
-    constexpr int KPITCH = DQ * 2 + 16, VPITCH = DV * 2 + 64, NTHR = 64 * NW, KB = 16 * NW, QT = 32 * NW;
+    constexpr int KPITCH = DQ * 2 + 16, VPITCH = DV * 2 + 64, NW = NQ * KS, NTHR = 64 * NW, KB = 16 * NW, QT = 32 * NQ;
     constexpr int KCH = DQ / 8, VCH = DV / 8, KL = KB * KCH / NTHR, VL = KB * VCH / NTHR;
-    __shared__ __align__(16) uint8_t lds[KB * KPITCH + KB * VPITCH];
+    constexpr int STAGE = KB * KPITCH + KB * VPITCH, O_PITCH = DV + 4, SUM = KS > 1 ? NQ * 32 * (O_PITCH + 2) * 4 : 0;
+    static_assert(KS == 1 || (KS == 2 && KB >= 64), "every wave has a block of a stage");
+    __shared__ __align__(16) uint8_t lds[STAGE > SUM ? STAGE : SUM];
     uint8_t* const lds_v = lds + KB * KPITCH;
     const lds_u8_t lds_v3 = (lds_u8_t)lds + KB * KPITCH;
     const int b = blockIdx.z;
@@ -354,7 +357,7 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(2, 2)))
     const int kvh = h / (g.heads / g.kv_heads), head_w = g.dim_p + g.vdim_p, rw = g.kv_heads * head_w;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int col = lane & 31, hl = lane >> 5;
-    const int qw0 = qb0 + 32 * wave, t = qw0 + col;
+    const int qw = wave % NQ, ks = wave / NQ, qw0 = qb0 + 32 * qw, t = qw0 + col;
     const int pos0 = min(seqlens[b], g.Tmax - g.T);
     const int qpos = pos0 + min(t, g.T - 1);
     const int w_lo = pos0 + min(qw0, g.T - 1), w_hi = pos0 + min(qw0 + 31, g.T - 1);
@@ -375,7 +378,7 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(2, 2)))
     for (int dt = 0; dt < DV / 32; dt++)
 #pragma unroll
         for (int r = 0; r < 16; r++) o[dt][r] = 0.f;
-    float m_run = sink[h] * LOG2E, l_run = hl == 0 ? 1.f : 0.f;
+    float m_run = ks == 0 ? sink[h] * LOG2E : WA_M_FLOOR, l_run = ks == 0 && hl == 0 ? 1.f : 0.f;
     const float sc = g.scale * LOG2E;
 
     // staging: 16-byte piece idx = tid + NTHR i of the block's keys; past a head's own sizes zeros
@@ -462,7 +465,7 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(2, 2)))
         __syncthreads();
         if (vb + KB < list.count) fetch(vb + KB);
 #pragma unroll 1
-        for (int sb = 0; sb < KB / 32; sb++) {
+        for (int sb = ks; sb < KB / 32; sb += KS) {
             const int v0 = vb + 32 * sb;
             if (v0 >= list.count) break;
             // the smallest and largest key of these entries (the list rises), against the wave's queries
@@ -472,7 +475,27 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(2, 2)))
             sub_block(v0, sb, !all);
         }
     }
-    const float inv = g.out_scale / (l_run + __shfl_xor(l_run, 32));
+    l_run += __shfl_xor(l_run, 32);
+    if (KS == 2) {
+        float* const row = (float*)lds + (32 * qw + col) * (O_PITCH + 2);
+        __syncthreads();                       // the last stage has been read
+        if (ks == 1) {
+            if (hl == 0) row[O_PITCH] = m_run, row[O_PITCH + 1] = l_run;
+#pragma unroll
+            for (int dt = 0; dt < DV / 32; dt++)
+#pragma unroll
+                for (int r = 0; r < 16; r++) row[32 * dt + 8 * (r >> 2) + 4 * hl + (r & 3)] = o[dt][r];
+        }
+        __syncthreads();
+        if (ks == 1) return;
+        const float m2 = row[O_PITCH], mt = fmaxf(m_run, m2), f1 = __builtin_amdgcn_exp2f(m_run - mt), f2 = __builtin_amdgcn_exp2f(m2 - mt);
+        l_run = l_run * f1 + row[O_PITCH + 1] * f2;
+#pragma unroll
+        for (int dt = 0; dt < DV / 32; dt++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) o[dt][r] = o[dt][r] * f1 + row[32 * dt + 8 * (r >> 2) + 4 * hl + (r & 3)] * f2;
+    }
+    const float inv = g.out_scale / l_run;
     if (t >= g.T) return;
     bf16_t* orow = out + ((int64_t)b * g.T + t) * ldo + h * g.vdim_p;
 #pragma unroll
@@ -515,10 +538,10 @@ int launch_few(const NcWindowGeom& g, const bf16_t* q, int ldq, const bf16_t* ca
 template <int DQ, int DV>
 int launch_prefill(const NcWindowGeom& g, const bf16_t* q, int ldq, const bf16_t* cache, const float* sink, const int32_t* seqlens, bf16_t* out, int ldo,
                    hipStream_t s) {
-    if ((int64_t)((g.T + 127) / 128) * g.heads * g.B >= 200)
-        hipLaunchKernelGGL((window_prefill_kernel<DQ, DV, 4>), dim3((g.T + 127) / 128, g.heads, g.B), dim3(256), 0, s, g, q, ldq, cache, sink, seqlens, out, ldo);
+    if ((int64_t)((g.T + 127) / 128) * g.heads * g.B >= 2 * nc_cu_count())
+        hipLaunchKernelGGL((window_prefill_kernel<DQ, DV, 4, 1>), dim3((g.T + 127) / 128, g.heads, g.B), dim3(256), 0, s, g, q, ldq, cache, sink, seqlens, out, ldo);
     else
-        hipLaunchKernelGGL((window_prefill_kernel<DQ, DV, 2>), dim3((g.T + 63) / 64, g.heads, g.B), dim3(128), 0, s, g, q, ldq, cache, sink, seqlens, out, ldo);
+        hipLaunchKernelGGL((window_prefill_kernel<DQ, DV, 2, 2>), dim3((g.T + 63) / 64, g.heads, g.B), dim3(256), 0, s, g, q, ldq, cache, sink, seqlens, out, ldo);
     NC_CHECK_LAUNCH("window_prefill");
     return 0;
 }

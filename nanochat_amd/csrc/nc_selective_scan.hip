@@ -98,41 +98,64 @@ __global__ __launch_bounds__(256) void scan_step_kernel(NcScanGeom g, NcScanStep
     const int c = (int)blockIdx.x * 64 + lane, b0 = (int)blockIdx.y * RB, rows = min(RB, g.B - b0);
     const int bc_cols = nc_scan_bc_cols(g.state_p), N = g.dt_rank_p + 2 * bc_cols, per = g.state_p / 4, n0 = wave * per;
     const int64_t plane = (int64_t)(g.state_p + g.taps - 1) * g.inner_p;
+    // Loads come back in the order they are asked for: first what the first barrier waits for (the shares), then 16 weights of this wave's
+    // part of the sum over the step's rank, then the state, which nobody needs before the second barrier.
+    auto shares = [&](int i, int s0, v4f (&v)[8]) {
+        const float* src = p.parts + (int64_t)b0 * N + i;
+#pragma unroll
+        for (int s = 0; s < 8; s++) v[s] = *(const v4f*)(src + (int64_t)min(s0 + s, p.splits - 1) * g.B * N);
+    };
+    v4f first[8];
+    const int i0 = min(4 * tid, rows * N - 4);
+    shares(i0, 0, first);
+    const int share = g.dt_rank_p / 4, k0 = wave * share;    // a multiple of 16
+    const T* wp = (const T*)p.w_dt_t + (int64_t)k0 * g.inner_p + c;
+    T wv[16];
+#pragma unroll
+    for (int j = 0; j < 16; j++) wv[j] = wp[(int64_t)j * g.inner_p];
     float S[RB][SPW], a[SPW], uv[RB], zv[RB];
+    bool fresh[RB];
 #pragma unroll
     for (int r = 0; r < RB; r++) {
         const int b = b0 + min(r, rows - 1);
-        const bool fresh = p.seqlens[b] == 0;
+        fresh[r] = p.seqlens[b] == 0;
         uv[r] = ld_f32((const T*)p.u + (int64_t)b * g.inner_p + c);
         zv[r] = ld_f32((const T*)p.z + (int64_t)b * p.ldz + c);
 #pragma unroll
-        for (int i = 0; i < SPW; i++) S[r][i] = fresh || i >= per ? 0.f : p.state_in[b * plane + (int64_t)(n0 + i) * g.inner_p + c];
+        for (int i = 0; i < SPW; i++) S[r][i] = p.state_in[b * plane + (int64_t)(n0 + min(i, per - 1)) * g.inner_p + c];
     }
 #pragma unroll
-    for (int i = 0; i < SPW; i++) a[i] = i < per ? p.a_log2[(int64_t)(n0 + i) * g.inner_p + c] : 0.f;
+    for (int i = 0; i < SPW; i++) a[i] = p.a_log2[(int64_t)(n0 + min(i, per - 1)) * g.inner_p + c];
     const float bias = p.dt_b[c], d = p.skip[c];
     for (int i = 4 * tid; i < rows * N; i += 1024) {
         v4f sum = v4f{0.f, 0.f, 0.f, 0.f};
-        const float* src = p.parts + (int64_t)b0 * N + i;
-#pragma unroll 8
-        for (int s = 0; s < p.splits; s++) sum += *(const v4f*)(src + (int64_t)s * g.B * N);
+        for (int s0 = 0; s0 < p.splits; s0 += 8) {
+            if (s0 > 0 || i >= 1024) shares(i, s0, first);
+#pragma unroll
+            for (int s = 0; s < 8; s++)
+                if (s0 + s < p.splits) sum += first[s];
+        }
         *(v4f*)(lds + i) = sum;
     }
     __syncthreads();
     float dt[RB];
 #pragma unroll
     for (int r = 0; r < RB; r++) dt[r] = 0.f;
-    const int share = g.dt_rank_p / 4, k0 = wave * share;    // a multiple of 16
-    const T* wp = (const T*)p.w_dt_t + (int64_t)k0 * g.inner_p + c;
 #pragma unroll 1
     for (int k = 0; k < share; k += 16) {
-        float wv[16];
+        float w[16];
 #pragma unroll
-        for (int j = 0; j < 16; j++) wv[j] = ld_f32(wp + (int64_t)(k + j) * g.inner_p);
+        for (int j = 0; j < 16; j++) w[j] = ld_f32(&wv[j]);
+        if (k + 16 < share)
 #pragma unroll
-        for (int j = 0; j < 16; j++)
+            for (int j = 0; j < 16; j++) wv[j] = wp[(int64_t)(k + 16 + j) * g.inner_p];
 #pragma unroll
-            for (int r = 0; r < RB; r++) dt[r] = fmaf(wv[j], lds[min(r, rows - 1) * N + k0 + k + j], dt[r]);
+        for (int j = 0; j < 16; j += 4)
+#pragma unroll
+            for (int r = 0; r < RB; r++) {
+                const v4f x = *(const v4f*)(lds + min(r, rows - 1) * N + k0 + k + j);
+                dt[r] = fmaf(w[j + 3], x[3], fmaf(w[j + 2], x[2], fmaf(w[j + 1], x[1], fmaf(w[j], x[0], dt[r]))));
+            }
     }
 #pragma unroll
     for (int r = 0; r < RB; r++) red[wave][r][lane] = dt[r];
@@ -147,7 +170,7 @@ __global__ __launch_bounds__(256) void scan_step_kernel(NcScanGeom g, NcScanStep
 #pragma unroll
         for (int i = 0; i < SPW; i++)
             if (i < per) {                                   // uniform
-                S[r][i] = fmaf(__builtin_amdgcn_exp2f(dt[r] * a[i]), S[r][i], du * bj[i]);
+                S[r][i] = fmaf(__builtin_amdgcn_exp2f(dt[r] * a[i]), fresh[r] ? 0.f : S[r][i], du * bj[i]);
                 y[r] = fmaf(S[r][i], bj[bc_cols + i], y[r]);
             }
     }
@@ -249,37 +272,34 @@ __global__ __launch_bounds__(256) void scan_kernel(NcScanGeom g, int lg, const T
     }
 }
 
-// Every chunk's end from a zero state becomes the true start of the next chunk, in place.  One thread per four channels of one state.
+// Every chunk's end from a zero state becomes the true start of the next chunk, in place.  One thread per channel and state.
 __global__ __launch_bounds__(256) void scan_chunks_kernel(NcScanGeom g, const float* __restrict__ a_log2, const int32_t* __restrict__ seqlens,
                                                           const float* __restrict__ state_in, float* __restrict__ ends, const float* __restrict__ sum_dt, int chunks) {
-    const int c = 4 * ((int)blockIdx.x * 256 + (int)threadIdx.x), n = blockIdx.y, b = blockIdx.z;
+    const int c = (int)blockIdx.x * 256 + (int)threadIdx.x, n = blockIdx.y, b = blockIdx.z;
     if (c >= g.inner_p) return;
     const int64_t plane = (int64_t)g.state_p * g.inner_p;
-    const v4f a = *(const v4f*)(a_log2 + (int64_t)n * g.inner_p + c);
-    v4f S = v4f{0.f, 0.f, 0.f, 0.f};
-    if (seqlens[b] > 0) S = *(const v4f*)(state_in + ((int64_t)b * (g.state_p + g.taps - 1) + n) * g.inner_p + c);
+    const float a = a_log2[(int64_t)n * g.inner_p + c];
+    float S = seqlens[b] > 0 ? state_in[((int64_t)b * (g.state_p + g.taps - 1) + n) * g.inner_p + c] : 0.f;
     float* e = ends + (int64_t)b * (chunks - 1) * plane + (int64_t)n * g.inner_p + c;
     const float* sd = sum_dt + (int64_t)b * (chunks - 1) * g.inner_p + c;
-    constexpr int AHEAD = 8;
+    constexpr int AHEAD = 32;
     for (int k0 = 0; k0 < chunks - 1; k0 += AHEAD) {
-        v4f own[AHEAD], s[AHEAD];
+        float own[AHEAD], s[AHEAD];
 #pragma unroll
         for (int j = 0; j < AHEAD; j++) {
             const int k = min(k0 + j, chunks - 2);
-            own[j] = *(const v4f*)(e + k * plane), s[j] = *(const v4f*)(sd + (int64_t)k * g.inner_p);
+            own[j] = e[k * plane], s[j] = sd[(int64_t)k * g.inner_p];
         }
 #pragma unroll
         for (int j = 0; j < AHEAD; j++) {
             if (k0 + j >= chunks - 1) break;
-#pragma unroll
-            for (int r = 0; r < 4; r++) S[r] = fmaf(__builtin_amdgcn_exp2f(a[r] * s[j][r]), S[r], own[j][r]);
-            *(v4f*)(e + (k0 + j) * plane) = S;
+            S = fmaf(__builtin_amdgcn_exp2f(a * s[j]), S, own[j]);
+            e[(k0 + j) * plane] = S;
         }
     }
 }
 
 constexpr int CHUNK = 64, CHUNK_MIN_TOKENS = 96;
-int chunk_count(const NcScanGeom& g) { return g.T < CHUNK_MIN_TOKENS ? 1 : (g.T + CHUNK - 1) / CHUNK; }
 // states per lane and lanes per channel (0: not such a size)
 bool lanes_of(int state_p, int& sp, int& lg) {
     for (int s : {16, 12, 8, 4}) {
@@ -292,10 +312,26 @@ bool lanes_of(int state_p, int& sp, int& lg) {
     return false;
 }
 
+int channel_groups(const NcScanGeom& g, int lg) { return (g.inner_p + 4 * (64 / lg) - 1) / (4 * (64 / lg)); }
+// Tokens per chunk (0: one pass): at most CHUNK, and so few that the workgroups come out in whole rounds of compute units.
+int chunk_len(const NcScanGeom& g) {
+    int sp = 0, lg = 0;
+    if (g.T < CHUNK_MIN_TOKENS || !lanes_of(g.state_p, sp, lg)) return 0;
+    const int per_chunk = channel_groups(g, lg) * g.B, least = (g.T + CHUNK - 1) / CHUNK, cus = nc_cu_count();
+    const int64_t rounds = ((int64_t)per_chunk * least + cus - 1) / cus;
+    const int chunks = (int)(rounds * cus / per_chunk);
+    const int len = ((g.T + chunks - 1) / chunks + TB - 1) / TB * TB;
+    return len < 32 ? 32 : len;
+}
+int chunk_count(const NcScanGeom& g) {
+    const int len = chunk_len(g);
+    return len ? (g.T + len - 1) / len : 1;
+}
+
 template <typename T, int SP>
 int launch_scan(const NcScanGeom& g, int lg, const T* u, const float* dt, const float* bc, const float* a_log2, const float* skip, const T* z, int ldz,
                 const int32_t* seqlens, const float* state_in, float* state_out, T* out, int ldo, void* workspace, hipStream_t s) {
-    const int chunks = chunk_count(g), xs = (g.inner_p + 4 * (64 / lg) - 1) / (4 * (64 / lg)), bytes = TB * 2 * g.state_p * 4;
+    const int chunks = chunk_count(g), len = chunk_len(g), xs = channel_groups(g, lg), bytes = TB * 2 * g.state_p * 4;
     if (chunks == 1) {
         hipLaunchKernelGGL((scan_kernel<T, SP, SCAN_WHOLE>), dim3(xs, 1, g.B), dim3(256), bytes, s, g, lg, u, dt, bc, a_log2, skip, z, ldz, seqlens, state_in, state_out,
                            out, ldo, nullptr, nullptr, 1, 0);
@@ -305,10 +341,10 @@ int launch_scan(const NcScanGeom& g, int lg, const T* u, const float* dt, const 
     float* ends = (float*)workspace;
     float* sum_dt = ends + (int64_t)g.B * (chunks - 1) * g.state_p * g.inner_p;
     hipLaunchKernelGGL((scan_kernel<T, SP, SCAN_SUMS>), dim3(xs, chunks - 1, g.B), dim3(256), bytes, s, g, lg, u, dt, bc, a_log2, skip, z, ldz, seqlens, state_in,
-                       state_out, out, ldo, ends, sum_dt, chunks, CHUNK);
-    hipLaunchKernelGGL(scan_chunks_kernel, dim3((g.inner_p + 1023) / 1024, g.state_p, g.B), dim3(256), 0, s, g, a_log2, seqlens, state_in, ends, sum_dt, chunks);
+                       state_out, out, ldo, ends, sum_dt, chunks, len);
+    hipLaunchKernelGGL(scan_chunks_kernel, dim3((g.inner_p + 255) / 256, g.state_p, g.B), dim3(256), 0, s, g, a_log2, seqlens, state_in, ends, sum_dt, chunks);
     hipLaunchKernelGGL((scan_kernel<T, SP, SCAN_OUT>), dim3(xs, chunks, g.B), dim3(256), bytes, s, g, lg, u, dt, bc, a_log2, skip, z, ldz, seqlens, state_in, state_out,
-                       out, ldo, ends, sum_dt, chunks, CHUNK);
+                       out, ldo, ends, sum_dt, chunks, len);
     NC_CHECK_LAUNCH("scan_chunked");
     return 0;
 }
@@ -382,7 +418,7 @@ int nc_launch_scan(int dtype, const NcScanGeom& g, const void* u, const float* d
     int sp = 0, lg = 0;
     NC_CHECK_ARG(lanes_of(g.state_p, sp, lg) && g.state <= g.state_p, "scan: %d states per channel in %d", g.state, g.state_p);
     NC_CHECK_ARG(u && dt && bc && a_log2 && skip && z && out && state_in != state_out, "scan: null operand");
-    NC_CHECK_ARG(g.T <= 65535 * CHUNK && g.B <= 65535, "scan: %d tokens in one portion", g.T);
+    NC_CHECK_ARG(g.T <= 65535 * 32 && g.B <= 65535, "scan: %d tokens in one portion", g.T);
     // state in and out once; per token the projections and the result (bytes)
     NcProfScope prof(NC_CLS_SCAN, (double)g.B * (8.0 * g.state * g.inner_p + (double)g.T * g.inner_p * (4 + (dtype ? 12 : 6))), s, g.T);
 #define GO(SP)                                                                                                                                           \

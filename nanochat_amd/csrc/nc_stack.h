@@ -29,8 +29,18 @@ __device__ __forceinline__ void st4_f32(float* p, v4f v) { *(v4f*)p = v; }
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
     return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
-__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float sigmoid_f32(float z) { return __builtin_amdgcn_rcpf(1.0f + expf(-z)); }
+// max(z, 0) + log(1 + e), e = exp(-|z|).  The exponential is one exp2 with the rounding of its argument put right to first order; the logarithm
+// is 2 artanh(s), s = e / (2 + e) <= 1/3, by its series, so that a small e keeps all its digits.
+__device__ __forceinline__ float softplus_f32(float z) {
+    const float a = -fabsf(z), p = a * 1.44269504f, left = fmaf(a, 1.44269504f, -p) + a * 1.92596299e-8f;
+    const float e2 = __builtin_amdgcn_exp2f(p), e = fmaf(e2, left * 0.693147181f, e2);
+    const float s = e * __builtin_amdgcn_rcpf(2.f + e), q = s * s;
+    float t = 1.f / 17.f;
+#pragma unroll
+    for (int k = 15; k >= 1; k -= 2) t = fmaf(t, q, 1.f / (float)k);
+    return fmaf(2.f * s, t, fmaxf(z, 0.f));
+}
 __device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
 // gate and up of one unit -> its activation, both clamped: the gate from above, up on both sides
 __device__ __forceinline__ float clamped_glu_f32(float gate, float up, float limit) {

@@ -59,12 +59,12 @@ def palilix_config(width, heads, rank=512, experts=64, top=6, expert_ff=1024, vo
     head = width // heads
     moe = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "router": {"experts": experts, "top": top}, "shared": {"ff": 2 * expert_ff, "limit": 7.0}}
     if dense:
-        moe = {"kind": "dense", "ff": 4 * width}
+        moe = {"kind": "dense", "ff": 4 * width - 64}        # (off the round number: no matrix has the shape of another's by accident)
     lat = {"heads": heads, "dim": head, "rot_dim": head // 2, "vdim": head, "kv_rank": rank, "scale": (1.5 * head) ** -0.5,
            "rot": {"base": 10000.0, "dims": head // 2}}
     ret = {"heads": heads, "dim": head, "vdim": head, "decay": [1 - 2.0 ** -(5 + 6 * i / max(1, heads - 1)) for i in range(heads)],
            "rot": {"base": 10000.0, "dims": head}}
-    group = [{"type": "latent_attention", "mixer": lat, "mlp": {"kind": "dense", "ff": 4 * width}}, {"type": "retention", "mixer": ret, "mlp": moe},
+    group = [{"type": "latent_attention", "mixer": lat, "mlp": moe if dense else {"kind": "dense", "ff": 4 * width}}, {"type": "retention", "mixer": ret, "mlp": moe},
              {"type": "retention", "mixer": ret, "mlp": moe}, {"type": "latent_attention", "mixer": lat, "mlp": moe}]
     return {"architecture": "Palilix", "embedding": {"scale": 1.0}, "layers": group * groups, "logit_scale": 1.0, "logit_softcap": 30.0,
             "norm": {"eps": 1e-6}, "vocab": vocab, "width": width}

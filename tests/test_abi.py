@@ -69,7 +69,9 @@ def test_hot_kernels_use_no_scratch_memory():
            "nc_sample.hip": {"sample_kernel": 0},
            "nc_stack_gemm.hip": {"linear_few_kernel": 0, "linear_tiled_kernel": 0},
            "nc_latent_attention.hip": {"latent_mfma_kernel": 0, "latent_expanded_kernel": 0, "latent_combine_kernel": 0, "latent_append_kernel": 0},
-           "nc_stack_rows.hip": {"stack_row_add_kernel": 0, "route_sort_kernel": 0}}
+           "nc_stack_rows.hip": {"stack_row_add_kernel": 0, "route_sort_kernel": 0},
+           "nc_window_attention.hip": {"window_few_kernel": 0, "window_prefill_kernel": 0, "window_combine_kernel": 0, "window_append_kernel": 0},
+           "nc_selective_scan.hip": {"scan_kernel": 0, "scan_step_kernel": 0, "scan_chunks_kernel": 0, "scan_conv_kernel": 0}}
 
     def compile_remarks(src):
         cmd = ["hipcc", *nb.FLAGS, "-Rpass-analysis=kernel-resource-usage", "-c", os.path.join(nb.CSRC, src), "-o", os.devnull]

@@ -282,7 +282,7 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(NcScanGeom g, const fl
     float S = seqlens[b] > 0 ? state_in[((int64_t)b * (g.state_p + g.taps - 1) + n) * g.inner_p + c] : 0.f;
     float* e = ends + (int64_t)b * (chunks - 1) * plane + (int64_t)n * g.inner_p + c;
     const float* sd = sum_dt + (int64_t)b * (chunks - 1) * g.inner_p + c;
-    constexpr int AHEAD = 32;
+    constexpr int AHEAD = 16;
     for (int k0 = 0; k0 < chunks - 1; k0 += AHEAD) {
         float own[AHEAD], s[AHEAD];
 #pragma unroll

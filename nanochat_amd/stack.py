@@ -686,14 +686,14 @@ class LayerStack(nn.Module):
             d.block, d.n_mixers = BLOCKS[cfg.block], len(spec.mixers)
             assert d.n_mixers <= _lib.STACK_MAX_MIXERS
             for j, (prefix, mixer) in enumerate(spec.mixer.parts):
-                md = d.mix[j]
+                mix = d.mix[j]
                 r, c, more = mixer.pack(pick(f"l{i}.mix.{prefix}", mixer.fp32))
                 rows.append(padded(r, r.shape[0], Wp))
                 cols.append(padded(c, Wp, mixer.out))
-                md.kind, md.cols, md.out, md.out_scale, md.rot_dims = mixer.kind, mixer.cols, mixer.out, mixer.out_scale, mixer.rotation.dims
-                mixer.describe(md)
+                mix.kind, mix.cols, mix.out, mix.out_scale, mix.rot_dims = mixer.kind, mixer.cols, mixer.out, mixer.out_scale, mixer.rotation.dims
+                mixer.describe(mix)
                 for name, t in more.items():
-                    setattr(md, name, own(t, self.dtype if name in WEIGHT_FIELDS else torch.float32))
+                    setattr(mix, name, own(t, self.dtype if name in WEIGHT_FIELDS else torch.float32))
                 d.mix_cols += mixer.cols
                 d.mix_out += mixer.out
             if ff is not None:
@@ -742,8 +742,8 @@ class LayerStack(nn.Module):
             self._rope_len = round_up(positions, 1024)
             self._rope = {}
             for d, spec in zip(layers, self.config.layers):
-                for md_mix, mixer in zip(d.mix, spec.mixers):
-                    md_mix.rope = self._rope_table(mixer.rotation).data_ptr() if mixer.rotation.dims else None
+                for mix, mixer in zip(d.mix, spec.mixers):
+                    mix.rope = self._rope_table(mixer.rotation).data_ptr() if mixer.rotation.dims else None
             md.rope_len = self._rope_len
         return md
 
